@@ -8,6 +8,8 @@ from a pool of ``max_bs``.  Here
   * layers with the same needs (kv heads, head size, window) form a *group* with pages of its own
     and one block table per request;
   * a group with a window gives pages back as soon as the window has passed them;
+  * a group may keep one row for every so many tokens (``tokens_per_row``): its pages hold page_size rows
+    and it takes one only when that many tokens are complete;
   * pages are handed out per portion (``reserve``) and a request's progress is recorded after the
     step (``commit``); ``release`` gives everything back;
   * a request *slot* (0 .. max_requests-1) stands for the request's rows of fixed-size state (the step
@@ -34,10 +36,22 @@ class CacheGroupSpec:
     # what a token keeps in each layer's pools: (heads, dim, bytes per value or None = the compute dtype's)
     # per pool; None = one key row and one value row per kv head
     rows: Optional[tuple] = None
+    tokens_per_row: int = 1       # one row per this many tokens, written when the last of them is in
 
     def bytes_per_token(self, itemsize: int) -> int:
         rows = self.rows if self.rows is not None else ((self.num_kv_heads, self.head_dim, None),) * 2
-        return sum(heads * dim * (size or itemsize) for heads, dim, size in rows) * len(self.layers)
+        return -(-sum(heads * dim * (size or itemsize) for heads, dim, size in rows) * len(self.layers) // self.tokens_per_row)
+
+    def rows_for(self, tokens: int) -> int:
+        """Rows the group holds for a request of ``tokens`` tokens."""
+        return tokens // self.tokens_per_row
+
+    def pages_beside(self, token_pages: int, max_requests: int) -> int:
+        """Pages this group needs so that it never runs out before a group with a row per token and ``token_pages``
+        pages does: a request's last page may be partly filled."""
+        if self.tokens_per_row == 1:
+            return token_pages
+        return -(-token_pages // self.tokens_per_row) + max_requests
 
 
 class CacheFull(RuntimeError):
@@ -73,7 +87,7 @@ class CacheManager:
         # no page: a step gathers its rows from here instead of converting Python lists
         self._rows = [np.full((max_requests, 16), -1, dtype=np.int32) for _ in groups]
         self.requests: Dict[str, RequestCache] = {}
-        shareable = all(g.window == 0 for g in groups) and len(groups) > 0
+        shareable = all(g.window == 0 and g.tokens_per_row == 1 for g in groups) and len(groups) > 0
         self.prefix_tree: Optional[PrefixTree] = (
             PrefixTree(page_size, self.allocators) if enable_prefix_cache and shareable else None)
 
@@ -125,8 +139,11 @@ class CacheManager:
     # ------------------------------------------------------------------ pages
     def pages_needed(self, rc: RequestCache, n_new: int) -> List[int]:
         """Pages each group lacks for positions [num_computed, num_computed + n_new)."""
-        last = (rc.num_computed + n_new - 1) // self.page_size
-        return [max(0, last + 1 - len(t)) for t in rc.tables]
+        return [max(0, need - len(t)) for need, t in zip(self.pages_for(rc.num_computed + n_new), rc.tables)]
+
+    def pages_for(self, tokens: int) -> List[int]:
+        """Block table entries each group has for a request of ``tokens`` tokens."""
+        return [-(-g.rows_for(tokens) // self.page_size) for g in self.groups]
 
     def can_reserve(self, rc: RequestCache, n_new: int) -> bool:
         return all(need <= a.num_free for need, a in zip(self.pages_needed(rc, n_new), self.allocators))
@@ -163,7 +180,7 @@ class CacheManager:
             raise PageError(f"request {rc.request_id!r} was released")
         P = self.page_size
         for g in range(len(self.groups)):
-            if rc.num_computed + n_new > len(rc.tables[g]) * P:
+            if self.groups[g].rows_for(rc.num_computed + n_new) > len(rc.tables[g]) * P:
                 raise PageError(f"request {rc.request_id!r} computed past its reserved pages")
         rc.num_computed += n_new
         for g, spec in enumerate(self.groups):

@@ -795,3 +795,193 @@ def _kumudra_time_mix(m) -> KumudraTimeMix:
     if r.heads < 1 or r.dim < 1 or r.rank < 1:
         raise ConfigError("time mixing: 'heads', 'dim' and 'rank' must be positive")
     return r
+
+
+# ----------------------------------------------------------------------------------------- Nadevik
+
+@dataclass(frozen=True)
+class NadevikAttention:
+    """The attention half of a parallel mixer: convolved and normed queries and keys without positions, soft-capped
+    scores, sigmoid weights, a window beside which blocks of ``pool`` tokens are seen as one key each."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    conv: int                       # taps of the convolutions behind q, k and v
+    scale: float
+    softcap: float                  # 0: none
+    window: int                     # keys a query sees, itself included; 0: all
+    pool: int                       # tokens of a block seen beyond the window as one key; 0: none
+
+
+@dataclass(frozen=True)
+class NadevikScan:
+    """The recurrent half of a parallel mixer: a selective scan with a state per channel."""
+    inner: int
+    state: int
+    dt_rank: int
+    conv: int
+
+
+@dataclass(frozen=True)
+class NadevikParallel:
+    left: NadevikAttention
+    right: NadevikScan
+    left_scale: float
+    right_scale: float
+
+
+@dataclass(frozen=True)
+class NadevikLatentAttention:
+    """Attention over a small latent per token with a rotated key part shared by the heads; ``kv_from``: the layer
+    whose latents it reads (None: its own)."""
+    heads: int
+    dim: int                        # unrotated query / key dims per head
+    rot_dim: int
+    vdim: int
+    kv_rank: int
+    scale: float
+    window: int
+    rot_base: float
+    kv_from: Optional[int]
+
+
+@dataclass(frozen=True)
+class NadevikExperts:
+    experts: int
+    top: int
+    groups: int                     # experts form this many equal groups of neighbours
+    keep: int                       # and only the best this many are chosen from
+    ff: int
+    limit: float
+
+
+@dataclass(frozen=True)
+class NadevikLayer:
+    type: str                       # "parallel" | "latent_attention"
+    mixer: object
+    mlp: Optional[NadevikExperts]
+
+
+@dataclass(frozen=True)
+class NadevikConfig:
+    """Keys of a Nadevik config.json: layers listed one by one, each a mixer and a routed feed-forward (or none) with a
+    norm behind each, a short convolution over time ahead of the mixer (``canon``), a scaled embedding with a hashed
+    bigram table added; the head is the embedding table."""
+    architecture: str
+    vocab_size: int
+    hidden_size: int
+    layers: tuple                   # of NadevikLayer
+    norm_eps: float
+    canon_taps: int
+    embedding_scale: float
+    bigram_buckets: int             # 0: no bigram table
+    bigram_mul_prev: int
+    bigram_mul_cur: int
+
+    @classmethod
+    def from_dict(cls, d: Mapping[str, Any]) -> "NadevikConfig":
+        norm, emb, canon = d.get("norm") or {}, d.get("embedding") or {}, d.get("canon") or {}
+        bigram = emb.get("bigram") or {}
+        raw_layers = d.get("layers")
+        if not isinstance(raw_layers, (list, tuple)) or not raw_layers:
+            raise ConfigError("config.json: key 'layers' must be a non-empty list")
+        layers = []
+        for i, L in enumerate(raw_layers):
+            try:
+                if not isinstance(L, Mapping):
+                    raise ConfigError("a layer must be an object")
+                kind, m = _take(L, "type", str), L.get("mixer")
+                if not isinstance(m, Mapping):
+                    raise ConfigError("no 'mixer' object")
+                if kind == "parallel":
+                    mixer = NadevikParallel(left=_nadevik_attention(m.get("left")), right=_nadevik_scan(m.get("right")),
+                                            left_scale=_take(m, "left_scale", float, 1.0),
+                                            right_scale=_take(m, "right_scale", float, 1.0))
+                elif kind == "latent_attention":
+                    mixer = _nadevik_latent(m)
+                else:
+                    raise ConfigError(f"type {kind!r}; known: ['latent_attention', 'parallel']")
+                mlp = L.get("mlp")
+                layers.append(NadevikLayer(kind, mixer, None if mlp is None else _nadevik_experts(mlp)))
+            except ConfigError as e:
+                raise ConfigError(f"{e} (layer {i})") from None
+        for i, L in enumerate(layers):
+            if L.type != "latent_attention" or L.mixer.kv_from is None:
+                continue
+            j = L.mixer.kv_from
+            if not 0 <= j < i or layers[j].type != "latent_attention" or layers[j].mixer.kv_from is not None:
+                raise ConfigError(f"config.json: layer {i}: 'kv_from' = {j} must be an earlier latent_attention layer "
+                                  "with latents of its own")
+            a, b = L.mixer, layers[j].mixer
+            if (a.kv_rank, a.rot_dim, a.rot_base if a.rot_dim else 0) != (b.kv_rank, b.rot_dim, b.rot_base if b.rot_dim else 0):
+                raise ConfigError(f"config.json: layer {i} reads the latents of layer {j} but their 'kv_rank', "
+                                  "'rot_dim' or rotation differ")
+        cfg = cls(architecture=_take(d, "architecture", str, "Nadevik"), vocab_size=_take(d, "vocab", int),
+                  hidden_size=_take(d, "width", int), layers=tuple(layers), norm_eps=_take(norm, "eps", float),
+                  canon_taps=_take(canon, "taps", int), embedding_scale=_take(emb, "scale", float, 1.0),
+                  bigram_buckets=_take(bigram, "buckets", int, 0), bigram_mul_prev=_take(bigram, "mul_prev", int, 0),
+                  bigram_mul_cur=_take(bigram, "mul_cur", int, 0))
+        if cfg.vocab_size < 1 or cfg.hidden_size < 1 or cfg.norm_eps < 0 or cfg.canon_taps < 1 or cfg.bigram_buckets < 0:
+            raise ConfigError("config.json: 'vocab', 'width' and 'canon.taps' must be positive, 'norm.eps' and the "
+                              "bigram's 'buckets' not negative")
+        return cfg
+
+    @property
+    def num_hidden_layers(self) -> int:
+        return len(self.layers)
+
+
+def _nadevik_attention(m) -> NadevikAttention:
+    if not isinstance(m, Mapping):
+        raise ConfigError("a parallel mixer needs a 'left' object")
+    mask = m.get("mask") or {}
+    dim = _take(m, "dim", int)
+    a = NadevikAttention(heads=_take(m, "heads", int), kv_heads=_take(m, "kv_heads", int), dim=dim,
+                         vdim=_take(m, "vdim", int, dim), conv=_take(m, "conv", int), scale=_take(m, "scale", float, dim ** -0.5),
+                         softcap=_take(m, "softcap", float, 0.0), window=_take(mask, "size", int, 0),
+                         pool=_take(mask, "pool", int, 0))
+    if a.heads < 1 or a.kv_heads < 1 or a.heads % a.kv_heads or dim < 1 or a.vdim < 1:
+        raise ConfigError(f"{a.heads} heads over {a.kv_heads} kv heads of sizes {dim} and {a.vdim}")
+    if a.conv < 1 or a.softcap < 0 or a.window < 0 or a.pool < 0 or (a.pool and not a.window):
+        raise ConfigError(f"'conv' = {a.conv} must be positive, 'softcap' and 'mask' not negative, and pooled blocks need a window")
+    return a
+
+
+def _nadevik_scan(m) -> NadevikScan:
+    if not isinstance(m, Mapping):
+        raise ConfigError("a parallel mixer needs a 'right' object")
+    r = NadevikScan(inner=_take(m, "inner", int), state=_take(m, "state", int), dt_rank=_take(m, "dt_rank", int),
+                    conv=_take(m, "conv", int))
+    if min(r.inner, r.state, r.dt_rank, r.conv) < 1:
+        raise ConfigError("selective scan: 'inner', 'state', 'dt_rank' and 'conv' must be positive")
+    return r
+
+
+def _nadevik_latent(m: Mapping) -> NadevikLatentAttention:
+    rot, mask = m.get("rot") or {}, m.get("mask") or {}
+    dim, rot_dim = _take(m, "dim", int), _take(m, "rot_dim", int)
+    if _take(rot, "dims", int, rot_dim) != rot_dim:
+        raise ConfigError(f"'rot.dims' = {rot['dims']} differs from 'rot_dim' = {rot_dim}: the rotated part is rotated whole")
+    a = NadevikLatentAttention(
+        heads=_take(m, "heads", int), dim=dim, rot_dim=rot_dim, vdim=_take(m, "vdim", int, dim), kv_rank=_take(m, "kv_rank", int),
+        scale=_take(m, "scale", float, (dim + rot_dim) ** -0.5), window=_take(mask, "size", int, 0),
+        rot_base=_take(rot, "base", float, 10000.0), kv_from=_take(m, "kv_from", int, None))
+    if a.heads < 1 or dim < 1 or rot_dim < 0 or rot_dim % 2 or a.vdim < 1 or a.kv_rank < 1 or a.window < 0 or a.rot_base <= 0:
+        raise ConfigError("latent attention sizes must be positive, 'rot_dim' even and 'mask.size' not negative")
+    return a
+
+
+def _nadevik_experts(f) -> NadevikExperts:
+    if not isinstance(f, Mapping) or _take(f, "kind", str) != "moe":
+        raise ConfigError("'mlp' must be null or an object of kind 'moe'")
+    router, expert = f.get("router") or {}, f.get("expert") or {}
+    groups = router.get("groups") or {}
+    count = _take(groups, "count", int, 1)
+    e = NadevikExperts(experts=_take(router, "experts", int), top=_take(router, "top", int), groups=count,
+                       keep=_take(groups, "keep", int, count), ff=_take(expert, "ff", int), limit=_take(expert, "limit", float))
+    if e.experts < 1 or e.groups < 1 or e.experts % e.groups or not 1 <= e.keep <= e.groups:
+        raise ConfigError(f"{e.experts} experts in {e.groups} equal groups of which {e.keep} are kept")
+    if not 1 <= e.top <= e.experts // e.groups * e.keep or e.ff < 1 or not e.limit > 0:
+        raise ConfigError(f"top = {e.top} of {e.experts // e.groups * e.keep} experts in the kept groups; sizes and 'limit' must be positive")
+    return e

@@ -32,12 +32,14 @@ def pages_from_memory(model, env, page_size: int, utilization: float, context_le
     free, _ = torch.cuda.mem_get_info(env.device)
     itemsize = torch.empty((), dtype=env.dtype).element_size()
     per_token = sum(g.bytes_per_token(itemsize) for g in groups)
-    tokens = int(free * utilization) // max(1, per_token)
+    # a group with a row for many tokens holds up to a page more per request
+    spare = sum(max_bs * page_size * g.tokens_per_row * g.bytes_per_token(itemsize) for g in groups if g.tokens_per_row > 1)
+    tokens = (int(free * utilization) - spare) // max(1, per_token)
     cap = max_bs * (-(-context_len // page_size))
     pages = min(tokens // page_size, cap)
     if pages < 1:
         raise RuntimeError("no device memory left for the cache after loading the model")
-    return [pages] * len(groups)
+    return [g.pages_beside(pages, max_bs) for g in groups]
 
 
 @dataclass
@@ -64,7 +66,7 @@ class Engine:
         self.model_config, self.model, self.env = model_config, model, env
         if config.num_pages is not None:
             groups, _, _ = model.cache_layout()
-            num_pages = [config.num_pages] * len(groups)
+            num_pages = [g.pages_beside(config.num_pages, config.max_bs) for g in groups]
         else:
             num_pages = pages_from_memory(model, env, config.page_size, config.gpu_memory_utilization,
                                           config.context_len, config.max_bs)

@@ -59,10 +59,11 @@ class ModelRunner:
         self.max_requests = max_requests
         groups, cache_group, states = model.cache_layout()
         if isinstance(num_pages, int):
-            num_pages = [num_pages] * len(groups)
+            num_pages = [g.pages_beside(num_pages, max_requests) for g in groups]
         self.cache = CacheManager(groups, list(num_pages), page_size, max_requests,
                                   enable_prefix_cache=enable_prefix_cache and not states)
         self.max_table = -(-env.context_len // page_size)
+        self.max_tables = [max(1, n) for n in self.cache.pages_for(env.context_len)]      # per cache group
         views: Dict[tuple, LayerCache] = {}      # (cache id, index of the need in its block) -> view
         for g, (spec, need) in enumerate(zip(groups, model.group_needs())):
             for key in spec.layers:
@@ -87,8 +88,11 @@ class ModelRunner:
                     raise StepError(f"two parts name different step planners {name!r}")
         # per cache id what its block sees: the one view, or one view per declared need
         self.caches: Dict[int, LayerCache] = {}
-        for cache_id in sorted({c for c, _ in views}):
-            self.caches[cache_id] = LayerCache.of_parts([views[(cache_id, i)] for i in range(model.num_needs(cache_id))])
+        seen = dict(views)
+        for key, source in model.borrowed_caches().items():
+            seen[key] = views[source].reader()
+        for cache_id in sorted({c for c, _ in seen}):
+            self.caches[cache_id] = LayerCache.of_parts([seen[(cache_id, i)] for i in range(model.num_needs(cache_id))])
         self._upload = StagedUpload(env.device)
         # int32 device tensor the steps take late token ids from (the sampler's output of the step before), or None
         self.feed_source: Optional[torch.Tensor] = None
@@ -114,7 +118,7 @@ class ModelRunner:
                     total += t.numel() * t.element_size()
         return total
 
-    def _pack(self, entries: Sequence[StepEntry], pad_entries: int = 0, table_stride: Optional[int] = None,
+    def _pack(self, entries: Sequence[StepEntry], pad_entries: int = 0, table_strides: Optional[Sequence[int]] = None,
               allow_unknown: bool = False, kv_bucket: Optional[int] = None):
         """Flatten the entries into one int32 host array.  Returns (host array, layout, facts); the layout
         maps a field's name to its (first, end) in the array.
@@ -136,10 +140,10 @@ class ModelRunner:
         strides = []
         for g in range(len(groups)):
             widest = max(1, max(len(e.cache.tables[g]) for e in entries))
-            if table_stride is not None:
-                if widest > table_stride:
+            if table_strides is not None:
+                if widest > table_strides[g]:
                     raise StepError("a block table is wider than the captured graph's")
-                widest = table_stride
+                widest = table_strides[g]
             strides.append(widest)
         caches = [e.cache for e in entries]
         starts = [rc.num_computed for rc in caches]
@@ -151,8 +155,8 @@ class ModelRunner:
                 raise StepError(f"request {rc.request_id!r} was released")
             if s0 + n > self.env.context_len:
                 raise StepError(f"request {rc.request_id!r}: {s0 + n} tokens exceed context_len={self.env.context_len}")
-            for tab in rc.tables:
-                if len(tab) * P < s0 + n:
+            for spec, tab in zip(groups, rc.tables):
+                if len(tab) * P < spec.rows_for(s0 + n):
                     raise StepError(f"request {rc.request_id!r}: no pages reserved for positions up to {s0 + n - 1}")
         if len(set(slots)) != n_real:
             seen = set()
@@ -291,7 +295,7 @@ class ModelRunner:
             while kv_bucket < longest:
                 kv_bucket *= 2
             kv_bucket = min(kv_bucket, self.max_table * self.page_size)
-            host, layout, facts = self._pack(entries, pad_entries=b_pad, table_stride=self.max_table,
+            host, layout, facts = self._pack(entries, pad_entries=b_pad, table_strides=self.max_tables,
                                              allow_unknown=allow_unknown, kv_bucket=kv_bucket)
             return PreparedStep(entries, host, layout, facts, (b_pad, kv_bucket))
         host, layout, facts = self._pack(entries, allow_unknown=allow_unknown)

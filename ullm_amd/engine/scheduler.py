@@ -39,12 +39,10 @@ class Scheduler:
     def add(self, req: Request) -> None:
         if req.request_id in self.requests:
             raise ValueError(f"request id {req.request_id!r} is already in use")
-        P = self.cache.page_size
-        need = -(-(req.num_tokens) // P)
-        smallest = min(a.num_pages for a in self.cache.allocators) if self.cache.allocators else need
-        if need > smallest:
-            raise ValueError(f"request {req.request_id!r}: a prompt of {req.num_tokens} tokens needs {need} "
-                             f"pages but the cache has {smallest}")
+        for need, pool in zip(self.cache.pages_for(req.num_tokens), self.cache.allocators):
+            if need > pool.num_pages:
+                raise ValueError(f"request {req.request_id!r}: a prompt of {req.num_tokens} tokens needs {need} "
+                                 f"pages but the cache has {pool.num_pages}")
         req.status = RequestStatus.WAITING
         self.waiting.append(req)
         self.requests[req.request_id] = req

@@ -405,6 +405,35 @@ def add_norm_general(branch: Optional[torch.Tensor], residual: torch.Tensor, gai
     return out
 
 
+def post_add(branch: torch.Tensor, residual: torch.Tensor, gain: torch.Tensor, eps: float, out_dtype: Optional[torch.dtype],
+             second: Optional[torch.Tensor] = None, a: float = 1.0, b: float = 1.0, conv=None) -> Optional[torch.Tensor]:
+    """residual (float32 [T, H], in place) += the RMS norm of a * branch (+ b * second) times ``gain``; returns the new rows in
+    ``out_dtype`` (None: nothing).  Each branch is [T, H] or a stack of partial sums [S, T, H].  ``conv`` = (weights float32
+    [taps, H], state rows float32 [slots, >= (taps-1) * H], slots int32 [T]), for steps of single tokens: what is returned is
+    the row plus the causal convolution over it and the rows before it in its state row, which moves on."""
+    T, H = residual.shape
+    _need(residual.dtype == torch.float32 and residual.is_contiguous(), "residual must be contiguous float32")
+    _need(gain.dtype == torch.float32 and gain.numel() == H and gain.is_contiguous(), "gain must be float32 [H]")
+    for y in (branch, second):
+        _need(y is None or (y.is_contiguous() and y.dim() in (2, 3) and tuple(y.shape[-2:]) == (T, H)),
+              "a branch must be contiguous [T, H] or [S, T, H]")
+    out = torch.empty((T, H), dtype=out_dtype, device=residual.device) if out_dtype is not None else None
+    w = rows = slots = None
+    if conv is not None:
+        w, rows, slots = conv
+        _need(out is not None and w.dtype == torch.float32 and w.dim() == 2 and w.shape[1] == H and w.is_contiguous()
+              and 1 <= w.shape[0] <= SHORT_CONV_MAX_TAPS, "conv weights must be float32 [taps, H]")
+        _check_step_state(rows, 0, (w.shape[0] - 1) * H, "the convolution's state")
+        _i32(slots, "slots", T)
+    n = lambda y: 0 if y is None else (y.shape[0] if y.dim() == 3 else 1)      # noqa: E731
+    _check(build.load("postnorm").ullm_post_add(
+        _p(branch), _c_int(n(branch)), _c_int(_dt(branch)), _p(second), _c_int(n(second)),
+        _c_int(_dt(second) if second is not None else F32), _c_float(a), _c_float(b), _p(gain), _c_float(eps), _p(residual), _p(out),
+        _c_int(_dt(out) if out is not None else F32), _c_int(T), _c_int(H), _p(w), _c_int(w.shape[0] if w is not None else 0), _p(rows),
+        ctypes.c_longlong(rows.stride(0) if rows is not None else 0), _p(slots), _stream()), "post_add")
+    return out
+
+
 def qk_whole_norm_write(proj: torch.Tensor, q_off: int, k_off: int, v_off: int, q_out: torch.Tensor,
                         q_gain: Optional[torch.Tensor], k_gain: Optional[torch.Tensor], eps: float, q_count: int,
                         k_count: int, positions: torch.Tensor, token_entry: torch.Tensor, block_table: torch.Tensor,
@@ -1294,20 +1323,195 @@ def paged_attention(q: torch.Tensor, k_pool: torch.Tensor, v_pool: torch.Tensor,
     return out
 
 
+# ---------------------------------------------------------------------------------- short convolutions, a scan per channel
+
+SHORT_CONV_MAX_TAPS = 16
+CONV_SILU, CONV_RESIDUAL = 0, 1          # what short_conv stores: silu(bias + conv), or its input + conv
+
+
+def _check_step_state(state: torch.Tensor, off: int, n: int, name: str) -> None:
+    _need(state.dtype == torch.float32 and state.dim() == 2 and state.stride(1) == 1 and off >= 0 and off + n <= state.shape[1],
+          f"{name} must be float32 [slots, row] holding {n} values from {off} on")
+
+
+def short_conv(x: torch.Tensor, weight: torch.Tensor, bias: Optional[torch.Tensor], state: torch.Tensor, state_off: int, ctx,
+               mode: int, out_dtype: torch.dtype, write_state: bool = True) -> torch.Tensor:
+    """A causal convolution over time per channel of ``x`` ([T, channels], may be columns of wider rows), 32-bit sums:
+    ``weight`` float32 [taps, channels] (the last row is the current token's), ``bias`` float32 [channels].  The inputs of
+    the taps-1 tokens before an entry's first lie in its state row (``state[slot, state_off ..]``, float32, oldest first)
+    and are replaced by those of its last tokens.  CONV_SILU: silu(bias + conv); CONV_RESIDUAL: x + conv."""
+    T, channels = x.shape
+    taps = weight.shape[0]
+    _need(x.stride(1) == 1, "x must have unit stride along its rows")
+    _need(weight.dtype == torch.float32 and weight.shape == (taps, channels) and weight.is_contiguous(), "weight must be float32 [taps, channels]")
+    _need(1 <= taps <= SHORT_CONV_MAX_TAPS, f"a convolution of {taps} taps: at most {SHORT_CONV_MAX_TAPS}")
+    if bias is not None:
+        _need(bias.dtype == torch.float32 and bias.numel() == channels and bias.is_contiguous(), "bias must be float32 [channels]")
+    _check_step_state(state, state_off, (taps - 1) * channels, "the convolution's state")
+    out = torch.empty((T, channels), dtype=out_dtype, device=x.device)
+    _check(build.load("short_conv").ullm_short_conv(
+        _p(x), _c_int(x.stride(0)), _p(weight), _p(bias), _p(state[:, state_off:]), ctypes.c_longlong(state.stride(0)),
+        _p(ctx.token_entry), _p(ctx.q_start), _p(ctx.entry_slot), _p(out), _c_int(T), _c_int(ctx.num_entries), _c_int(channels),
+        _c_int(taps), _c_int(mode), _c_int(1 if ctx.decode_only else 0), _c_int(1 if write_state else 0), _c_int(_dt(x)),
+        _c_int(_dt(out)), _stream()), "short_conv")
+    return out
+
+
+SELECTIVE_SCAN_MAX_STATE = 256
+
+
+def selective_scan(x: torch.Tensor, raw_dt: torch.Tensor, bc: torch.Tensor, z: torch.Tensor, a_log2: torch.Tensor,
+                   dt_bias: torch.Tensor, d_skip: torch.Tensor, state: torch.Tensor, state_off: int, ctx,
+                   write_state: bool = True) -> torch.Tensor:
+    """Per channel c and state n over each entry's tokens: dt = softplus(raw_dt + dt_bias), S = exp(dt A) S + dt x B,
+    y = sum_n S C + d_skip x; returns y * silu(z) ([T, inner] of x's dtype).  ``raw_dt`` float32 [T, inner], ``bc`` float32
+    [T, >= 2 n] (B, then C), ``a_log2`` float32 [inner, n] = A log2(e); ``x`` and ``z`` may be columns of wider rows.  The
+    states are float32 at ``state[slot, state_off + c * n ..]``."""
+    T, inner = x.shape
+    n = a_log2.shape[1]
+    _need(x.stride(1) == 1 and z.shape == (T, inner) and z.stride(1) == 1 and z.dtype == x.dtype, "x and z must be [T, inner] of one dtype")
+    _f32_rows(raw_dt, "raw_dt", T, inner)
+    _f32_rows(bc, "bc", T, 2 * n)
+    _need(a_log2.dtype == torch.float32 and a_log2.shape == (inner, n) and a_log2.is_contiguous() and n <= SELECTIVE_SCAN_MAX_STATE,
+          f"A must be float32 [inner, n <= {SELECTIVE_SCAN_MAX_STATE}]")
+    for v, nm in ((dt_bias, "dt_bias"), (d_skip, "d_skip")):
+        _need(v.dtype == torch.float32 and v.numel() == inner and v.is_contiguous(), f"{nm} must be float32 [inner]")
+    _check_step_state(state, state_off, inner * n, "the scan's state")
+    out = torch.empty((T, inner), dtype=x.dtype, device=x.device)
+    ll = ctypes.c_longlong
+    _check(build.load("selective_scan").ullm_selective_scan(
+        _p(x), _c_int(x.stride(0)), _p(raw_dt), _c_int(raw_dt.stride(0)), _p(bc), _c_int(bc.stride(0)), _p(z), _c_int(z.stride(0)),
+        _p(a_log2), _p(dt_bias), _p(d_skip), _p(state), ll(state.stride(0)), ll(state_off), _p(ctx.q_start), _p(ctx.entry_slot),
+        _p(out), _c_int(ctx.num_entries), _c_int(inner), _c_int(n), _c_int(1 if write_state else 0), _c_int(_dt(x)), _stream()),
+        "selective_scan")
+    return out
+
+
+# ---------------------------------------------------------------------------------- a window and pooled blocks
+
+def conv_norm_write(proj: torch.Tensor, weight: torch.Tensor, state: torch.Tensor, state_off: int, q_gain: torch.Tensor,
+                    k_gain: torch.Tensor, eps: float, q_count: int, k_count: int, ctx, group, k_pool, v_pool, nq: int, nkv: int,
+                    hd: int, pool: int = 0, pooled_group=None, pk_pool=None, pv_pool=None) -> torch.Tensor:
+    """``proj`` [T, q | k | v] through a causal convolution per channel (``weight`` float32 [taps, columns], the inputs of
+    the tokens before in the state row), q and k over the root mean square of all their values of a token (sums of
+    squares / ``q_count``, ``k_count``) times a gain per value.  Returns q [T, nq * hd]; k and v go to the paged pools.  In a
+    step of single tokens a token that completes a block of ``pool`` tokens also leaves the block's mean key and value in
+    the pooled pools; in other steps :func:`block_means` does that."""
+    T = proj.shape[0]
+    cols, taps = (nq + 2 * nkv) * hd, weight.shape[0]
+    _need(proj.dim() == 2 and proj.shape[1] == cols and proj.stride(1) == 1, "proj must be [T, (nq + 2 nkv) * hd]")
+    _need(weight.dtype == torch.float32 and weight.shape == (taps, cols) and weight.is_contiguous() and 1 <= taps <= SHORT_CONV_MAX_TAPS,
+          "weight must be float32 [taps, (nq + 2 nkv) * hd]")
+    _need(q_gain.dtype == torch.float32 and q_gain.numel() == nq * hd and q_gain.is_contiguous()
+          and k_gain.dtype == torch.float32 and k_gain.numel() == nkv * hd and k_gain.is_contiguous(), "gains must be float32 [nq*hd] and [nkv*hd]")
+    _check_step_state(state, state_off, (taps - 1) * cols, "the convolution's state")
+    _check_pools(k_pool, v_pool, nkv, group.page_size, hd, proj.dtype)
+    if pool:
+        _check_pools(pk_pool, pv_pool, nkv, group.page_size, hd, proj.dtype)
+    q = torch.empty((T, nq * hd), dtype=proj.dtype, device=proj.device)
+    _check(build.load("pooled").ullm_conv_norm_write(
+        _p(proj), _c_int(proj.stride(0)), _p(weight), _c_int(taps), _p(state[:, state_off:]), ctypes.c_longlong(state.stride(0)),
+        _p(q_gain), _p(k_gain), _c_float(eps), _c_float(float(q_count)), _c_float(float(k_count)), _p(ctx.positions),
+        _p(ctx.token_entry), _p(ctx.q_start), _p(ctx.entry_slot), _p(group.block_table), _c_int(group.block_table.stride(0)), _p(q),
+        _p(k_pool), _p(v_pool), _c_int(group.page_size), _c_int(nq), _c_int(nkv), _c_int(hd), _c_int(T), _c_int(ctx.num_entries),
+        _c_int(1 if ctx.decode_only else 0), _c_int(pool), _p(pooled_group.block_table if pool else None),
+        _c_int(pooled_group.block_table.stride(0) if pool else 0), _p(pk_pool if pool else None), _p(pv_pool if pool else None),
+        _c_int(_dt(proj)), _stream()), "conv_norm_write")
+    return q
+
+
+def block_means(blocks: torch.Tensor, n_blocks: int, group, pooled_group, k_pool, v_pool, pk_pool, pv_pool, pool: int, nkv: int,
+                hd: int) -> None:
+    """For every pair (entry, block) of ``blocks`` (int32 [n, 2] flat): row ``block`` of the entry's pooled pools becomes the mean
+    of the keys and of the values of its tokens block * pool .. + pool - 1, as the pools hold them."""
+    _i32(blocks, "blocks", 2 * n_blocks)
+    _check_pools(k_pool, v_pool, nkv, group.page_size, hd, k_pool.dtype)
+    _check_pools(pk_pool, pv_pool, nkv, group.page_size, hd, k_pool.dtype)
+    _check(build.load("pooled").ullm_block_means(
+        _p(blocks), _c_int(n_blocks), _p(group.block_table), _c_int(group.block_table.stride(0)), _p(pooled_group.block_table),
+        _c_int(pooled_group.block_table.stride(0)), _p(k_pool), _p(v_pool), _p(pk_pool), _p(pv_pool), _c_int(pool),
+        _c_int(group.page_size), _c_int(nkv), _c_int(hd), _c_int(_dt(k_pool)), _stream()), "block_means")
+
+
+def pooled_mfma_supports(dtype: torch.dtype, hd: int, page_size: int, nq: int, nkv: int) -> bool:
+    return dtype == torch.bfloat16 and bool(build.load("attention_pooled").ullm_pooled_mfma_supports(
+        _c_int(hd), _c_int(page_size), _c_int(nq), _c_int(nkv)))
+
+
+def pooled_decode_split(n_items: int, nkv: int, groups: int, keys: int, units: int = 256):
+    """(waves, splits) of the decode launch: few (token, kv head) pairs are cut over several blocks, and these over four
+    waves, until the launch has about a wave per SIMD; every wave keeps at least two 32-key tiles where it can."""
+    pairs, tiles = max(1, n_items * nkv * groups), max(1, -(-keys // 32))
+    want = max(1, 4 * units // pairs)                     # waves a pair may have
+    shares = max(1, min(want, tiles // 2))
+    if shares <= 4:
+        return (4 if shares >= 3 else 1), 1
+    return 4, min(16, -(-shares // 4))
+
+
+def pooled_attention(q: torch.Tensor, k_pool, v_pool, ctx, group, nq: int, nkv: int, hd: int, scale: float, window: int,
+                     plan, softcap: float = 0.0, head_bias: Optional[torch.Tensor] = None, pool: int = 0, pooled_group=None,
+                     pk_pool=None, pv_pool=None, softmax: bool = False, splits: int = 0, waves: int = 0) -> torch.Tensor:
+    """Attention of the batch's queries [T, nq * hd] over the last ``window`` tokens (0: all) and, with ``pool``, one key and
+    value for every block of ``pool`` tokens wholly before the window (pools of one row per block).  Scores q . k * scale,
+    ``softcap`` * tanh(. / softcap) if > 0, + ``head_bias`` (float32 [nq]).  The weights are the sigmoids of the scores, not
+    normalised, or with ``softmax`` the softmax over all visible keys.  bfloat16 shapes with sigmoid weights that the
+    matrix-core kernels take go there, everything else to the general kernel; every choice computes the same function."""
+    T = q.shape[0]
+    _need(q.dim() == 2 and q.shape[1] == nq * hd and q.stride(1) == 1, "q must be [T, nq * hd]")
+    _check_pools(k_pool, v_pool, nkv, group.page_size, hd, q.dtype)
+    _need(pool >= 0 and (pool == 0 or window > 0), "pooled blocks need a window")
+    if pool:
+        _check_pools(pk_pool, pv_pool, nkv, group.page_size, hd, q.dtype)
+    if head_bias is not None:
+        _need(head_bias.dtype == torch.float32 and head_bias.numel() == nq and head_bias.is_contiguous(), "head_bias must be float32 [nq]")
+    out = torch.empty((T, nq * hd), dtype=q.dtype, device=q.device)
+    tables = (_p(k_pool), _p(v_pool), _p(group.block_table), _c_int(group.block_table.stride(0)), _p(pk_pool if pool else None),
+              _p(pv_pool if pool else None), _p(pooled_group.block_table if pool else None),
+              _c_int(pooled_group.block_table.stride(0) if pool else 0))
+    if softmax or not pooled_mfma_supports(q.dtype, hd, group.page_size, nq, nkv):
+        if q.dtype == torch.bfloat16 and not softmax:
+            _warn_general_attention(hd, group.page_size)
+        _check(build.load("pooled").ullm_pooled_attention_general(
+            _p(q), _c_int(q.stride(0)), _p(out), *tables, _p(ctx.positions), _p(ctx.token_entry), _c_int(group.page_size), _c_int(T),
+            _c_int(nq), _c_int(nkv), _c_int(hd), _c_float(scale), _c_float(softcap), _p(head_bias), _c_int(window), _c_int(pool),
+            _c_int(1 if softmax else 0), _c_int(_dt(q)), _stream()), "pooled_attention_general")
+        return out
+    lib, n = build.load("attention_pooled"), plan.facts
+    if n["num_decode"]:
+        kv = n["max_decode_kv"]
+        keys = kv if window <= 0 or kv <= window else window + 31 + ((kv - window) // pool if pool else 0)
+        auto = pooled_decode_split(n["num_decode"], nkv, -(-(nq // nkv) // 16), keys, compute_units(q.device))
+        w, s = waves or auto[0], splits or auto[1]
+        part = torch.empty(n["num_decode"] * nq * s * hd, dtype=torch.float32, device=q.device) if s > 1 else None
+        _check(lib.ullm_pooled_decode(
+            _p(q), _c_int(q.stride(0)), _p(out), *tables, _p(plan.arrays["decode_tokens"]), _c_int(n["num_decode"]), _p(ctx.positions),
+            _p(ctx.token_entry), _c_int(group.page_size), _c_int(nq), _c_int(nkv), _c_int(hd), _c_float(scale), _c_float(softcap),
+            _p(head_bias), _c_int(window), _c_int(pool), _c_int(s), _c_int(w), _p(part), _stream()), "pooled_decode")
+    if n["num_tiles"]:
+        _check(lib.ullm_pooled_prefill(
+            _p(q), _c_int(q.stride(0)), _p(out), *tables, _p(plan.arrays["tiles"]), _c_int(n["num_tiles"]), _p(ctx.positions),
+            _p(ctx.token_entry), _c_int(group.page_size), _c_int(nq), _c_int(nkv), _c_int(hd), _c_float(scale), _c_float(softcap),
+            _p(head_bias), _c_int(window), _c_int(pool), _stream()), "pooled_prefill")
+    return out
+
+
 # ---------------------------------------------------------------------------------- latent attention
 
 def latent_prepare(proj: torch.Tensor, q_off: int, q_rank: int, kv_off: int, kv_rank: int, kr_off: int, rot: int,
                    g_off: int, n_gate: int, q_gain: Optional[torch.Tensor], kv_gain: torch.Tensor, eps: float,
                    cos_sin: Optional[torch.Tensor], positions: torch.Tensor, token_entry: torch.Tensor,
                    block_table: torch.Tensor, k_pool: torch.Tensor, v_pool: torch.Tensor, page_size: int, hd: int,
-                   write_kv: bool, dtype: torch.dtype):
-    """What a latent-attention layer does with its first product ``proj`` (float32 [T, columns]: q latent at ``q_off``,
+                   write_kv: bool, dtype: torch.dtype, style: int = 1):
+    """What a latent-attention layer does with its first product ``proj`` ([T, columns], float32 or ``dtype``: q latent at ``q_off``,
     kv latent at ``kv_off``, the rotated key part at ``kr_off``, gate logits at ``g_off``): returns (cq, gate) with
     cq = rmsnorm(q latent) * ``q_gain`` as [T, q_rank] and gate = the logits as [T, n_gate rounded up to 8], both of
     ``dtype``; with ``write_kv`` the token's cache row [rmsnorm(kv latent) * ``kv_gain`` | rotated key part] goes to
-    ``k_pool`` ([pages, 1, page_size, hd]) and the normed latent to ``v_pool`` ([pages, 1, hd, page_size])."""
+    ``k_pool`` ([pages, 1, page_size, hd]) and the normed latent to ``v_pool`` ([pages, 1, hd, page_size]).
+    ``style``: how the rotated dims are paired (1: half-split, 2: adjacent)."""
     T = proj.shape[0]
-    _need(proj.dtype == torch.float32 and proj.dim() == 2 and proj.stride(1) == 1, "proj must be float32 [T, columns]")
+    _need(proj.dtype in (torch.float32, dtype) and proj.dim() == 2 and proj.stride(1) == 1,
+          "proj must be float32 or the compute dtype, [T, columns]")
     _i32(positions, "positions", T)
     _i32(token_entry, "token_entry", T)
     _need(block_table.dtype == torch.int32 and block_table.dim() == 2 and block_table.stride(1) == 1,
@@ -1326,8 +1530,9 @@ def latent_prepare(proj: torch.Tensor, q_off: int, q_rank: int, kv_off: int, kv_
     ldg = -(-n_gate // 8) * 8
     gate = torch.empty((T, ldg), dtype=dtype, device=proj.device) if n_gate else None    # the kernel writes all ldg columns
     _check(build.load("latent").ullm_latent_prepare(
-        _p(proj), _c_int(proj.stride(0)), _c_int(q_off), _c_int(q_rank), _c_int(kv_off), _c_int(kv_rank), _c_int(kr_off),
-        _c_int(rot), _c_int(g_off), _c_int(n_gate), _p(q_gain), _p(kv_gain), _c_float(eps), _p(cos_sin), _c_int(table_rows),
+        _p(proj), _c_int(_dt(proj)), _c_int(proj.stride(0)), _c_int(q_off), _c_int(q_rank), _c_int(kv_off), _c_int(kv_rank),
+        _c_int(kr_off), _c_int(rot), _c_int(g_off), _c_int(n_gate), _p(q_gain), _p(kv_gain), _c_float(eps), _p(cos_sin),
+        _c_int(table_rows), _c_int(1 if style == 2 else 0),
         _p(positions), _p(token_entry), _p(block_table), _c_int(block_table.stride(0)), _p(k_pool), _p(v_pool),
         _c_int(page_size), _c_int(hd), _c_int(1 if write_kv else 0), _p(cq), _p(gate), _c_int(ldg), _c_int(T),
         _c_int(F32 if dtype == torch.float32 else BF16), _stream()), "latent_prepare")
@@ -1338,11 +1543,13 @@ HEAD_LINEAR_MAX_K = 1024          # the widest rows the per-head kernel keeps in
 HEAD_LINEAR_LIBRARY_FROM = 128    # from this many rows on a bfloat16 product per head is the library's batched product
 
 
-def head_linear(x: torch.Tensor, w: torch.Tensor, out: Optional[torch.Tensor] = None) -> torch.Tensor:
+def head_linear(x: torch.Tensor, w: torch.Tensor, out: Optional[torch.Tensor] = None,
+                gate: Optional[torch.Tensor] = None) -> torch.Tensor:
     """y[t, h] = w[h]^T x[t, h] for x [T, heads, K] (unit stride along K, any strides otherwise), w contiguous
     [heads, K, N] of x's dtype; y [T, heads, N] (``out`` may be a strided view with unit stride along N; without
     ``out`` the result may be one).  Few rows, and float32 always, take the hand-written kernel (32-bit sums in an
-    order that depends on the row alone); many bfloat16 rows the library's batched product."""
+    order that depends on the row alone); many bfloat16 rows the library's batched product.  ``gate`` ([T, heads * N], may be
+    columns of wider rows; with a contiguous ``out`` only): the result is multiplied by its sigmoid."""
     T, heads, K = x.shape
     _need(w.dim() == 3 and w.shape[0] == heads and w.shape[1] == K and w.is_contiguous() and w.dtype == x.dtype
           and w.data_ptr() % 8 == 0, "w must be contiguous [heads, K, N] of x's dtype")
@@ -1350,10 +1557,19 @@ def head_linear(x: torch.Tensor, w: torch.Tensor, out: Optional[torch.Tensor] = 
     N = w.shape[2]
     if out is not None:
         _need(out.shape == (T, heads, N) and out.stride(2) == 1 and out.dtype == x.dtype, "bad head_linear output")
+    if gate is not None:
+        _need(out is not None and out.is_contiguous() and gate.dtype == x.dtype and gate.dim() == 2
+              and gate.shape == (T, heads * N) and gate.stride(1) == 1, "a gate per value must be [T, heads * N] of x's dtype")
     if x.dtype == torch.bfloat16 and T >= HEAD_LINEAR_LIBRARY_FROM and x.is_cuda:
         y = torch.bmm(x.transpose(0, 1), w).transpose(0, 1)          # [heads, T, N] seen as [T, heads, N]
         if out is None:
             return y
+        if gate is not None:
+            ll = ctypes.c_longlong
+            _check(build.load("latent").ullm_value_gate(_p(y), ll(y.stride(0)), ll(y.stride(1)), _p(gate), ll(gate.stride(0)),
+                                                        _p(out), _c_int(T), _c_int(heads), _c_int(N), _c_int(_dt(x)), _stream()),
+                   "value_gate")
+            return out
         out.copy_(y)
         return out
     _need(K <= HEAD_LINEAR_MAX_K, f"head_linear takes rows of up to {HEAD_LINEAR_MAX_K} values")
@@ -1361,13 +1577,14 @@ def head_linear(x: torch.Tensor, w: torch.Tensor, out: Optional[torch.Tensor] = 
         out = torch.empty((T, heads, N), dtype=x.dtype, device=x.device)
     ll = ctypes.c_longlong
     _check(build.load("latent").ullm_head_linear(_p(x), ll(x.stride(0)), ll(x.stride(1)), _p(w), _p(out), ll(out.stride(0)),
-                                                 ll(out.stride(1)), _c_int(T), _c_int(heads), _c_int(N), _c_int(K),
-                                                 _c_int(_dt(x)), _stream()), "head_linear")
+                                                 ll(out.stride(1)), _p(gate), ll(gate.stride(0) if gate is not None else 0),
+                                                 _c_int(T), _c_int(heads), _c_int(N), _c_int(K), _c_int(_dt(x)), _stream()),
+           "head_linear")
     return out
 
 
 def latent_query(qa: torch.Tensor, q: torch.Tensor, plain: int, rot: int, hd: int, cos_sin: Optional[torch.Tensor],
-                 positions: torch.Tensor) -> torch.Tensor:
+                 positions: torch.Tensor, style: int = 1) -> torch.Tensor:
     """The query rows [T, heads * hd] a latent-attention layer hands the attention kernels: per head
     [qa[t, h] (rank values) | the head's last ``rot`` dims of ``q`` turned by the token's position | zeros], for
     qa [T, heads, rank] (unit stride along rank) and q [T, heads * (plain + rot)]."""
@@ -1384,7 +1601,7 @@ def latent_query(qa: torch.Tensor, q: torch.Tensor, plain: int, rot: int, hd: in
     ll = ctypes.c_longlong
     _check(build.load("latent").ullm_latent_query(_p(qa), ll(qa.stride(0)), ll(qa.stride(1)), _p(q), _c_int(q.stride(0)),
                                                   _c_int(plain), _c_int(rot), _c_int(rank), _c_int(heads), _c_int(hd),
-                                                  _p(cos_sin), _c_int(table_rows), _p(positions), _p(out),
+                                                  _p(cos_sin), _c_int(table_rows), _c_int(1 if style == 2 else 0), _p(positions), _p(out),
                                                   _c_int(out.stride(0)), _c_int(T), _c_int(_dt(qa)), _stream()),
            "latent_query")
     return out
@@ -1399,14 +1616,19 @@ MOE_TILE_ROWS = (16, 32, 64, 128)     # grouped rows a block of the matrix-core 
 ROUTE_SOFTMAX_ALL, ROUTE_TOP_LOGITS, ROUTE_SIGMOID = 0, 1, 2      # how a router turns logits into experts and weights
 
 
+MOE_MAX_GROUPS = 64               # groups a router may choose from before it chooses experts
+
+
 def moe_route(logits: torch.Tensor, correction: Optional[torch.Tensor], top: int, mode: int = ROUTE_SOFTMAX_ALL,
-              weight_scale: float = 1.0):
+              weight_scale: float = 1.0, groups: int = 1, keep: int = 1, raw: bool = False):
     """(ids int32 [T, top], weights float32 [T, top]) from router logits float32 [T, R]: the softmax over all R, the
     ``top`` largest of softmax + ``correction`` (float32 [R] or None; ties go to the lower index), and as weights the
     chosen outputs' softmax values over their sum (+ 1e-20).  With ``mode`` ROUTE_TOP_LOGITS: the ``top`` largest of
     logits + ``correction`` (a bias on the logits), weighed by the softmax over those alone.  With ROUTE_SIGMOID the
     scores are the sigmoids of the logits, each on its own; choice and weights as with the softmax.  Every weight is
-    multiplied by ``weight_scale``."""
+    multiplied by ``weight_scale``.  ``groups`` > 1: only outputs of the ``keep`` best of that many equal groups of
+    neighbours can be chosen (a group counts as much as the largest choice score in it); ``raw``: the weights are the
+    chosen scores as they are."""
     T, R = logits.shape
     _need(logits.dtype == torch.float32 and logits.stride(1) == 1, "router logits must be float32 [T, R]")
     _need(1 <= top <= min(R, MOE_MAX_TOP) and R <= MOE_MAX_ROUTER, f"top {top} of {R} router outputs: at most "
@@ -1418,7 +1640,7 @@ def moe_route(logits: torch.Tensor, correction: Optional[torch.Tensor], top: int
     weights = torch.empty((T, top), dtype=torch.float32, device=logits.device)
     _check(build.load("moe").ullm_moe_route(_p(logits), _c_int(logits.stride(0)), _p(correction), _c_int(T), _c_int(R),
                                             _c_int(top), _p(ids), _p(weights), _c_int(mode), _c_float(weight_scale),
-                                            _stream()), "moe_route")
+                                            _c_int(groups), _c_int(keep), _c_int(1 if raw else 0), _stream()), "moe_route")
     return ids, weights
 
 
@@ -1426,7 +1648,7 @@ MOE_ROUTER_MAX_WIDTH = 12288      # widest row the fused router kernel keeps in 
 
 
 def moe_router(x: torch.Tensor, w_router: torch.Tensor, correction: Optional[torch.Tensor], top: int,
-               mode: int = ROUTE_SOFTMAX_ALL, weight_scale: float = 1.0):
+               mode: int = ROUTE_SOFTMAX_ALL, weight_scale: float = 1.0, groups: int = 1, keep: int = 1, raw: bool = False):
     """:func:`moe_route` of the 32-bit product of ``x`` [T, H] with ``w_router`` (float32 [R, H]), in one kernel: every
     router output is summed along the row in an order that depends on nothing but the row."""
     T, H = x.shape
@@ -1443,7 +1665,7 @@ def moe_router(x: torch.Tensor, w_router: torch.Tensor, correction: Optional[tor
     weights = torch.empty((T, top), dtype=torch.float32, device=x.device)
     _check(build.load("moe").ullm_moe_router(_p(x), _c_int(x.stride(0)), _p(w_router), _p(correction), _c_int(T), _c_int(H),
                                              _c_int(R), _c_int(top), _p(ids), _p(weights), _c_int(mode), _c_float(weight_scale),
-                                             _c_int(_dt(x)),
+                                             _c_int(groups), _c_int(keep), _c_int(1 if raw else 0), _c_int(_dt(x)),
                                              _stream()), "moe_router")
     return ids, weights
 

@@ -7,7 +7,7 @@ Reference shape of the same thing: ullm/models/qwen3.py:199-286 (embedding, laye
 """
 from __future__ import annotations
 
-from dataclasses import dataclass, field
+from dataclasses import dataclass, field, replace
 from typing import Any, Dict, List, Optional, Sequence, Tuple
 
 import torch
@@ -59,6 +59,10 @@ class ModelPlan:
     # and writes it; later entries with the same id only read it, so a layer can read the cache
     # another layer wrote.  Default: every layer once, cache id = layer index.
     run_order: Optional[List[Tuple[int, int]]] = None
+    # {cache id: cache id}: the layer that owns the first reads the paged caches of the second, written by a layer that
+    # runs before it, in place of paged caches of its own; what it keeps beside those (fixed-size state) is its own.
+    # The pages live as long as the widest window of the writer and all such readers asks for.
+    kv_from: Dict[int, int] = field(default_factory=dict)
     # names a checkpoint may hold although this configuration has no use for them (a layer without a feed-forward
     # whose export still wrote that sublayer's norm): not loaded, and no error
     unused_tensors: Tuple[str, ...] = ()
@@ -80,6 +84,10 @@ class Model:
             if not (0 <= layer < len(self.blocks)):
                 raise ValueError(f"run order names layer {layer}: out of range")
             self.cache_owner.setdefault(cache_id, idx)
+        for reader, source in plan.kv_from.items():
+            if (reader not in self.cache_owner or source not in self.cache_owner or source in plan.kv_from
+                    or self.cache_owner[source] >= self.cache_owner[reader]):
+                raise ValueError(f"cache {reader} reads the keys of cache {source}: no layer with keys of its own that runs before it")
         self._keeps_embedding = any(b.needs_embedding for b in self.blocks)
         self.embedding: Optional[torch.Tensor] = None
         self.head: Optional[torch.Tensor] = None
@@ -125,8 +133,21 @@ class Model:
             if not isinstance(need, StateNeed):
                 raise TypeError("an embedder keeps fixed-size state per request or nothing")
             states[(EMBEDDER_CACHE, 0)] = need
-        for cache_id, idx in self.cache_owner.items():
-            for i, need in enumerate(cache_needs_of(self.blocks[self.run_order[idx][0]])):
+        own = {c: list(cache_needs_of(self.blocks[self.run_order[idx][0]])) for c, idx in self.cache_owner.items()}
+        self._borrowed = {}
+        for reader, source in self.plan.kv_from.items():
+            mine = [i for i, n in enumerate(own[reader]) if isinstance(n, KVNeed)]
+            theirs = [i for i, n in enumerate(own[source]) if isinstance(n, KVNeed)]
+            if [replace(own[reader][i], window=0) for i in mine] != [replace(own[source][i], window=0) for i in theirs]:
+                raise ValueError(f"cache {reader} reads the keys of cache {source} but their rows differ")
+            for i, j in zip(mine, theirs):
+                a, b = own[reader][i].window, own[source][j].window
+                own[source][j] = replace(own[source][j], window=max(a, b) if a and b else 0)
+                self._borrowed[(reader, i)] = (source, j)
+        for cache_id, needs in own.items():
+            for i, need in enumerate(needs):
+                if (cache_id, i) in self._borrowed:
+                    continue
                 if isinstance(need, KVNeed):
                     keyed.setdefault(need, []).append((cache_id, i))
                 else:
@@ -137,7 +158,8 @@ class Model:
                 cache_group[c] = len(groups)
             rows = tuple((r.heads, r.dim, None if r.dtype is None else torch.empty((), dtype=r.dtype).element_size())
                          for r in need.rows) if need.rows else None
-            groups.append(CacheGroupSpec(need.num_kv_heads, need.head_dim, need.window, tuple(keys), rows))
+            groups.append(CacheGroupSpec(need.num_kv_heads, need.head_dim, need.window, tuple(keys), rows,
+                                         need.tokens_per_row))
         self._group_needs = list(keyed)
         for idx, (layer, cache_id) in enumerate(self.run_order):
             owner_layer = self.run_order[self.cache_owner[cache_id]][0]
@@ -151,6 +173,11 @@ class Model:
         """The paged need of every cache group, in the order of :meth:`cache_layout`'s groups."""
         self.cache_layout()
         return self._group_needs
+
+    def borrowed_caches(self) -> Dict[Tuple[int, int], Tuple[int, int]]:
+        """{(cache id, need index): (cache id, need index) of the cache it reads instead} (see ``ModelPlan.kv_from``)."""
+        self.cache_layout()
+        return self._borrowed
 
     def num_needs(self, cache_id: int) -> int:
         """How many needs the block that owns this cache declares."""

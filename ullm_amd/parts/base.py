@@ -69,6 +69,7 @@ class KVNeed:
     head_dim: int
     window: int = 0               # keys a query looks back over, itself included; 0 = all
     rows: Tuple[CacheRows, ...] = ()
+    tokens_per_row: int = 1       # > 1: one row per this many tokens (row b stands for tokens b*n .. b*n + n - 1)
 
     def pools(self) -> Tuple[CacheRows, ...]:
         if self.rows:
@@ -319,9 +320,21 @@ class NormedBranch:
     norm that adds it (``Norm.add_norm``) applies ``post`` (a :class:`Norm` with ``kernel_form()``), the
     multiplier, the add and its own norm in one pass over the row.  Without ``post`` the branch joins the
     stream as ``mult * branch`` (a block that only scales what it adds)."""
-    branch: torch.Tensor          # [T, hidden] in the compute dtype or float32
+    branch: torch.Tensor          # [T, hidden] in the compute dtype or float32, or a stack [S, T, hidden] of partial sums
     post: Optional["Norm"]
     mult: float = 1.0
+    # two branches side by side: what is normed is a * branch + b * second (either may be a stack of partial sums)
+    second: Optional[torch.Tensor] = None
+    a: float = 1.0
+    b: float = 1.0
+
+    def joined(self) -> torch.Tensor:
+        """The branch as one tensor [T, hidden]."""
+        from ..kernels import ops
+        one = lambda y: ops.branch_sum(y) if y.dim() == 3 else y        # noqa: E731
+        if self.second is None:
+            return one(self.branch)
+        return ops.weighted_sum(one(self.branch), one(self.second), self.a, self.b)
 
 
 @dataclass

@@ -12,7 +12,7 @@ from typing import Optional
 import torch
 
 from ..kernels import ops
-from .base import (Block, FeedForward, LayerCache, Mixer, Norm, NormedBranch, PartEnv, PendingNorm, StepContext, StreamsBranch,
+from .base import (Block, FeedForward, LayerCache, Mixer, Norm, NormedBranch, PartEnv, PendingNorm, StateNeed, StepContext, StreamsBranch,
                    WeightDecl, register_part)
 
 
@@ -144,6 +144,87 @@ class ParallelBlock(Block):
             return residual, NormedBranch(self.ffn.forward_onto(h, ctx, _one_branch(mixed)), None, self.mult)
         # one kernel adds the two branches, whichever of them are stacks of partial sums
         return residual, NormedBranch(ops.branch_sum(mixed, self.ffn.forward(h, ctx)), None, self.mult)
+
+
+@register_part("block", "postnorm")
+class PostNormBlock(Block):
+    """Norms behind the sublayers and nowhere else: x += mixer_post(mixer(h)); x += ffn_post(ffn(x)).  The feed-forward (if
+    there is one) reads the stream itself; the mixer reads h = x or, with ``conv_taps``, h = x + conv(x) with a short causal
+    convolution over time per channel (``conv_weight`` [hidden, taps]: column ``taps - 1`` is the current token's), whose last
+    inputs are part of a request's state.  The mixer's needs follow the block's own.
+
+    A sublayer's output travels on as a :class:`NormedBranch`; one kernel norms it, adds it and stores what the next
+    sublayer reads (in a step of single tokens the convolution included)."""
+
+    def __init__(self, hidden_size: int, mixer: Mixer, mixer_post: Norm, ffn: Optional[FeedForward] = None,
+                 ffn_post: Optional[Norm] = None, conv_taps: int = 0, conv_weight: Optional[str] = None):
+        if (ffn is None) != (ffn_post is None):
+            raise ValueError("a feed-forward comes with its norm, or not at all")
+        if conv_taps and (conv_weight is None or not 1 <= conv_taps <= ops.SHORT_CONV_MAX_TAPS):
+            raise ValueError(f"a convolution of {conv_taps} taps: 1 to {ops.SHORT_CONV_MAX_TAPS}, with the name of its tensor")
+        self.hidden_size, self.taps, self.conv_weight = int(hidden_size), int(conv_taps), conv_weight
+        self.mixer, self.mixer_post, self.ffn, self.ffn_post = mixer, mixer_post, ffn, ffn_post
+        need = mixer.cache_need()
+        self._mixer_needs = [] if need is None else list(need) if isinstance(need, (list, tuple)) else [need]
+        self.w_conv: Optional[torch.Tensor] = None
+
+    def children(self):
+        return [p for p in (self.mixer, self.mixer_post, self.ffn, self.ffn_post) if p is not None]
+
+    def cache_need(self):
+        if not self.taps:
+            return self._mixer_needs or None
+        own = StateNeed((max(1, (self.taps - 1) * self.hidden_size),), torch.float32, graph_safe=True)
+        return [own] + self._mixer_needs
+
+    def weights(self):
+        return [WeightDecl(self.conv_weight, (self.hidden_size, self.taps), keep_fp32=True)] if self.taps else []
+
+    def bind(self, tensors, env: PartEnv) -> None:
+        if self.taps:
+            self.w_conv = tensors[self.conv_weight].t().contiguous()
+
+    def _mixer_input(self, residual, pending, ctx: StepContext, state):
+        if not self.taps:
+            return settle_normed(residual, pending, ctx.dtype)
+        rows = state.view(state.shape[0], -1)
+        if pending is not None and ctx.decode_only:
+            return settle_normed(residual, pending, ctx.dtype, conv=(self.w_conv, rows, ctx.entry_slot))
+        if pending is not None:
+            settle_normed(residual, pending, None)
+        return ops.short_conv(residual, self.w_conv, None, rows, 0, ctx, ops.CONV_RESIDUAL, ctx.dtype)
+
+    def forward(self, residual, pending, ctx: StepContext, cache: LayerCache):
+        if isinstance(pending, PendingNorm):
+            pending = None
+        own, mixer_cache = None, cache
+        if self.taps:
+            parts = cache.parts if cache.parts else [cache]
+            own = parts[0].state
+            mixer_cache = LayerCache.of_parts(parts[1:]) if self._mixer_needs else LayerCache()
+        h = self._mixer_input(residual, pending, ctx, own)
+        if hasattr(self.mixer, "forward_pair"):
+            first, a, second, b = self.mixer.forward_pair(h, ctx, mixer_cache, stacks=True)
+            pending = NormedBranch(first, self.mixer_post, second=second, a=a, b=b)
+        else:
+            pending = NormedBranch(self.mixer.forward(h, ctx, mixer_cache), self.mixer_post)
+        if self.ffn is None:
+            return residual, pending
+        x = settle_normed(residual, pending, ctx.dtype)
+        return residual, NormedBranch(self.ffn.forward(x, ctx), self.ffn_post)
+
+
+def settle_normed(residual, pending, out_dtype, conv=None):
+    """Add what is pending (a :class:`NormedBranch` with a norm behind it and no multiplier, or nothing) to the stream;
+    returns the stream in ``out_dtype`` (None: nothing), with ``conv`` = (weights, state rows, slots) plus its convolution."""
+    if pending is None:
+        return residual if out_dtype in (None, torch.float32) else residual.to(out_dtype)
+    if not isinstance(pending, NormedBranch) or pending.post is None or pending.mult != 1.0:
+        raise TypeError("a block that norms what its sublayers put out takes what a block of its kind left pending")
+    gain, eps, kind = pending.post.kernel_form()
+    if kind != ops.NORM_RMS:
+        raise TypeError("the norm behind a sublayer must be an RMS norm here")
+    return ops.post_add(pending.branch, residual, gain, eps, out_dtype, second=pending.second, a=pending.a, b=pending.b, conv=conv)
 
 
 @register_part("block", "mix_in_embedding")

@@ -236,11 +236,13 @@ class SideBySide(Mixer):
             at += n
         return out
 
-    def forward_pair(self, x: torch.Tensor, ctx: StepContext, cache: LayerCache):
-        """(left, left_scale, right, right_scale): the two branches, not yet added."""
+    def forward_pair(self, x: torch.Tensor, ctx: StepContext, cache: LayerCache, stacks: bool = False):
+        """(left, left_scale, right, right_scale): the two branches, not yet added.  ``stacks``: the caller also takes a
+        branch that is a stack of partial sums."""
+        one = (lambda y: y) if stacks else _plain
         left_cache, right_cache = self._views(cache)
-        return (_plain(self.left.forward(x, ctx, left_cache)), self.left_scale,
-                _plain(self.right.forward(x, ctx, right_cache)), self.right_scale)
+        return (one(self.left.forward(x, ctx, left_cache)), self.left_scale,
+                one(self.right.forward(x, ctx, right_cache)), self.right_scale)
 
     def forward(self, x: torch.Tensor, ctx: StepContext, cache: LayerCache) -> torch.Tensor:
         left, a, right, b = self.forward_pair(x, ctx, cache)

@@ -11,7 +11,9 @@ Two more forms, each a parameter: ``routing="top_logits"`` picks the ``top`` lar
 output (the ``correction`` tensor, then a bias on the logits) and weighs them by the softmax over the picked ones
 alone; ``routing="sigmoid"`` scores every output by the sigmoid of its own logit, chooses by score + correction and
 weighs by the chosen scores over their sum (+ 1e-20); ``weight_scale`` multiplies every weight; ``limit=None`` makes
-every expert the plain gated unit ``silu(g) * u``.
+every expert the plain gated unit ``silu(g) * u``; ``renormalize=False`` takes the chosen scores as weights as they are;
+``groups`` and ``keep_groups``: the router's outputs form that many equal groups of neighbours, and only outputs of the
+best ``keep_groups`` (by their largest choice score) can be chosen.
 
 The experts' matrices are stacked ([experts, 2 ff, hidden] with gate rows, then up rows, per expert, and
 [experts, hidden, ff]); the loader puts the checkpoint's per-expert tensors into their rows.  A step groups
@@ -50,11 +52,20 @@ class RoutedExperts(FeedForward):
     def __init__(self, hidden_size: int, experts: int, intermediate_size: int, top: int, limit: Optional[float],
                  prefix: str, identity: int = 0, alpha: float = 1.702, correction: bool = True,
                  shared_size: int = 0, shared_limit: Optional[float] = None, names: Optional[Dict[str, str]] = None,
-                 routing: str = "softmax_all", weight_scale: float = 1.0):
+                 routing: str = "softmax_all", weight_scale: float = 1.0, renormalize: bool = True, groups: int = 1,
+                 keep_groups: Optional[int] = None):
         modes = {"softmax_all": ops.ROUTE_SOFTMAX_ALL, "top_logits": ops.ROUTE_TOP_LOGITS, "sigmoid": ops.ROUTE_SIGMOID}
         if routing not in modes:
             raise ValueError(f"routing={routing!r}: one of {sorted(modes)}")
         self.mode, self.weight_scale = modes[routing], float(weight_scale)
+        self.raw, self.groups, self.keep_groups = not renormalize, int(groups), int(groups if keep_groups is None else keep_groups)
+        if self.raw and routing == "top_logits":
+            raise ValueError("routing='top_logits' weighs by a softmax over the chosen: always normalised")
+        outputs = experts + identity
+        if not 1 <= self.groups <= ops.MOE_MAX_GROUPS or outputs % self.groups or not 1 <= self.keep_groups <= self.groups \
+                or top > outputs // self.groups * self.keep_groups:
+            raise ValueError(f"{outputs} router outputs in {groups} equal groups (at most {ops.MOE_MAX_GROUPS}) of which "
+                             f"{self.keep_groups} are kept, {top} chosen")
         limit = 0.0 if limit is None else limit            # the kernels read a limit of 0 as the plain unit
         if experts < 0 or identity < 0 or experts + identity < 1:
             raise ValueError(f"{experts} experts and {identity} identity experts: a router needs at least one output")
@@ -109,9 +120,11 @@ class RoutedExperts(FeedForward):
     def route(self, x: torch.Tensor):
         """(ids int32 [T, top], weights float32 [T, top]) of the rows of x."""
         if self.hidden_size <= ops.MOE_ROUTER_MAX_WIDTH:
-            return ops.moe_router(x, self.w_router, self.correction, self.top, self.mode, self.weight_scale)     # the product and the routing in one
+            return ops.moe_router(x, self.w_router, self.correction, self.top, self.mode, self.weight_scale,     # the product and the routing in one
+                                  self.groups, self.keep_groups, self.raw)
         logits = ops.gemm_simple(x, self.w_router, out_dtype=torch.float32)       # 32-bit sums in a fixed order
-        return ops.moe_route(logits, self.correction, self.top, self.mode, self.weight_scale)
+        return ops.moe_route(logits, self.correction, self.top, self.mode, self.weight_scale, self.groups, self.keep_groups,
+                             self.raw)
 
     def forward(self, x: torch.Tensor, ctx: StepContext) -> torch.Tensor:
         return self.forward_onto(x, ctx, None, None)

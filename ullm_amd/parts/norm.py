@@ -18,17 +18,19 @@ from .base import Norm, NormedBranch, PartEnv, PendingNorm, WeightDecl, register
 class RMSNorm(Norm):
     adds_stacks = True
 
-    def __init__(self, size: int, eps: float, weight_name: str):
+    def __init__(self, size: int, eps: float, weight_name: str, around_zero: bool = False):
         self.size = size
         self.eps = float(eps)
         self.weight_name = weight_name
+        self.around_zero = bool(around_zero)             # the checkpoint stores the gain minus one
         self.gain: Optional[torch.Tensor] = None
 
     def weights(self) -> List[WeightDecl]:
-        return [WeightDecl(self.weight_name, (self.size,), init="gain", keep_fp32=True)]
+        return [WeightDecl(self.weight_name, (self.size,), init="normal" if self.around_zero else "gain", keep_fp32=True)]
 
     def bind(self, tensors: Dict[str, torch.Tensor], env: PartEnv) -> None:
-        self.gain = tensors[self.weight_name].contiguous()
+        gain = tensors[self.weight_name]
+        self.gain = (1.0 + gain if self.around_zero else gain).contiguous()
 
     def add_norm(self, branch, residual, rows=None, out_dtype=None):
         if isinstance(branch, NormedBranch):
@@ -57,7 +59,10 @@ def add_normed_branch(branch: NormedBranch, residual, form, rows, out_dtype):
         if post is None:
             raise TypeError(f"{type(branch.post).__name__} cannot stand behind a branch: it has no kernel form")
         post_gain, post_eps, post_kind = post
-    return ops.add_norm_general(branch.branch, residual, gain, eps, kind, out_dtype or branch.branch.dtype, rows=rows,
+    y = branch.branch
+    if branch.second is not None or y.dim() == 3:
+        y = branch.joined()
+    return ops.add_norm_general(y, residual, gain, eps, kind, out_dtype or y.dtype, rows=rows,
                                 post_gain=post_gain, post_eps=post_eps, post_kind=post_kind, mult=branch.mult)
 
 

@@ -40,7 +40,8 @@ class Rotary(PositionEncoding):
     keep their size."""
 
     def __init__(self, head_dim: int, theta: float, rotary_dim: Optional[int] = None,
-                 pairing: str = "half", max_positions: Optional[int] = None, scaling: Optional[tuple] = None):
+                 pairing: str = "half", max_positions: Optional[int] = None, scaling: Optional[tuple] = None,
+                 exact: bool = False):
         self.head_dim = head_dim
         self.theta = float(theta)
         self.rotary_dim = head_dim if rotary_dim is None else rotary_dim
@@ -50,6 +51,9 @@ class Rotary(PositionEncoding):
             raise ValueError(f"unknown rotary pairing {pairing!r}")
         self.style = 1 if pairing == "half" else 2
         self.max_positions = max_positions
+        # angles formed in 64-bit (with a stretch they always are): far positions' 32-bit cosines and sines are then the
+        # roundings of the exact values
+        self.exact = bool(exact)
         self.scaling = None
         if scaling is not None and scaling[0] == "by_wavelength":
             self.scaling = ("by_wavelength",) + tuple(float(v) for v in scaling[1:])
@@ -62,7 +66,12 @@ class Rotary(PositionEncoding):
         self.table: Optional[torch.Tensor] = None
 
     @staticmethod
-    def make_table(rotary_dim: int, theta: float, rows: int, scaling: Optional[tuple] = None) -> torch.Tensor:
+    def make_table(rotary_dim: int, theta: float, rows: int, scaling: Optional[tuple] = None, exact: bool = False) -> torch.Tensor:
+        if scaling is None and exact:
+            i = torch.arange(rotary_dim // 2, dtype=torch.float64)
+            freq = torch.pow(torch.tensor(float(theta), dtype=torch.float64), -2.0 * i / rotary_dim)
+            angles = torch.arange(rows, dtype=torch.float64)[:, None] * freq[None, :]
+            return torch.cat((angles.cos(), angles.sin()), dim=-1).to(torch.float32).contiguous()
         if scaling is None:
             inv_freq = 1.0 / (theta ** (torch.arange(0, rotary_dim, 2, dtype=torch.float32) / rotary_dim))
             angles = torch.arange(rows, dtype=torch.float32)[:, None] * inv_freq[None, :]
@@ -95,8 +104,8 @@ class Rotary(PositionEncoding):
     def bind(self, tensors: Dict[str, torch.Tensor], env: PartEnv) -> None:
         rows = env.context_len if self.max_positions is None else min(env.context_len, self.max_positions)
         # every layer with the same rotation shares one table: built once, read by all their kernels
-        self.table = env.shared(("rotary", self.rotary_dim, self.theta, rows, self.scaling),
-                                lambda: self.make_table(self.rotary_dim, self.theta, rows, self.scaling).to(env.device))
+        self.table = env.shared(("rotary", self.rotary_dim, self.theta, rows, self.scaling, self.exact),
+                                lambda: self.make_table(self.rotary_dim, self.theta, rows, self.scaling, self.exact).to(env.device))
 
     def kernel_args(self):
         return self.table, self.rotary_dim, self.style

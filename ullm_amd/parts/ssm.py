@@ -1,4 +1,6 @@
-"""A selective state-space mixer (the Mamba-2 form) over per-request state.
+"""Selective state-space mixers over per-request state.
+
+``mamba2``, the Mamba-2 form:
 
 The input projection's rows are z | x | B | C | dt (z, x: heads * head_dim; B, C: groups * state; dt: heads).
 x | B | C pass a short causal convolution per channel and silu; dt = softplus(dt + dt_bias).  Per head h
@@ -10,9 +12,18 @@ What a request keeps between steps is one float32 row per slot: the convolution'
 every head's state.  Everything behind the input projection is 32-bit (the projection leaves float32 rows
 also where the model computes in bfloat16); the recurrence walks an entry's tokens in order whatever the
 batch holds, so a token's result does not depend on how its prompt was cut.
+
+``selective_scan``, the first Mamba form, with a state per channel:
+
+The input projection's rows are x | z (``inner`` each).  x passes the short convolution (with a bias) and silu; W_x x is
+dt | B | C (``dt_rank``, ``state``, ``state`` values); the step sizes are softplus(W_dt dt + bias), one per channel.  Per
+channel c and state n:  S = exp(-exp(A_log) dt) S + dt x B,  y = sum_n S C + D x;  y * silu(z) is projected out.  A
+request's float32 row holds the convolution's last inputs, then the states.  Step sizes, decays and states are 32-bit;
+the projections and the convolution's result are stored in the compute dtype (B, C and the step sizes in 32-bit).
 """
 from __future__ import annotations
 
+import math
 from typing import Dict, List, Optional
 
 import torch
@@ -75,3 +86,59 @@ class Mamba2(Mixer):
                          self.head_dim, write_state=cache.owner)
         gated = ops.gated_group_norm(y, proj, 0, self.norm_gain, self.norm_eps, self.norm_groups, ctx.dtype)
         return linear_into_stream(gated, self.w_out, ctx)
+
+
+SCAN_NAMES = {"in": "in", "conv": "conv", "conv_bias": "conv.b", "x": "x", "dt": "dt", "dt_bias": "dt.b", "a_log": "A_log",
+              "d": "D", "out": "o"}
+
+
+@register_part("mixer", "selective_scan")
+class SelectiveScan(Mixer):
+    def __init__(self, hidden_size: int, inner: int, state: int, dt_rank: int, conv: int, prefix: str,
+                 names: Optional[Dict[str, str]] = None):
+        if min(inner, state, dt_rank) < 1 or state > ops.SELECTIVE_SCAN_MAX_STATE:
+            raise ValueError(f"sizes must be positive and the state at most {ops.SELECTIVE_SCAN_MAX_STATE}")
+        if not 1 <= conv <= ops.SHORT_CONV_MAX_TAPS:
+            raise ValueError(f"a convolution of {conv} taps: 1 to {ops.SHORT_CONV_MAX_TAPS}")
+        self.hidden_size, self.inner, self.state, self.dt_rank, self.taps = hidden_size, inner, state, dt_rank, conv
+        self.prefix, self.names = prefix, {**SCAN_NAMES, **(names or {})}
+        self.carry = (conv - 1) * inner                               # the convolution's part of the state row
+
+    def _name(self, role: str) -> str:
+        return f"{self.prefix}.{self.names[role]}"
+
+    def cache_need(self):
+        return StateNeed((self.carry + self.inner * self.state,), torch.float32, graph_safe=True)
+
+    def weights(self) -> List[WeightDecl]:
+        H, n, small = self.hidden_size, self.inner, dict(keep_fp32=True)
+        return [WeightDecl(self._name("in"), (2 * n, H)),
+                WeightDecl(self._name("conv"), (n, self.taps), **small), WeightDecl(self._name("conv_bias"), (n,), **small),
+                WeightDecl(self._name("x"), (self.dt_rank + 2 * self.state, n)),
+                WeightDecl(self._name("dt"), (n, self.dt_rank)), WeightDecl(self._name("dt_bias"), (n,), **small),
+                WeightDecl(self._name("a_log"), (n, self.state), **small), WeightDecl(self._name("d"), (n,), **small),
+                WeightDecl(self._name("out"), (H, n))]
+
+    def bind(self, tensors: Dict[str, torch.Tensor], env: PartEnv) -> None:
+        get = lambda role: tensors[self._name(role)]                     # noqa: E731
+        self.w_in, self.w_out = get("in").contiguous(), get("out").contiguous()
+        self.w_conv, self.b_conv = get("conv").t().contiguous(), get("conv_bias").contiguous()
+        # the low-rank step sizes' inner size is padded with zeros to a multiple of eight: whole 16-byte pieces
+        r, pad = self.dt_rank, -self.dt_rank % 8
+        x, dt = get("x"), get("dt")
+        self.w_dt_low = torch.cat((x[:r], x.new_zeros((pad, self.inner)))).contiguous()
+        self.w_bc = x[r:].contiguous()
+        self.w_dt = torch.cat((dt, dt.new_zeros((self.inner, pad))), dim=1).contiguous()
+        self.dt_bias, self.d_skip = get("dt_bias").contiguous(), get("d").contiguous()
+        # A log2(e), rounded to 32-bit once: a decay is then one exponent of two
+        self.a_log2 = (-torch.exp(get("a_log").to(torch.float64)) * math.log2(math.e)).to(torch.float32).contiguous()
+
+    def forward(self, x: torch.Tensor, ctx: StepContext, cache: LayerCache) -> torch.Tensor:
+        n, rows = self.inner, cache.state.view(cache.state.shape[0], -1)
+        proj = linear(x, self.w_in)                                      # x | z
+        u = ops.short_conv(proj[:, :n], self.w_conv, self.b_conv, rows, 0, ctx, ops.CONV_SILU, ctx.dtype, write_state=cache.owner)
+        bc = linear(u, self.w_bc, out_dtype=torch.float32)
+        dt = linear(linear(u, self.w_dt_low), self.w_dt, out_dtype=torch.float32)
+        y = ops.selective_scan(u, dt, bc, proj[:, n:], self.a_log2, self.dt_bias, self.d_skip, rows, self.carry, ctx,
+                               write_state=cache.owner)
+        return linear_into_stream(y, self.w_out, ctx)
