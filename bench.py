@@ -55,13 +55,15 @@ def parse_args():
                     help="instead of the default workload: Pamopel (attention with a distance bias and head gates, a "
                          "layer on another's keys and values, a Mamba-2 layer) beside a Qwen3 stack of the same width, "
                          f"heads, feed-forward, vocabulary and depth, random weights; shapes: {sorted(DESIGN_SHAPES)}")
-    ap.add_argument("--design-model", choices=("both", "all", "pamopel", "qwen3", "ziferax", "dovisun", "kumudra"), default="both",
+    ap.add_argument("--design-model", choices=("both", "all", "pamopel", "qwen3", "ziferax", "dovisun", "kumudra", "nadevik"), default="both",
                     help="with --design: one design only (for profiles), Pamopel and Qwen3 (both), or these, Ziferax "
                          "(a stack of parallel blocks of windowed attention with sinks and a routed feed-forward) and "
                          "Dovisun (parallel blocks of unit-norm attention with a fixed sink or latent attention, dense "
                          "or routed feed-forwards, two layers passed twice) and Kumudra (two copies of the residual "
                          "stream, gated linear attention, lightning attention and windowed attention beside time "
-                         "mixing, four layers passed twice) (all)")
+                         "mixing, four layers passed twice) and Nadevik (norms behind the sublayers, sigmoid attention "
+                         "over a window and pooled blocks beside a selective scan, windowed latent attention, experts "
+                         "from the best groups) (all)")
     ap.add_argument("--prefill-only", type=int, default=0, metavar="T",
                     help="only time a T-token prompt and print its figures (for profiling)")
     return ap.parse_args()
@@ -210,13 +212,37 @@ def kumudra_config(shape):
                 residual_mult=0.5, embedding=dict(scale=1.0), loop=dict(start=0, stop=4, times=max(1, L // 4)))
 
 
+# Nadevik at a design shape: the same width, heads and depth.  Of every four layers the first and the last are two mixers
+# side by side, attention (the other stacks' heads, a window of 1024 keys, beyond it a key per block of 16 tokens) and a
+# selective scan (twice the width, 16 states a channel, step sizes of rank width / 16); the second is latent attention (the
+# other latent stack's sizes, the same window) and the third reads the second's latents.  Every feed-forward is routed,
+# with as many columns a token as the dense stack's (top 4 of 32 experts of a sixth of it, in four groups of which three
+# are kept).
+def nadevik_config(shape):
+    (W, H, G, D, F, L), _ = DESIGN_SHAPES[shape]
+    mlp = dict(kind="moe", router=dict(experts=32, top=4, groups=dict(count=4, keep=3)), expert=dict(ff=F // 6, limit=7.0))
+    left = dict(heads=H, kv_heads=G, dim=D, vdim=D, conv=4, scale=D ** -0.5, softcap=30.0, mask=dict(size=1024, pool=16))
+    parallel = dict(left=left, right=dict(inner=2 * W, state=16, dt_rank=W // 16, conv=4), left_scale=0.7, right_scale=0.8)
+    latent = dict(heads=H, dim=D, rot_dim=D // 2, vdim=D, kv_rank=192, scale=(D + D // 2) ** -0.5, mask=dict(size=1024),
+                  rot=dict(base=1e6, dims=D // 2))
+    layers = []
+    for i in range(L):
+        if i % 4 in (0, 3):
+            layers.append(dict(type="parallel", mixer=parallel, mlp=mlp))
+        else:
+            layers.append(dict(type="latent_attention", mixer=dict(latent, kv_from=i - 1) if i % 4 == 2 else latent, mlp=mlp))
+    return dict(architecture="Nadevik", vocab=DESIGN_VOCAB, width=W, norm=dict(eps=1e-6), canon=dict(taps=4), layers=layers,
+                embedding=dict(scale=float(W) ** 0.5, bigram=dict(buckets=65521, mul_prev=8191, mul_cur=127)))
+
+
 def design_run(args):
     """Decode at batch 1 / 8 / 64 (1024-token prompts) and one 2048-token prompt, for the designs of a shape."""
     out = {"metric": f"decode and prefill tok/s, designs beside Qwen3 at shape {args.design}, random weights",
            "unit": "tokens/s", "dtype": args.dtype, "data": "synthetic", "shape": args.design, "designs": {}}
-    configs = design_configs(args.design) + (ziferax_config(args.design), dovisun_config(args.design), kumudra_config(args.design))
-    for label, config in zip(("pamopel", "qwen3", "ziferax", "dovisun", "kumudra"), configs):
-        if args.design_model not in ("both", "all", label) or (label in ("ziferax", "dovisun", "kumudra") and args.design_model == "both"):
+    configs = design_configs(args.design) + (ziferax_config(args.design), dovisun_config(args.design), kumudra_config(args.design),
+                                             nadevik_config(args.design))
+    for label, config in zip(("pamopel", "qwen3", "ziferax", "dovisun", "kumudra", "nadevik"), configs):
+        if args.design_model not in ("both", "all", label) or (label not in ("pamopel", "qwen3") and args.design_model == "both"):
             continue
         m = Sized(label, args.dtype, 4096, eager=args.eager, config=config)
         rec = {"weights_GB": round(m.wbytes / 1e9, 3), "decode": {}}

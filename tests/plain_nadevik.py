@@ -188,17 +188,19 @@ MARGINS = None      # a list: every routed layer run appends, per token, how clo
 
 def choose_experts(s, top, groups, keep):
     """(indices of the ``top`` largest of the scores ``s`` [n] among the ``keep`` best of ``groups`` equal groups of
-    neighbours, the smaller of the two gaps between what was taken and what was left)."""
+    neighbours, the smaller of the two gaps between what was taken and what was left: differences of the scores'
+    logarithms, that is of the router's logits)."""
+    gap = lambda a, b: math.log(a.item() / b.item()) if b.item() > 0 else math.inf        # noqa: E731
     n = s.numel()
     size = n // groups
     best = s.view(groups, size).max(-1).values
     order = sorted(range(groups), key=lambda g: (-best[g].item(), g))
     allowed = sorted(order[:keep])
-    margin = math.inf if keep >= groups else (best[order[keep - 1]] - best[order[keep]]).item()
+    margin = math.inf if keep >= groups else gap(best[order[keep - 1]], best[order[keep]])
     cand = [e for g in allowed for e in range(g * size, (g + 1) * size)]
     cand.sort(key=lambda e: (-s[e].item(), e))
     if top < len(cand):
-        margin = min(margin, (s[cand[top - 1]] - s[cand[top]]).item())
+        margin = min(margin, gap(s[cand[top - 1]], s[cand[top]]))
     return cand[:top], margin
 
 
@@ -314,7 +316,7 @@ def random_weights(cfg, seed, std=None):
         elif last == "bigram":
             t = 0.5 * r
         elif last == "router":
-            t = r * 2.5 / math.sqrt(shape[-1])
+            t = r * 1.2 / math.sqrt(shape[-1])
         else:
             t = r * (std if std is not None else 1.2 / math.sqrt(shape[-1]))
         out[name] = t.to(torch.bfloat16)

@@ -1358,15 +1358,17 @@ def short_conv(x: torch.Tensor, weight: torch.Tensor, bias: Optional[torch.Tenso
 
 
 SELECTIVE_SCAN_MAX_STATE = 256
+SCAN_SEGMENT = 64                        # tokens of a segment of the scan over a prompt's portion
 
 
 def selective_scan(x: torch.Tensor, raw_dt: torch.Tensor, bc: torch.Tensor, z: torch.Tensor, a_log2: torch.Tensor,
-                   dt_bias: torch.Tensor, d_skip: torch.Tensor, state: torch.Tensor, state_off: int, ctx,
+                   dt_bias: torch.Tensor, d_skip: torch.Tensor, state: torch.Tensor, state_off: int, ctx, plan=None,
                    write_state: bool = True) -> torch.Tensor:
     """Per channel c and state n over each entry's tokens: dt = softplus(raw_dt + dt_bias), S = exp(dt A) S + dt x B,
     y = sum_n S C + d_skip x; returns y * silu(z) ([T, inner] of x's dtype).  ``raw_dt`` float32 [T, inner], ``bc`` float32
-    [T, >= 2 n] (B, then C), ``a_log2`` float32 [inner, n] = A log2(e); ``x`` and ``z`` may be columns of wider rows.  The
-    states are float32 at ``state[slot, state_off + c * n ..]``."""
+    [T, 2 n] (B, then C), ``a_log2`` float32 [inner, n] = A log2(e); ``x``, ``z`` and ``bc`` may be columns of wider rows.  The
+    states are float32 at ``state[slot, state_off + c * n ..]``.  ``plan`` lists the segments the entries' tokens are cut
+    into (:func:`~ullm_amd.parts.ssm.plan_scan_segments`; None: every entry is walked in order)."""
     T, inner = x.shape
     n = a_log2.shape[1]
     _need(x.stride(1) == 1 and z.shape == (T, inner) and z.stride(1) == 1 and z.dtype == x.dtype, "x and z must be [T, inner] of one dtype")
@@ -1378,12 +1380,24 @@ def selective_scan(x: torch.Tensor, raw_dt: torch.Tensor, bc: torch.Tensor, z: t
         _need(v.dtype == torch.float32 and v.numel() == inner and v.is_contiguous(), f"{nm} must be float32 [inner]")
     _check_step_state(state, state_off, inner * n, "the scan's state")
     out = torch.empty((T, inner), dtype=x.dtype, device=x.device)
-    ll = ctypes.c_longlong
-    _check(build.load("selective_scan").ullm_selective_scan(
-        _p(x), _c_int(x.stride(0)), _p(raw_dt), _c_int(raw_dt.stride(0)), _p(bc), _c_int(bc.stride(0)), _p(z), _c_int(z.stride(0)),
-        _p(a_log2), _p(dt_bias), _p(d_skip), _p(state), ll(state.stride(0)), ll(state_off), _p(ctx.q_start), _p(ctx.entry_slot),
-        _p(out), _c_int(ctx.num_entries), _c_int(inner), _c_int(n), _c_int(1 if write_state else 0), _c_int(_dt(x)), _stream()),
-        "selective_scan")
+    ll, lib = ctypes.c_longlong, build.load("selective_scan")
+    head = (_p(x), _c_int(x.stride(0)), _p(raw_dt), _c_int(raw_dt.stride(0)), _p(bc), _c_int(bc.stride(0)), _p(z), _c_int(z.stride(0)),
+            _p(a_log2), _p(dt_bias), _p(d_skip), _p(state), ll(state.stride(0)), ll(state_off))
+    tail = (_c_int(inner), _c_int(n), _c_int(1 if write_state else 0), _c_int(_dt(x)), _stream())
+    if ctx.decode_only:
+        _check(lib.ullm_selective_scan_step(*head, _p(ctx.entry_slot), _p(out), _c_int(ctx.num_entries), *tail), "selective_scan_step")
+    elif plan is not None and n <= 64:
+        items, chains = plan.facts["num_items"], plan.facts["num_chains"]
+        chain = torch.empty(items * n * inner if chains else 0, dtype=torch.float32, device=x.device)
+        sums = torch.empty(items * inner if chains else 0, dtype=torch.float32, device=x.device)
+        _i32(plan.arrays["items"], "items", 4 * items)
+        _i32(plan.arrays["chains"], "chains", 3 * chains)
+        _check(lib.ullm_selective_scan_segments(
+            *head, _p(ctx.entry_slot), _p(plan.arrays["items"]), _c_int(items), _p(plan.arrays["chains"]), _c_int(chains),
+            _p(chain), _p(sums), _p(out), *tail), "selective_scan_segments")
+    else:
+        _check(lib.ullm_selective_scan(*head, _p(ctx.q_start), _p(ctx.entry_slot), _p(out), _c_int(ctx.num_entries), *tail),
+               "selective_scan")
     return out
 
 

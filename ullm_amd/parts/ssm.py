@@ -26,10 +26,11 @@ from __future__ import annotations
 import math
 from typing import Dict, List, Optional
 
+import numpy as np
 import torch
 
 from ..kernels import ops
-from .base import LayerCache, Mixer, PartEnv, StateNeed, StepContext, WeightDecl, register_part
+from .base import LayerCache, Mixer, PartEnv, StateNeed, StepContext, StepPlan, StepShape, WeightDecl, register_part
 from .linear import linear, linear_into_stream
 
 DEFAULT_NAMES = {"in": "in_proj.weight", "conv": "conv1d.weight", "conv_bias": "conv1d.bias", "dt_bias": "dt_bias",
@@ -88,12 +89,32 @@ class Mamba2(Mixer):
         return linear_into_stream(gated, self.w_out, ctx)
 
 
+def plan_scan_segments(shape: StepShape) -> StepPlan:
+    """The segments of up to ``ops.SCAN_SEGMENT`` tokens an entry's tokens are cut into, as (entry, first token, tokens, what:
+    0 its only one, 1 one of several, 2 the last of several), and for entries of several (entry, first item, items).  A step
+    of single tokens lists none."""
+    items, chains, t0 = [], [], 0
+    if any(n != 1 for n in shape.lens):
+        for b, n in enumerate(shape.lens):
+            count = -(-n // ops.SCAN_SEGMENT)
+            if count > 1:
+                chains.extend((b, len(items) // 4, count))
+            for i in range(count):
+                first = i * ops.SCAN_SEGMENT
+                items.extend((b, t0 + first, min(ops.SCAN_SEGMENT, n - first), 0 if count == 1 else 1 if i + 1 < count else 2))
+            t0 += n
+    return StepPlan(arrays={"items": np.asarray(items, dtype=np.int32), "chains": np.asarray(chains, dtype=np.int32)},
+                    facts={"num_items": len(items) // 4, "num_chains": len(chains) // 3})
+
+
 SCAN_NAMES = {"in": "in", "conv": "conv", "conv_bias": "conv.b", "x": "x", "dt": "dt", "dt_bias": "dt.b", "a_log": "A_log",
               "d": "D", "out": "o"}
 
 
 @register_part("mixer", "selective_scan")
 class SelectiveScan(Mixer):
+    step_planners = {"scan segments": plan_scan_segments}
+
     def __init__(self, hidden_size: int, inner: int, state: int, dt_rank: int, conv: int, prefix: str,
                  names: Optional[Dict[str, str]] = None):
         if min(inner, state, dt_rank) < 1 or state > ops.SELECTIVE_SCAN_MAX_STATE:
@@ -140,5 +161,5 @@ class SelectiveScan(Mixer):
         bc = linear(u, self.w_bc, out_dtype=torch.float32)
         dt = linear(linear(u, self.w_dt_low), self.w_dt, out_dtype=torch.float32)
         y = ops.selective_scan(u, dt, bc, proj[:, n:], self.a_log2, self.dt_bias, self.d_skip, rows, self.carry, ctx,
-                               write_state=cache.owner)
+                               ctx.plans["scan segments"], write_state=cache.owner)
         return linear_into_stream(y, self.w_out, ctx)
