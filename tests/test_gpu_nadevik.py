@@ -195,6 +195,26 @@ def test_whole_prompts(replayers, models, name, dtype):
         agree(models, name, toks, run(rep, "r", toks, [n]), dtype)
 
 
+@pytest.mark.parametrize("name,dtype", [("par", "float32"), ("par", "bfloat16"), ("C", "float32"), ("A", "float32")])
+def test_long_portions_of_two_requests_in_one_step(replayers, models, name, dtype):
+    """Steps of more than 512 tokens (kernels that take several tokens a block), the second request's tokens off every
+    block's edge, then the rest of both."""
+    rep = replayers(name, dtype, max_tokens=1280)
+    vocab = models[name][1]["vocab"]
+    a, b = tokens(vocab, 597, 80), tokens(vocab, 390, 81)
+    got = {"a": [], "b": []}
+    for step, cut in enumerate(({"a": 333, "b": 279}, {"a": 264, "b": 111})):
+        at = {"a": 0 if step == 0 else 333, "b": 0 if step == 0 else 279}
+        entries = [{"id": k, "tokens": t[at[k]:at[k] + cut[k]], "want": list(range(cut[k]))} for k, t in (("a", a), ("b", b))]
+        out = rep.step({"step": step, "entries": entries, "end": [] if step == 0 else ["a", "b"]})
+        got["a"].append(out[:cut["a"]])
+        got["b"].append(out[cut["a"]:])
+    agree(models, name, a, np.concatenate(got["a"]), dtype)
+    agree(models, name, b, np.concatenate(got["b"]), dtype)
+    one = run(rep, "r", a, [597])                        # and one request alone, from a page's first row on
+    agree(models, name, a, one, dtype)
+
+
 @pytest.mark.parametrize("name", ["A", "B", "C"])
 def test_the_stream_after_every_layer(models, name):
     """Layer by layer in 32-bit: the stream once what the layer left pending is normed and added."""
@@ -419,22 +439,24 @@ def step_context(lens, starts=None, slots=None):
 
 
 STEPS = ([37, 1, 70], [2, 18, 1], [1, 1, 1], [1, 1, 1])
+LONG_STEPS = ([301, 2, 1], [1, 1800, 270], [5, 1, 1])
 
 
 @pytest.mark.parametrize("channels,taps", [(24, 1), (24, 2), (300, 3), (1028, 4), (7, 4), (40, 9)])
 @pytest.mark.parametrize("mode", ["silu", "residual"])
+@pytest.mark.parametrize("steps", [STEPS, LONG_STEPS], ids=["short", "long"])
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
-def test_the_short_convolution_alone(channels, taps, mode, dtype):
-    """Three requests in four steps; the inputs in columns of wider rows, the state behind other values."""
+def test_the_short_convolution_alone(channels, taps, mode, steps, dtype):
+    """Three requests in several steps; the inputs in columns of wider rows, the state behind other values."""
     from ullm_amd.kernels import ops
     g = torch.Generator().manual_seed(channels + taps)
-    xs = [torch.randn(sum(s[i] for s in STEPS), channels, generator=g).to(dtype) for i in range(3)]
+    xs = [torch.randn(sum(s[i] for s in steps), channels, generator=g).to(dtype) for i in range(3)]
     w, bias = torch.randn(channels, taps, generator=g), torch.randn(channels, generator=g)
     off = 4
     state = torch.full((5, off + max(1, (taps - 1) * channels)), 3.0, device=DEV)
     state[:, off:] = 0.0
     at, got = [0, 0, 0], [[], [], []]
-    for lens in STEPS:
+    for lens in steps:
         ctx = step_context(lens)
         rows = torch.cat([x[a:a + n] for x, a, n in zip(xs, at, lens)])
         wide = torch.cat((torch.randn(rows.shape[0], 8).to(dtype), rows), dim=1).to(DEV)
@@ -469,7 +491,7 @@ def test_the_selective_scan_alone(inner, N, segments, dtype):
     seqs = []
     for i in range(3):
         n = sum(s[i] for s in STEPS)
-        seqs.append((torch.randn(n, inner, generator=g).to(dtype), torch.randn(n, inner, generator=g) * 2, torch.randn(n, 2 * N, generator=g),
+        seqs.append((torch.randn(n, inner, generator=g).to(dtype), torch.randn(n, inner, generator=g) * 2, torch.randn(n, 2 * N, generator=g).to(dtype),
                      torch.randn(n, inner, generator=g).to(dtype)))
     want = []
     for x, raw, bc, z in seqs:

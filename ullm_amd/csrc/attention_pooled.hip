@@ -265,9 +265,18 @@ pooled_reduce_kernel(const float* __restrict__ part, bf16_t* __restrict__ out, c
 //   keys   LDS row = one key, hd values + 32 bytes of padding
 //   values LDS row = one dim, its 32 keys in the order [g][half][4] (the 8 keys lane group g feeds to one product are 16
 //          adjacent bytes) + 32 bytes of padding
-// Two LDS tiles take turns and the loads of the next tile are in flight during the products of the current one.
+// Two LDS tiles take turns, and the loads of the next two tiles are in flight during the products of the current one (the
+// barrier between tiles waits for shared memory alone).
 // grid (n_tiles * nkv, unit chunks); kv heads vary fastest, so that a kv head's keys stay in one die's cache where the
 // number of kv heads is a multiple of the dies'.
+__device__ __forceinline__ void lds_barrier() {
+#ifdef __HIP_DEVICE_COMPILE__
+  asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+  __builtin_amdgcn_s_barrier();
+  asm volatile("" ::: "memory");
+#endif
+}
+
 #define PF_WAVES 4
 #define PF_THREADS (64 * PF_WAVES)
 
@@ -320,99 +329,117 @@ pooled_prefill_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t* __rest
 #pragma unroll
     for (int n = 0; n < 2 * NQK; ++n) acc[u][n] = f32x4_t{0.f, 0.f, 0.f, 0.f};
 
-  uint4 rk[PIECES], rv[PIECES];
-  auto fetch = [&](int i) __attribute__((always_inline)) {
+  const KeyRanges ranges = {k_pool, v_pool, pk_pool, pv_pool, bt, pbt, page_size, nkv, kvh};
+  struct Stage {                                          // a tile on its way from the cache to LDS
+    uint4 k[PIECES], v[PIECES];
+  };
+  PieceWindow win = load_pieces(0, nb_max, pt, first, p_last, ranges);
+  auto fetch = [&](int i, Stage& st) __attribute__((always_inline)) {
+    if (2 * i + 1 >= win.base + 64) win = load_pieces(2 * i, nb_max, pt, first, p_last, ranges);
     const bool pooled = i < pt;
-    const int key0 = pooled ? 32 * i : first + 32 * (i - pt), limit = pooled ? nb_max - 1 : p_last;
     const bf16_t* const kb = pooled ? pk_pool : k_pool;
     const bf16_t* const vb = pooled ? pv_pool : v_pool;
-    const int* const table = pooled ? pbt : bt;
 #pragma unroll
     for (int j = 0; j < PIECES; ++j) {
       const int piece = tid + j * PF_THREADS;
-      const int sb = piece / (2 * HD), rem = piece % (2 * HD), kb16 = key0 + 16 * sb;
-      rk[j] = rv[j] = make_uint4(0, 0, 0, 0);
-      if (piece >= 4 * HD || kb16 > limit) continue;
-      const int page = table[kb16 / page_size], off = kb16 % page_size;
+      const int sb = piece / (2 * HD), rem = piece % (2 * HD);            // the half is the same for a whole wave
+      st.k[j] = st.v[j] = make_uint4(0, 0, 0, 0);
+      if (piece >= 4 * HD) continue;
+      const int at = __builtin_amdgcn_readfirstlane(2 * i + sb - win.base);
+      const int page = __builtin_amdgcn_readlane(win.page, at), off = __builtin_amdgcn_readlane(win.off, at);
       if (page < 0) continue;
-      rk[j] = ld16(kb + (((size_t)page * nkv + kvh) * page_size + off + rem / (HD / 8)) * HD + 8 * (rem % (HD / 8)));
-      rv[j] = ld16(vb + (((size_t)page * nkv + kvh) * HD + rem / 2) * page_size + off + 8 * (rem % 2));
-      // values of rows behind the data are not to be multiplied, even by zero
-      const int over = kb16 + 8 * (rem % 2) + 7 - limit;                          // how many of the eight lie behind
-      if (over > 0) {
-        Pack8 v;
-        v.u4 = rv[j];
-#pragma unroll
-        for (int e = 0; e < 8; ++e)
-          if (e >= 8 - over) v.h[e] = 0;
-        rv[j] = v.u4;
-      }
+      st.k[j] = ld16(kb + (((size_t)page * nkv + kvh) * page_size + off + rem / (HD / 8)) * HD + 8 * (rem % (HD / 8)));
+      st.v[j] = ld16(vb + (((size_t)page * nkv + kvh) * HD + rem / 2) * page_size + off + 8 * (rem % 2));
     }
   };
-  auto put = [&](char* buf) __attribute__((always_inline)) {
+  auto put = [&](int i, Stage& st, char* buf) __attribute__((always_inline)) {
+    const bool pooled = i < pt;
+    const int key0 = pooled ? 32 * i : first + 32 * (i - pt), limit = pooled ? nb_max - 1 : p_last;
 #pragma unroll
     for (int j = 0; j < PIECES; ++j) {
       const int piece = tid + j * PF_THREADS;
       if (piece >= 4 * HD) continue;
       const int sb = piece / (2 * HD), rem = piece % (2 * HD);
-      *reinterpret_cast<uint4*>(buf + (16 * sb + rem / (HD / 8)) * KROW + 16 * (rem % (HD / 8))) = rk[j];
+      if (key0 + 31 > limit) {
+        // values of rows behind the data are not to be multiplied, even by zero
+        const int over = key0 + 16 * sb + 8 * (rem % 2) + 7 - limit;                // how many of the eight lie behind
+        Pack8 v;
+        v.u4 = st.v[j];
+#pragma unroll
+        for (int e = 0; e < 8; ++e)
+          if (e >= 8 - over) v.h[e] = 0;
+        st.v[j] = v.u4;
+      }
+      *reinterpret_cast<uint4*>(buf + (16 * sb + rem / (HD / 8)) * KROW + 16 * (rem % (HD / 8))) = st.k[j];
       char* v = buf + KBYTES + (rem / 2) * VROW + 8 * sb + 32 * (rem % 2);
-      *reinterpret_cast<uint2*>(v) = make_uint2(rv[j].x, rv[j].y);
-      *reinterpret_cast<uint2*>(v + 16) = make_uint2(rv[j].z, rv[j].w);
+      *reinterpret_cast<uint2*>(v) = make_uint2(st.v[j].x, st.v[j].y);
+      *reinterpret_cast<uint2*>(v + 16) = make_uint2(st.v[j].z, st.v[j].w);
     }
   };
-  fetch(0);
-  put(lds);
-  __syncthreads();
-  for (int i = 0; i < tiles; ++i) {
-    const char* const buf = lds + (i & 1) * (KBYTES + VBYTES);
-    if (i + 1 < tiles) fetch(i + 1);
-    if (any) {
-      const bool pooled = i < pt;
-      const int key0 = pooled ? 32 * i : first + 32 * (i - pt);
-      const bool whole = pooled ? key0 + 32 <= nb_min : (key0 >= lo_last && key0 + 31 <= p_first);   // every column sees every key
-      Pack8 p[NG];
-      {
-        f32x4_t s[NG][2];
+  auto work = [&](int i, const char* buf) __attribute__((always_inline)) {
+    if (!any) return;
+    const bool pooled = i < pt;
+    const int key0 = pooled ? 32 * i : first + 32 * (i - pt);
+    const bool whole = pooled ? key0 + 32 <= nb_min : (key0 >= lo_last && key0 + 31 <= p_first);   // every column sees every key
+    Pack8 p[NG];
+    {
+      f32x4_t s[NG][2];
 #pragma unroll
-        for (int u = 0; u < NG; ++u) s[u][0] = s[u][1] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+      for (int u = 0; u < NG; ++u) s[u][0] = s[u][1] = f32x4_t{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-        for (int ch = 0; ch < NQK; ++ch)
+      for (int ch = 0; ch < NQK; ++ch)
 #pragma unroll
-          for (int sb = 0; sb < 2; ++sb) {
-            Pack8 k;
-            k.u4 = *reinterpret_cast<const uint4*>(buf + (16 * sb + c) * KROW + 64 * ch + 16 * g);
+        for (int sb = 0; sb < 2; ++sb) {
+          Pack8 k;
+          k.u4 = *reinterpret_cast<const uint4*>(buf + (16 * sb + c) * KROW + 64 * ch + 16 * g);
 #pragma unroll
-            for (int u = 0; u < NG; ++u) s[u][sb] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(k.v, qreg[u][ch].v, s[u][sb], 0, 0, 0);
-          }
+          for (int u = 0; u < NG; ++u) s[u][sb] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(k.v, qreg[u][ch].v, s[u][sb], 0, 0, 0);
+        }
 #pragma unroll
-        for (int u = 0; u < NG; ++u)
+      for (int u = 0; u < NG; ++u)
 #pragma unroll
-          for (int sb = 0; sb < 2; ++sb) {
-            float e[4];
+        for (int sb = 0; sb < 2; ++sb) {
+          float e[4];
+#pragma unroll
+          for (int r = 0; r < 4; ++r) e[r] = key_weight<CAP>(s[u][sb][r], kc[u]);
+          if (!whole) {
 #pragma unroll
             for (int r = 0; r < 4; ++r) {
-              e[r] = key_weight<CAP>(s[u][sb][r], kc[u]);
-              if (!whole) {
-                const int kk = key0 + 16 * sb + 4 * g + r;
-                const bool ok = pooled ? kk < nb[u] : (kk >= lo[u] && kk <= hi[u]);
-                if (!ok) e[r] = 0.f;
-              }
+              const int kk = key0 + 16 * sb + 4 * g + r;
+              const bool ok = pooled ? kk < nb[u] : (kk >= lo[u] && kk <= hi[u]);
+              if (!ok) e[r] = 0.f;
             }
-            p[u].w[2 * sb] = pack2_bf16(e[0], e[1]);
-            p[u].w[2 * sb + 1] = pack2_bf16(e[2], e[3]);
           }
-      }
-#pragma unroll
-      for (int n = 0; n < 2 * NQK; ++n) {
-        Pack8 v;
-        v.u4 = *reinterpret_cast<const uint4*>(buf + KBYTES + (16 * n + c) * VROW + 16 * g);
-#pragma unroll
-        for (int u = 0; u < NG; ++u) acc[u][n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(v.v, p[u].v, acc[u][n], 0, 0, 0);
-      }
+          p[u].w[2 * sb] = pack2_bf16(e[0], e[1]);
+          p[u].w[2 * sb + 1] = pack2_bf16(e[2], e[3]);
+        }
     }
-    if (i + 1 < tiles) put(lds + ((i + 1) & 1) * (KBYTES + VBYTES));
-    __syncthreads();
+#pragma unroll
+    for (int n = 0; n < 2 * NQK; ++n) {
+      Pack8 v;
+      v.u4 = *reinterpret_cast<const uint4*>(buf + KBYTES + (16 * n + c) * VROW + 16 * g);
+#pragma unroll
+      for (int u = 0; u < NG; ++u) acc[u][n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(v.v, p[u].v, acc[u][n], 0, 0, 0);
+    }
+  };
+  char* const buf0 = lds;
+  char* const buf1 = lds + KBYTES + VBYTES;
+  Stage s0, s1;
+  fetch(0, s0);
+  if (tiles > 1) fetch(1, s1);
+  put(0, s0, buf0);
+  lds_barrier();
+  for (int i = 0; i < tiles; i += 2) {
+    if (i + 2 < tiles) fetch(i + 2, s0);
+    work(i, buf0);
+    if (i + 1 >= tiles) break;
+    put(i + 1, s1, buf1);
+    lds_barrier();
+    if (i + 3 < tiles) fetch(i + 3, s1);
+    work(i + 1, buf1);
+    if (i + 2 >= tiles) break;
+    put(i + 2, s0, buf0);
+    lds_barrier();
   }
 #pragma unroll
   for (int u = 0; u < NG; ++u) {

@@ -141,6 +141,36 @@ extern "C" int ullm_zero_fresh_rows(void* state, long long row_bytes, int n_rows
   ULLM_LAUNCH_CHECK();
 }
 
+// The same for many states at once: table [n_states][2] = (address, bytes of a row).  grid (entries, states, pieces of a
+// row); rows are cleared 16 bytes at a time as far as their size and address allow, else 4, else 1.
+__global__ void __launch_bounds__(256)
+zero_fresh_many_kernel(const long long* __restrict__ table, int n_rows, const int* __restrict__ slot, const int* __restrict__ start) {
+  const int b = blockIdx.x;
+  if (start[b] != 0) return;
+  const int row = slot[b];
+  if (row < 0 || row >= n_rows) return;
+  const long long bytes = table[2 * blockIdx.y + 1];
+  unsigned char* p = reinterpret_cast<unsigned char*>(table[2 * blockIdx.y]) + (size_t)row * bytes;
+  const long long at = (long long)blockIdx.z * 256 + threadIdx.x, step = (long long)gridDim.z * 256;
+  if (((uintptr_t)p & 15) == 0 && bytes % 16 == 0) {
+    for (long long i = at; i < bytes / 16; i += step) reinterpret_cast<uint4*>(p)[i] = make_uint4(0, 0, 0, 0);
+  } else if (((uintptr_t)p & 3) == 0 && bytes % 4 == 0) {
+    for (long long i = at; i < bytes / 4; i += step) reinterpret_cast<uint32_t*>(p)[i] = 0;
+  } else {
+    for (long long i = at; i < bytes; i += step) p[i] = 0;
+  }
+}
+
+extern "C" int ullm_zero_fresh_many(const long long* table, int n_states, long long most_bytes, int n_rows, const int* slot,
+                                    const int* start, int n_entries, hipStream_t stream) {
+  if (n_entries <= 0 || n_states <= 0) return 0;
+  if (n_rows <= 0 || n_states > 65535) return ULLM_ERR_SHAPE;
+  long long pieces = (most_bytes / 16 + 255) / 256;
+  pieces = pieces < 1 ? 1 : pieces > 16 ? 16 : pieces;
+  hipLaunchKernelGGL(zero_fresh_many_kernel, dim3(n_entries, n_states, (unsigned)pieces), dim3(256), 0, stream, table, n_rows, slot, start);
+  ULLM_LAUNCH_CHECK();
+}
+
 // out[i, :] = src[index[i], :] for float32 rows (an index outside [0, n_src) gives a row of zeros).
 // grid (rows, pieces of a row).
 __global__ void gather_rows_kernel(const float* __restrict__ src, long long src_stride, int n_src,

@@ -64,64 +64,82 @@ __device__ __forceinline__ void write_block_mean(int block, int pool, const int*
   const float inv = 1.f / (float)pool;
   for (int d = tid; d < hd; d += nthreads) {
     float ks = 0.f, vs = 0.f;
-    for (int j = 0; j < pool; ++j) {
-      const int pos = block * pool + j, page = bt[pos / page_size], off = pos % page_size;
-      if (page < 0) continue;                                       // never: a block's tokens are held until it is complete
-      ks += ld_f32(k_pool + (((size_t)page * nkv + kvh) * page_size + off) * hd + d);
-      vs += ld_f32(v_pool + (((size_t)page * nkv + kvh) * hd + d) * page_size + off);
+    for (int j0 = 0; j0 < pool; j0 += 8) {                            // eight rows under way; added in order
+      float kv[8], vv[8];
+#pragma unroll
+      for (int u = 0; u < 8; ++u) {
+        const int pos = block * pool + (j0 + u < pool ? j0 + u : pool - 1), off = pos % page_size;
+        const int page = max(bt[pos / page_size], 0);                 // (a block's tokens are held until it is complete)
+        kv[u] = ld_f32(k_pool + (((size_t)page * nkv + kvh) * page_size + off) * hd + d);
+        vv[u] = ld_f32(v_pool + (((size_t)page * nkv + kvh) * hd + d) * page_size + off);
+      }
+#pragma unroll
+      for (int u = 0; u < 8; ++u)
+        if (j0 + u < pool) ks += kv[u], vs += vv[u];
     }
     st_f32(pk_pool + (((size_t)to * nkv + kvh) * page_size + slot) * hd + d, ks * inv);
     st_f32(pv_pool + (((size_t)to * nkv + kvh) * hd + d) * page_size + slot, vs * inv);
   }
 }
 
-// One block of threads per run of `tok` tokens.  A row of `proj` is q | k | v, (nq + 2 nkv) * hd = C values; weights lie
-// tap by tap [taps, C]; the entry's state row holds the last taps-1 rows before the step, oldest first.  A thread owns
-// PIECES pieces of V neighbouring channels and keeps their last inputs in registers along the run.  `single`: every
-// entry brings one token: the thread moves its channels' state on itself, and a token that completes a block of `pool`
-// tokens (pool > 0) leaves that block's mean behind.
-template <typename T, int TAPS, int V, int PIECES>
+// One block of threads per run of RUN tokens.  A row of `proj` is q | k | v, (nq + 2 nkv) * hd = C values; weights lie tap
+// by tap [taps, C]; the entry's state row holds the last taps-1 rows before the step, oldest first.  A thread owns PIECES
+// pieces of V neighbouring channels: the run's rows are all asked for at once, and the last inputs stay in registers
+// along the run.  Where the run's tokens lie side by side in a page, a channel's four values go out in one store.
+// `single`: every entry brings one token: the thread moves its channels' state on itself, and a token that completes a
+// block of `pool` tokens (pool > 0) leaves that block's mean behind.
+template <typename T, int TAPS, int V, int PIECES, int RUN>
 __global__ void __launch_bounds__(1024)
 conv_norm_write_kernel(const T* __restrict__ proj, int ld, const float* __restrict__ w, int taps_rt, float* __restrict__ carry,
                        long long carry_stride, const float* __restrict__ q_gain, const float* __restrict__ k_gain, float eps,
                        float q_count, float k_count, const int* __restrict__ positions, const int* __restrict__ token_entry,
                        const int* __restrict__ q_start, const int* __restrict__ entry_slot, const int* __restrict__ block_table,
                        int bt_stride, T* __restrict__ q_out, T* k_pool, T* v_pool, int page_size, int nq, int nkv, int hd,
-                       int T_, int tok, int single, int pool, const int* __restrict__ pooled_table, int pooled_stride,
+                       int T_, int single, int pool, const int* __restrict__ pooled_table, int pooled_stride,
                        T* pk_pool, T* pv_pool) {
-  __shared__ float scratch[32];
+  __shared__ float scratch[2][32];
   const int C = (nq + 2 * nkv) * hd, nqv = nq * hd, nkvv = nkv * hd, tid = threadIdx.x, nthreads = blockDim.x;
   constexpr int HT = TAPS > 0 ? TAPS : 1;
   const int taps = TAPS > 0 ? TAPS : taps_rt;
-  float wt[PIECES][HT][V], hist[PIECES][HT][V];
-  if constexpr (TAPS > 0) {
+  const int t0 = blockIdx.x * RUN;
+  float wt[PIECES][HT][V], hist[PIECES][HT][V], y[PIECES][RUN][V], gain[PIECES][V];
+  int ent[RUN], pos[RUN], page[RUN];
 #pragma unroll
-    for (int p = 0; p < PIECES; ++p) {
-      const int c = V * (tid + p * nthreads);
-#pragma unroll
-      for (int j = 0; j < TAPS; ++j) {
-        if (c < C) cnw_load<float, V>(w + (size_t)j * C + c, wt[p][j]);
-        else
-#pragma unroll
-          for (int u = 0; u < V; ++u) wt[p][j][u] = 0.f, hist[p][j][u] = 0.f;
-      }
-    }
+  for (int r = 0; r < RUN; ++r) {
+    const int t = t0 + r < T_ ? t0 + r : T_ - 1;
+    ent[r] = token_entry[t];
+    pos[r] = positions[t];
+    page[r] = block_table[(size_t)ent[r] * bt_stride + pos[r] / page_size];
   }
-  const int t0 = blockIdx.x * tok;
-  for (int t = t0; t < t0 + tok && t < T_; ++t) {
-    const int b = token_entry[t], first = q_start[b], i = t - first, pos = positions[t];
-    const int page = block_table[(size_t)b * bt_stride + pos / page_size];
+#pragma unroll
+  for (int p = 0; p < PIECES; ++p) {
+    const int c = V * (tid + p * nthreads);
+    if (c >= C) continue;
+    if constexpr (TAPS > 0) {
+#pragma unroll
+      for (int r = 0; r < RUN; ++r) cnw_load<T, V>(proj + (size_t)(t0 + r < T_ ? t0 + r : T_ - 1) * ld + c, y[p][r]);
+#pragma unroll
+      for (int j = 0; j < TAPS; ++j) cnw_load<float, V>(w + (size_t)j * C + c, wt[p][j]);
+    }
+    if (c < nqv + nkvv) cnw_load<float, V>(c < nqv ? q_gain + c : k_gain + (c - nqv), gain[p]);
+  }
+  const bool side_by_side = RUN == 4 && t0 + RUN <= T_ && ent[0] == ent[RUN - 1] && pos[0] % 4 == 0 && page_size % 4 == 0 && page[0] >= 0;
+#pragma unroll
+  for (int r = 0; r < RUN; ++r) {
+    const int t = t0 + r;
+    if (t >= T_) break;
+    const int b = ent[r], first = q_start[b], i = t - first;
     float* old = carry + (size_t)entry_slot[b] * carry_stride;
-    float y[PIECES][V];
     float ssq = 0.f, ssk = 0.f;
 #pragma unroll
     for (int p = 0; p < PIECES; ++p) {
       const int c = V * (tid + p * nthreads);
-#pragma unroll
-      for (int u = 0; u < V; ++u) y[p][u] = 0.f;
       if (c >= C) continue;
+      float out[V];
+#pragma unroll
+      for (int u = 0; u < V; ++u) out[u] = 0.f;
       if constexpr (TAPS > 0) {
-        if (t == t0 || i == 0) {
+        if (r == 0 || i == 0) {
 #pragma unroll
           for (int k = 0; k < TAPS - 1; ++k) {
             const int l = i - (TAPS - 1) + k;
@@ -129,11 +147,12 @@ conv_norm_write_kernel(const T* __restrict__ proj, int ld, const float* __restri
             else cnw_load<float, V>(old + (size_t)(l + TAPS - 1) * C + c, hist[p][k]);
           }
         }
-        cnw_load<T, V>(proj + (size_t)t * ld + c, hist[p][TAPS - 1]);
+#pragma unroll
+        for (int u = 0; u < V; ++u) hist[p][TAPS - 1][u] = y[p][r][u];
 #pragma unroll
         for (int j = 0; j < TAPS; ++j)
 #pragma unroll
-          for (int u = 0; u < V; ++u) y[p][u] += wt[p][j][u] * hist[p][j][u];
+          for (int u = 0; u < V; ++u) out[u] += wt[p][j][u] * hist[p][j][u];
         if (single) {
 #pragma unroll
           for (int k = 0; k < TAPS - 1; ++k) cnw_store<float, V>(old + (size_t)k * C + c, hist[p][k + 1]);
@@ -150,18 +169,19 @@ conv_norm_write_kernel(const T* __restrict__ proj, int ld, const float* __restri
           else cnw_load<float, V>(old + (size_t)(l + taps - 1) * C + c, in);
           cnw_load<float, V>(w + (size_t)j * C + c, ww);
 #pragma unroll
-          for (int u = 0; u < V; ++u) y[p][u] += ww[u] * in[u];
+          for (int u = 0; u < V; ++u) out[u] += ww[u] * in[u];
         }
       }
 #pragma unroll
       for (int u = 0; u < V; ++u) {
-        if (c < nqv) ssq += y[p][u] * y[p][u];
-        else if (c < nqv + nkvv) ssk += y[p][u] * y[p][u];
+        y[p][r][u] = out[u];
+        if (c < nqv) ssq += out[u] * out[u];
+        else if (c < nqv + nkvv) ssk += out[u] * out[u];
       }
     }
-    cnw_block_sum2(ssq, ssk, scratch);
+    cnw_block_sum2(ssq, ssk, scratch[r & 1]);
     const float rsq = 1.f / sqrtf(ssq / q_count + eps), rsk = 1.f / sqrtf(ssk / k_count + eps);
-    const int slot = pos % page_size;
+    const int slot = pos[r] % page_size;
 #pragma unroll
     for (int p = 0; p < PIECES; ++p) {
       const int c = V * (tid + p * nthreads);
@@ -169,28 +189,45 @@ conv_norm_write_kernel(const T* __restrict__ proj, int ld, const float* __restri
       if (c < nqv) {
         float o[V];
 #pragma unroll
-        for (int u = 0; u < V; ++u) o[u] = (y[p][u] * rsq) * q_gain[c + u];
+        for (int u = 0; u < V; ++u) o[u] = (y[p][r][u] * rsq) * gain[p][u];
         cnw_store<T, V>(q_out + (size_t)t * nqv + c, o);
-      } else if (page >= 0 && c < nqv + nkvv) {
+      } else if (page[r] >= 0 && c < nqv + nkvv) {
         const int kc = c - nqv, kvh = kc / hd, d = kc % hd;
         float o[V];
 #pragma unroll
-        for (int u = 0; u < V; ++u) o[u] = (y[p][u] * rsk) * k_gain[kc + u];
-        cnw_store<T, V>(k_pool + (((size_t)page * nkv + kvh) * page_size + slot) * hd + d, o);
-      } else if (page >= 0) {
+        for (int u = 0; u < V; ++u) o[u] = (y[p][r][u] * rsk) * gain[p][u];
+        cnw_store<T, V>(k_pool + (((size_t)page[r] * nkv + kvh) * page_size + slot) * hd + d, o);
+      } else if (page[r] >= 0 && !side_by_side) {
         const int vc = c - nqv - nkvv, kvh = vc / hd, d = vc % hd;
-        T* dst = v_pool + (((size_t)page * nkv + kvh) * hd + d) * page_size + slot;
+        T* dst = v_pool + (((size_t)page[r] * nkv + kvh) * hd + d) * page_size + slot;
 #pragma unroll
-        for (int u = 0; u < V; ++u) st_f32(dst + (size_t)u * page_size, y[p][u]);
+        for (int u = 0; u < V; ++u) st_f32(dst + (size_t)u * page_size, y[p][r][u]);
       }
     }
-    if (single && pool > 0 && page >= 0 && (pos + 1) % pool == 0) {
+    if (single && pool > 0 && page[r] >= 0 && (pos[r] + 1) % pool == 0) {
       __threadfence_block();
       __syncthreads();                                      // the block's own stores of this token's key and value
       const int lane = tid & 63, wave = tid / 64, nwaves = nthreads / 64;
       for (int kvh = wave; kvh < nkv; kvh += nwaves)
-        write_block_mean<T>(pos / pool, pool, block_table + (size_t)b * bt_stride, pooled_table + (size_t)b * pooled_stride,
+        write_block_mean<T>(pos[r] / pool, pool, block_table + (size_t)b * bt_stride, pooled_table + (size_t)b * pooled_stride,
                             k_pool, v_pool, pk_pool, pv_pool, page_size, nkv, hd, kvh, lane, 64);
+    }
+  }
+  if constexpr (RUN == 4) {
+    if (!side_by_side) return;
+#pragma unroll
+    for (int p = 0; p < PIECES; ++p) {
+      const int c = V * (tid + p * nthreads);
+      if (c >= C || c < nqv + nkvv) continue;
+      const int vc = c - nqv - nkvv, kvh = vc / hd, d = vc % hd;
+      T* dst = v_pool + (((size_t)page[0] * nkv + kvh) * hd + d) * page_size + pos[0] % page_size;
+#pragma unroll
+      for (int u = 0; u < V; ++u) {
+        float o[4];
+#pragma unroll
+        for (int r = 0; r < 4; ++r) o[r] = y[p][r < RUN ? r : 0][u];
+        cnw_store<T, 4>(dst + (size_t)u * page_size, o);
+      }
     }
   }
 }
@@ -210,18 +247,19 @@ extern "C" int ullm_conv_norm_write(const void* proj, int ld, const float* w, in
   if (pool > 0 && single && (!pooled_table || !pk_pool || !pv_pool)) return ULLM_ERR_UNSUPPORTED;
   const size_t item = dtype == ULLM_F32 ? 4 : 2;
   const bool by4 = hd % 4 == 0 && ld % 4 == 0 && carry_stride % 4 == 0 && (uintptr_t)proj % (4 * item) == 0 &&
-                   (uintptr_t)carry % 16 == 0 && (uintptr_t)w % 16 == 0;
+                   (uintptr_t)carry % 16 == 0 && ((uintptr_t)w | (uintptr_t)q_gain | (uintptr_t)k_gain) % 16 == 0;
   const int pieces_all = by4 ? C / 4 : C;
   int pieces = 1;
   while (pieces * 1024 < pieces_all) pieces *= 2;
   if (pieces > 16) return ULLM_ERR_SHAPE;                    // rows of up to 65536 values (16384 where not by fours)
   const int threads = ((pieces_all + pieces - 1) / pieces + 63) / 64 * 64;
-  const int tok = single || T_ < 512 ? 1 : 4;
-#define GO(TT, TAPS, V, P) hipLaunchKernelGGL((conv_norm_write_kernel<TT, TAPS, V, P>), dim3((T_ + tok - 1) / tok), dim3(threads), 0, \
+  const bool runs = !single && T_ >= 512;
+#define GO_R(TT, TAPS, V, P, R) hipLaunchKernelGGL((conv_norm_write_kernel<TT, TAPS, V, P, R>), dim3((T_ + R - 1) / R), dim3(threads), 0, \
     stream, (const TT*)proj, ld, w, taps, carry, carry_stride, q_gain, k_gain, eps, q_count, k_count, positions, token_entry,        \
-    q_start, entry_slot, block_table, bt_stride, (TT*)q_out, (TT*)k_pool, (TT*)v_pool, page_size, nq, nkv, hd, T_, tok, single,      \
+    q_start, entry_slot, block_table, bt_stride, (TT*)q_out, (TT*)k_pool, (TT*)v_pool, page_size, nq, nkv, hd, T_, single,           \
     pool, pooled_table, pooled_stride, (TT*)pk_pool, (TT*)pv_pool)
-#define GO_P(TT, TAPS, V) do { if (pieces == 1) GO(TT, TAPS, V, 1); else if (pieces == 2) GO(TT, TAPS, V, 2); \
+#define GO(TT, TAPS, V, P) GO_R(TT, TAPS, V, P, 1)
+#define GO_P(TT, TAPS, V) do { if (pieces == 1 && runs && V == 4) GO_R(TT, TAPS, V, 1, 4); else if (pieces == 1) GO(TT, TAPS, V, 1); else if (pieces == 2) GO(TT, TAPS, V, 2); \
     else if (pieces == 4) GO(TT, TAPS, V, 4); else if (pieces == 8) GO(TT, 0, V, 8); else GO(TT, 0, V, 16); } while (0)
   // up to 4 taps with up to 4 pieces a thread the inputs are kept in registers; else every tap is read where it lies,
   // and the state is moved on by a kernel of its own
@@ -238,6 +276,7 @@ extern "C" int ullm_conv_norm_write(const void* proj, int ld, const float* w, in
 #undef GO_T
 #undef GO_P
 #undef GO
+#undef GO_R
   const bool moved = single && by4 && taps >= 2 && taps <= 4 && pieces <= 4;
   if (taps > 1 && !moved) {
     if (dtype == ULLM_F32) launch_carry<float>(proj, ld, carry, carry_stride, q_start, entry_slot, B_, C, taps, stream);

@@ -48,7 +48,8 @@ struct PostConv {
 };
 
 // One block per token; a thread owns K pieces of V neighbouring values.
-template <typename TA, typename TB, typename TO, int V, int K>
+// TAPS: the convolution's taps (0: none, or read one after the other).
+template <typename TA, typename TB, typename TO, int V, int K, int TAPS>
 __global__ void __launch_bounds__(256)
 post_add_kernel(const TA* __restrict__ branch, int n_a, const TB* __restrict__ second, int n_b, float a, float b,
                 const float* __restrict__ gain, float eps, float* __restrict__ stream_rows, TO* __restrict__ out, int T_, int H,
@@ -56,13 +57,22 @@ post_add_kernel(const TA* __restrict__ branch, int n_a, const TB* __restrict__ s
   __shared__ float scratch[16];
   const int t = blockIdx.x, tid = threadIdx.x;
   const size_t row = (size_t)t * H, slice = (size_t)T_ * H;
-  float y[K][V], x[K][V];
+  constexpr int HT = TAPS > 1 ? TAPS - 1 : 1, WT = TAPS > 0 ? TAPS : 1;
+  float y[K][V], x[K][V], g[K][V], past[K][HT][V], w[K][WT][V];
+  float* old = conv.w ? conv.carry + (size_t)conv.entry_slot[t] * conv.carry_stride : nullptr;
   float ss = 0.f;
 #pragma unroll
   for (int k = 0; k < K; ++k) {
     const int c = V * (tid + 256 * k);
     if (c < H) {
       post_load<V>(stream_rows + row + c, x[k]);
+      post_load<V>(gain + c, g[k]);
+      if constexpr (TAPS > 0) {
+#pragma unroll
+        for (int j = 0; j < TAPS - 1; ++j) post_load<V>(old + (size_t)j * H + c, past[k][j]);
+#pragma unroll
+        for (int j = 0; j < TAPS; ++j) post_load<V>(conv.w + (size_t)j * H + c, w[k][j]);
+      }
       float v[V];
       post_load<V>(branch + row + c, y[k]);
       for (int s = 1; s < n_a; ++s) {
@@ -88,35 +98,46 @@ post_add_kernel(const TA* __restrict__ branch, int n_a, const TB* __restrict__ s
     }
   }
   const float rs = 1.f / sqrtf(block_sum(ss, scratch) / (float)H + eps);
-  float* old = conv.w ? conv.carry + (size_t)conv.entry_slot[t] * conv.carry_stride : nullptr;
 #pragma unroll
   for (int k = 0; k < K; ++k) {
     const int c = V * (tid + 256 * k);
     if (c >= H) continue;
-    float g[V];
-    post_load<V>(gain + c, g);
 #pragma unroll
-    for (int u = 0; u < V; ++u) x[k][u] += (y[k][u] * rs) * g[u];
+    for (int u = 0; u < V; ++u) x[k][u] += (y[k][u] * rs) * g[k][u];
     post_store<V>(stream_rows + row + c, x[k]);
     if (!out) continue;
     if (!conv.w) {
       post_store<V>(out + row + c, x[k]);
       continue;
     }
-    float acc[V], in[V], w[V];
+    float acc[V];
 #pragma unroll
     for (int u = 0; u < V; ++u) acc[u] = 0.f;
+    if constexpr (TAPS > 0) {
+#pragma unroll
+      for (int j = 0; j < TAPS - 1; ++j) {
+        if (j > 0) post_store<V>(old + (size_t)(j - 1) * H + c, past[k][j]);
+#pragma unroll
+        for (int u = 0; u < V; ++u) acc[u] += w[k][j][u] * past[k][j][u];
+      }
+      if (TAPS > 1) post_store<V>(old + (size_t)(TAPS - 2) * H + c, x[k]);
+#pragma unroll
+      for (int u = 0; u < V; ++u) acc[u] = x[k][u] + (acc[u] + w[k][TAPS - 1][u] * x[k][u]);
+      post_store<V>(out + row + c, acc);
+      continue;
+    }
+    float in[V], wj[V];
     for (int j = 0; j < conv.taps - 1; ++j) {
       post_load<V>(old + (size_t)j * H + c, in);
-      post_load<V>(conv.w + (size_t)j * H + c, w);
+      post_load<V>(conv.w + (size_t)j * H + c, wj);
       if (j > 0) post_store<V>(old + (size_t)(j - 1) * H + c, in);          // the state moves up by one
 #pragma unroll
-      for (int u = 0; u < V; ++u) acc[u] += w[u] * in[u];
+      for (int u = 0; u < V; ++u) acc[u] += wj[u] * in[u];
     }
-    post_load<V>(conv.w + (size_t)(conv.taps - 1) * H + c, w);
+    post_load<V>(conv.w + (size_t)(conv.taps - 1) * H + c, wj);
     if (conv.taps > 1) post_store<V>(old + (size_t)(conv.taps - 2) * H + c, x[k]);
 #pragma unroll
-    for (int u = 0; u < V; ++u) acc[u] = x[k][u] + (acc[u] + w[u] * x[k][u]);
+    for (int u = 0; u < V; ++u) acc[u] = x[k][u] + (acc[u] + wj[u] * x[k][u]);
     post_store<V>(out + row + c, acc);
   }
 }
@@ -128,14 +149,19 @@ static int launch_post(const void* branch, int n_a, const void* second, int n_b,
                    (uintptr_t)out % (4 * sizeof(TO)) == 0 && ((uintptr_t)gain | (uintptr_t)stream_rows) % 16 == 0 &&
                    (!conv.w || ((uintptr_t)conv.w | (uintptr_t)conv.carry) % 16 == 0) && (!conv.w || conv.carry_stride % 4 == 0);
   const int pieces = ((by4 ? H / 4 : H) + 255) / 256;
-#define GO(V, K) hipLaunchKernelGGL((post_add_kernel<TA, TB, TO, V, K>), dim3(T_), dim3(256), 0, stream, (const TA*)branch, n_a, \
+#define GO_T(V, K, TAPS) hipLaunchKernelGGL((post_add_kernel<TA, TB, TO, V, K, TAPS>), dim3(T_), dim3(256), 0, stream, (const TA*)branch, n_a, \
     (const TB*)second, n_b, a, b, gain, eps, stream_rows, (TO*)out, T_, H, conv)
+  // rows of up to 4096 values by fours with two to four taps: the convolution's operands wait in registers
+#define GO(V, K) do { if constexpr (V == 4 && K <= 4) {                                                                   \
+    if (conv.w && conv.taps == 2) GO_T(V, K, 2); else if (conv.w && conv.taps == 3) GO_T(V, K, 3);                          \
+    else if (conv.w && conv.taps == 4) GO_T(V, K, 4); else GO_T(V, K, 0); } else GO_T(V, K, 0); } while (0)
 #define GO_K(V) do { if (pieces <= 1) GO(V, 1); else if (pieces <= 2) GO(V, 2); else if (pieces <= 4) GO(V, 4); else if (pieces <= 8) GO(V, 8); \
     else if (pieces <= 16) GO(V, 16); else return ULLM_ERR_SHAPE; } while (0)
   if (by4) GO_K(4);
   else GO_K(1);
 #undef GO_K
 #undef GO
+#undef GO_T
   ULLM_LAUNCH_CHECK();
 }
 

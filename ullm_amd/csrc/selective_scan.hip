@@ -4,7 +4,7 @@
 //   y[t, c] = sum_n S[c, n] * C[t, n] + D[c] * x[t, c],   stored: y * silu(z[t, c])
 // A is handed over as A * log2(e), so that a decay is one exponent of two.  The states are float32 and come from and
 // go to the entry's state row (state[slot, off + c * N + n]).  Everything is 32-bit; x, z and the result are stored in
-// the compute dtype.
+// the compute dtype (B and C too: they are a projection's values).
 //
 // Three ways, by what the step holds:
 //   portions of prompts, N <= 64   an entry's tokens are cut into segments ("items") that are walked side by side.  Over a
@@ -26,10 +26,11 @@ __device__ __forceinline__ float sel_softplus(float v) {
   return fmaxf(v, 0.f) + l;
 }
 
+template <typename T>
 struct ScanIn {
   const float* raw;           // [T, raw_ld]
   int raw_ld;
-  const float* bc;            // [T, bc_ld]: B, then C
+  const T* bc;                // [T, bc_ld]: B, then C
   int bc_ld;
   const float* a_log2;        // [inner, N]
   const float* dt_bias;
@@ -42,10 +43,26 @@ struct ScanIn {
 // state row), 1 one of several (its first states lie in `chain`), 2 the last of several (and its last states go to the
 // state row).  chain float32 [n][N][inner], dt_sum float32 [n][inner].
 #define SEG_AHEAD 8            // tokens whose step sizes and inputs are under way
-// FULL: the model has N states a channel, not fewer (then a token's B and C are whole wide scalar loads).
+// A token's N values of B (or C), the same address for the whole wave: whole words, so that they are wide scalar loads.
+template <int N>
+__device__ __forceinline__ void uniform_row(const float* p, float (&v)[N]) {
+#pragma unroll
+  for (int n = 0; n < N; ++n) v[n] = p[n];
+}
+template <int N>
+__device__ __forceinline__ void uniform_row(const bf16_t* p, float (&v)[N]) {
+  const uint32_t* w = reinterpret_cast<const uint32_t*>(p);
+#pragma unroll
+  for (int n = 0; n < N / 2; ++n) {
+    v[2 * n] = __uint_as_float(w[n] << 16);
+    v[2 * n + 1] = __uint_as_float(w[n] & 0xffff0000u);
+  }
+}
+
+// FULL: the model has N states a channel, not fewer, and its rows of B and C are whole aligned words.
 template <typename T, int N, bool OUT, bool FULL>
 __global__ void __launch_bounds__(64)
-scan_segment_kernel(const T* __restrict__ x, int x_ld, const T* __restrict__ z, int z_ld, ScanIn in, const int* __restrict__ items,
+scan_segment_kernel(const T* __restrict__ x, int x_ld, const T* __restrict__ z, int z_ld, ScanIn<T> in, const int* __restrict__ items,
                     float* __restrict__ chain, float* __restrict__ dt_sum, float* __restrict__ state, long long state_stride,
                     long long state_off, const int* __restrict__ entry_slot, T* __restrict__ out, int write_state) {
   const int item = blockIdx.y, what = items[4 * item + 3];
@@ -94,14 +111,25 @@ scan_segment_kernel(const T* __restrict__ x, int x_ld, const T* __restrict__ z, 
 #pragma unroll
     for (int u = 0; u < SEG_AHEAD; ++u) {
       const int tt = t + u < n_tok ? t + u : n_tok - 1;
-      const float* const bcr = in.bc + (size_t)(t0 + tt) * in.bc_ld;
+      const T* const bcr = in.bc + (size_t)(t0 + tt) * in.bc_ld;
       const float dx = dt[u] * xv[u];
       float acc = 0.f;
+      if constexpr (FULL) {
+        float bv[N], cv[N];
+        uniform_row<N>(bcr, bv);
+        if (OUT) uniform_row<N>(bcr + N, cv);
 #pragma unroll
-      for (int n = 0; n < N; ++n) {
-        const int nn = n < n_states ? n : n_states - 1;   // states behind the last: no decay (a = 0), never stored
-        s[n] = __builtin_amdgcn_exp2f(dt[u] * a[n]) * s[n] + dx * bcr[nn];
-        if (OUT) acc += n < n_states ? s[n] * bcr[n_states + nn] : 0.f;
+        for (int n = 0; n < N; ++n) {
+          s[n] = __builtin_amdgcn_exp2f(dt[u] * a[n]) * s[n] + dx * bv[n];
+          if (OUT) acc += s[n] * cv[n];
+        }
+      } else {
+#pragma unroll
+        for (int n = 0; n < N; ++n) {
+          const int nn = n < n_states ? n : n_states - 1;   // states behind the last: no decay (a = 0), never stored
+          s[n] = __builtin_amdgcn_exp2f(dt[u] * a[n]) * s[n] + dx * ld_f32(bcr + nn);
+          if (OUT) acc += n < n_states ? s[n] * ld_f32(bcr + n_states + nn) : 0.f;
+        }
       }
       if (OUT) {
         if (t + u < n_tok && live) st_f32(out + (size_t)(t0 + t + u) * in.inner + c, (acc + skip * xv[u]) * sel_silu(zv[u]));
@@ -154,7 +182,7 @@ scan_chain_kernel(const int* __restrict__ chains, float* __restrict__ chain, con
   }
 }
 
-extern "C" int ullm_selective_scan_segments(const void* x, int x_ld, const float* raw, int raw_ld, const float* bc, int bc_ld,
+extern "C" int ullm_selective_scan_segments(const void* x, int x_ld, const float* raw, int raw_ld, const void* bc, int bc_ld,
                                             const void* z, int z_ld, const float* a_log2, const float* dt_bias,
                                             const float* d_skip, float* state, long long state_stride, long long state_off,
                                             const int* entry_slot, const int* items, int n_items, const int* chains, int n_chains,
@@ -164,11 +192,12 @@ extern "C" int ullm_selective_scan_segments(const void* x, int x_ld, const float
   if (n_items > 65535 || n_chains > 65535 || inner < 1 || N < 1 || N > 64 || x_ld < inner || raw_ld < inner || z_ld < inner ||
       bc_ld < 2 * N || (n_chains > 0 && (!chain || !dt_sum)))
     return ULLM_ERR_SHAPE;
-  const ScanIn in = {raw, raw_ld, bc, bc_ld, a_log2, dt_bias, d_skip, inner, N};
+  const bool words = dtype == ULLM_F32 || (bc_ld % 2 == 0 && (uintptr_t)bc % 4 == 0);
   const dim3 grid((inner + 63) / 64, n_items), block(64);
+#define SCAN_IN(TT) ScanIn<TT>{raw, raw_ld, (const TT*)bc, bc_ld, a_log2, dt_bias, d_skip, inner, N}
 #define GO_F(TT, NN, OUT, FULL) hipLaunchKernelGGL((scan_segment_kernel<TT, NN, OUT, FULL>), grid, block, 0, stream, (const TT*)x, x_ld, (const TT*)z, z_ld, \
-    in, items, chain, dt_sum, state, state_stride, state_off, entry_slot, (TT*)out, write_state)
-#define GO(TT, NN, OUT) do { if (N == NN) GO_F(TT, NN, OUT, true); else GO_F(TT, NN, OUT, false); } while (0)
+    SCAN_IN(TT), items, chain, dt_sum, state, state_stride, state_off, entry_slot, (TT*)out, write_state)
+#define GO(TT, NN, OUT) do { if (N == NN && words) GO_F(TT, NN, OUT, true); else GO_F(TT, NN, OUT, false); } while (0)
 #define GO_N(TT, OUT) do { if (N <= 8) GO(TT, 8, OUT); else if (N <= 16) GO(TT, 16, OUT); else if (N <= 32) GO(TT, 32, OUT); else GO(TT, 64, OUT); } while (0)
 #define GO_T(OUT) do { if (dtype == ULLM_F32) GO_N(float, OUT); else if (dtype == ULLM_BF16) GO_N(bf16_t, OUT); else return ULLM_ERR_DTYPE; } while (0)
   if (n_chains > 0) {
@@ -188,7 +217,7 @@ extern "C" int ullm_selective_scan_segments(const void* x, int x_ld, const float
 // `lanes` neighbouring lanes (a power of two, at most 64) share a channel and take its states V at a time.
 template <typename T, int V>
 __global__ void __launch_bounds__(256)
-scan_step_kernel(const T* __restrict__ x, int x_ld, const T* __restrict__ z, int z_ld, ScanIn in, float* __restrict__ state,
+scan_step_kernel(const T* __restrict__ x, int x_ld, const T* __restrict__ z, int z_ld, ScanIn<T> in, float* __restrict__ state,
                  long long state_stride, long long state_off, const int* __restrict__ entry_slot, T* __restrict__ out, int lanes,
                  int write_state) {
   const int t = blockIdx.y, ln = threadIdx.x & (lanes - 1), c = blockIdx.x * (256 / lanes) + threadIdx.x / lanes;
@@ -196,7 +225,7 @@ scan_step_kernel(const T* __restrict__ x, int x_ld, const T* __restrict__ z, int
   const int cc = live ? c : in.inner - 1;
   float* const row = state + (size_t)entry_slot[t] * state_stride + state_off + (size_t)cc * in.N;
   const float* const a = in.a_log2 + (size_t)cc * in.N;
-  const float* const bcr = in.bc + (size_t)t * in.bc_ld;
+  const T* const bcr = in.bc + (size_t)t * in.bc_ld;
   const float xv = ld_f32(x + (size_t)t * x_ld + cc), zv = ld_f32(z + (size_t)t * z_ld + cc);
   const float dt = sel_softplus(in.raw[(size_t)t * in.raw_ld + cc] + in.dt_bias[cc]), dx = dt * xv;
   float acc = 0.f;
@@ -204,19 +233,19 @@ scan_step_kernel(const T* __restrict__ x, int x_ld, const T* __restrict__ z, int
     if constexpr (V == 4) {
       float4 s = *reinterpret_cast<const float4*>(row + n);
       const float4 av = *reinterpret_cast<const float4*>(a + n);
-      s.x = __builtin_amdgcn_exp2f(dt * av.x) * s.x + dx * bcr[n];
-      s.y = __builtin_amdgcn_exp2f(dt * av.y) * s.y + dx * bcr[n + 1];
-      s.z = __builtin_amdgcn_exp2f(dt * av.z) * s.z + dx * bcr[n + 2];
-      s.w = __builtin_amdgcn_exp2f(dt * av.w) * s.w + dx * bcr[n + 3];
-      const float* cr = bcr + in.N + n;
-      acc += s.x * cr[0];
-      acc += s.y * cr[1];
-      acc += s.z * cr[2];
-      acc += s.w * cr[3];
+      s.x = __builtin_amdgcn_exp2f(dt * av.x) * s.x + dx * ld_f32(bcr + n);
+      s.y = __builtin_amdgcn_exp2f(dt * av.y) * s.y + dx * ld_f32(bcr + n + 1);
+      s.z = __builtin_amdgcn_exp2f(dt * av.z) * s.z + dx * ld_f32(bcr + n + 2);
+      s.w = __builtin_amdgcn_exp2f(dt * av.w) * s.w + dx * ld_f32(bcr + n + 3);
+      const T* cr = bcr + in.N + n;
+      acc += s.x * ld_f32(cr);
+      acc += s.y * ld_f32(cr + 1);
+      acc += s.z * ld_f32(cr + 2);
+      acc += s.w * ld_f32(cr + 3);
       if (live && write_state) *reinterpret_cast<float4*>(row + n) = s;
     } else {
-      const float s = __builtin_amdgcn_exp2f(dt * a[n]) * row[n] + dx * bcr[n];
-      acc += s * bcr[in.N + n];
+      const float s = __builtin_amdgcn_exp2f(dt * a[n]) * row[n] + dx * ld_f32(bcr + n);
+      acc += s * ld_f32(bcr + in.N + n);
       if (live && write_state) row[n] = s;
     }
   }
@@ -224,7 +253,7 @@ scan_step_kernel(const T* __restrict__ x, int x_ld, const T* __restrict__ z, int
   if (ln == 0 && live) st_f32(out + (size_t)t * in.inner + c, (acc + in.d_skip[cc] * xv) * sel_silu(zv));
 }
 
-extern "C" int ullm_selective_scan_step(const void* x, int x_ld, const float* raw, int raw_ld, const float* bc, int bc_ld,
+extern "C" int ullm_selective_scan_step(const void* x, int x_ld, const float* raw, int raw_ld, const void* bc, int bc_ld,
                                         const void* z, int z_ld, const float* a_log2, const float* dt_bias, const float* d_skip,
                                         float* state, long long state_stride, long long state_off, const int* entry_slot, void* out,
                                         int B_, int inner, int N, int write_state, int dtype, hipStream_t stream) {
@@ -233,10 +262,9 @@ extern "C" int ullm_selective_scan_step(const void* x, int x_ld, const float* ra
   const bool by4 = N % 4 == 0 && state_stride % 4 == 0 && state_off % 4 == 0 && ((uintptr_t)state | (uintptr_t)a_log2) % 16 == 0;
   int lanes = 1;
   while (lanes < 64 && lanes * (by4 ? 4 : 1) < N) lanes *= 2;
-  const ScanIn in = {raw, raw_ld, bc, bc_ld, a_log2, dt_bias, d_skip, inner, N};
   const int per = 256 / lanes;
 #define GO(TT, V) hipLaunchKernelGGL((scan_step_kernel<TT, V>), dim3((inner + per - 1) / per, B_), dim3(256), 0, stream, (const TT*)x, x_ld, \
-    (const TT*)z, z_ld, in, state, state_stride, state_off, entry_slot, (TT*)out, lanes, write_state)
+    (const TT*)z, z_ld, SCAN_IN(TT), state, state_stride, state_off, entry_slot, (TT*)out, lanes, write_state)
   if (dtype == ULLM_F32) { if (by4) GO(float, 4); else GO(float, 1); }
   else if (dtype == ULLM_BF16) { if (by4) GO(bf16_t, 4); else GO(bf16_t, 1); }
   else return ULLM_ERR_DTYPE;
@@ -257,7 +285,7 @@ extern "C" int ullm_selective_scan_step(const void* x, int x_ld, const float* ra
 template <typename T, int NPT>
 __global__ void __launch_bounds__(SEL_THREADS)
 selective_scan_kernel(const T* __restrict__ x, int x_ld, const float* __restrict__ raw, int raw_ld,
-                      const float* __restrict__ bc, int bc_ld, const T* __restrict__ z, int z_ld,
+                      const T* __restrict__ bc, int bc_ld, const T* __restrict__ z, int z_ld,
                       const float* __restrict__ a_log2, const float* __restrict__ dt_bias, const float* __restrict__ d_skip,
                       float* __restrict__ state, long long state_stride, long long state_off,
                       const int* __restrict__ q_start, const int* __restrict__ entry_slot, T* __restrict__ out, int inner,
@@ -286,8 +314,8 @@ selective_scan_kernel(const T* __restrict__ x, int x_ld, const float* __restrict
     for (int e = tid; e < SEL_CHUNK * NP; e += SEL_THREADS) {
       const int t = e / NP, n = e % NP;
       const bool ok = t0 + t < end && n < N;
-      s_b[t][n] = ok ? bc[(size_t)(t0 + t) * bc_ld + n] : 0.f;
-      s_c[t][n] = ok ? bc[(size_t)(t0 + t) * bc_ld + N + n] : 0.f;
+      s_b[t][n] = ok ? ld_f32(bc + (size_t)(t0 + t) * bc_ld + n) : 0.f;
+      s_c[t][n] = ok ? ld_f32(bc + (size_t)(t0 + t) * bc_ld + N + n) : 0.f;
     }
     {
       const bool ok = s_live && t0 + st < end;
@@ -339,7 +367,7 @@ selective_scan_kernel(const T* __restrict__ x, int x_ld, const float* __restrict
   }
 }
 
-extern "C" int ullm_selective_scan(const void* x, int x_ld, const float* raw, int raw_ld, const float* bc, int bc_ld,
+extern "C" int ullm_selective_scan(const void* x, int x_ld, const float* raw, int raw_ld, const void* bc, int bc_ld,
                                    const void* z, int z_ld, const float* a_log2, const float* dt_bias, const float* d_skip,
                                    float* state, long long state_stride, long long state_off, const int* q_start,
                                    const int* entry_slot, void* out, int B_, int inner, int N, int write_state, int dtype,
@@ -349,7 +377,7 @@ extern "C" int ullm_selective_scan(const void* x, int x_ld, const float* raw, in
     return ULLM_ERR_SHAPE;
   const dim3 grid((inner + SEL_CH - 1) / SEL_CH, B_), block(SEL_THREADS);
   const int npt = (N + SEL_LANES - 1) / SEL_LANES;
-#define GO(TT, NPT) hipLaunchKernelGGL((selective_scan_kernel<TT, NPT>), grid, block, 0, stream, (const TT*)x, x_ld, raw, raw_ld, bc,   \
+#define GO(TT, NPT) hipLaunchKernelGGL((selective_scan_kernel<TT, NPT>), grid, block, 0, stream, (const TT*)x, x_ld, raw, raw_ld, (const TT*)bc,   \
     bc_ld, (const TT*)z, z_ld, a_log2, dt_bias, d_skip, state, state_stride, state_off, q_start, entry_slot, (TT*)out, inner, N, \
     write_state)
 #define GO_N(TT) do { if (npt == 1) GO(TT, 1); else if (npt == 2) GO(TT, 2); else if (npt <= 4) GO(TT, 4); \

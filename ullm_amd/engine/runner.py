@@ -80,6 +80,7 @@ class ModelRunner:
                 state=torch.zeros((max_requests + 1,) + tuple(need.shape), dtype=need.dtype, device=env.device))
         self._views = views
         self._states = [c.state.view(c.state.shape[0], -1) for c in views.values() if c.state is not None]
+        self._state_table = ops.StateTable(self._states)
         # what the parts' kernels want to know about a step beside the flat batch (Part.step_planners)
         self._planners: Dict[str, object] = {}
         for part in model.parts():
@@ -271,8 +272,7 @@ class ModelRunner:
         if self.feed_source is not None:
             ops.feed_tokens(dev[layout["ids"][0]:layout["ids"][1]], dev[layout["feed"][0]:layout["feed"][1]],
                             self.feed_source)
-        for state in self._states:
-            ops.zero_fresh_rows(state, ctx.entry_slot, ctx.entry_start, ctx.num_entries)
+        self._state_table.zero_fresh(ctx.entry_slot, ctx.entry_start, ctx.num_entries)
         return self.model.forward(ctx, self.caches, rows)
 
     # ------------------------------------------------------------------ the step

@@ -120,6 +120,31 @@ def zero_fresh_rows(state: torch.Tensor, entry_slot: torch.Tensor, entry_start: 
            "zero_fresh_rows")
 
 
+class StateTable:
+    """Per-request state tensors ([rows, anything], contiguous, the same number of rows) whose fresh rows one kernel clears:
+    what :func:`zero_fresh_rows` does, for all of them at once."""
+
+    def __init__(self, states):
+        self.states = [s for s in states if s.numel() > 0]
+        self.rows = self.states[0].shape[0] if self.states else 0
+        sizes = []
+        for s in self.states:
+            _need(s.is_contiguous() and s.dim() >= 1 and s.shape[0] == self.rows, "states must be contiguous, all of as many rows")
+            sizes.append(s.numel() // self.rows * s.element_size())
+        self.most = max(sizes, default=0)
+        flat = [v for s, n in zip(self.states, sizes) for v in (s.data_ptr(), n)]
+        self.table = torch.tensor(flat, dtype=torch.int64, device=self.states[0].device) if self.states else None
+
+    def zero_fresh(self, entry_slot: torch.Tensor, entry_start: torch.Tensor, n_entries: int) -> None:
+        if not self.states:
+            return
+        _i32(entry_slot, "entry_slot", n_entries)
+        _i32(entry_start, "entry_start", n_entries)
+        _check(build.load("elementwise").ullm_zero_fresh_many(
+            _p(self.table), _c_int(len(self.states)), ctypes.c_longlong(self.most), _c_int(self.rows), _p(entry_slot),
+            _p(entry_start), _c_int(n_entries), _stream()), "zero_fresh_many")
+
+
 def gather_rows(src: torch.Tensor, index: torch.Tensor) -> torch.Tensor:
     """src[index] for float32 ``src`` [n, cols] and int32 ``index`` on the device: no index travels from the
     host and nothing waits for the device."""
@@ -1048,7 +1073,7 @@ def gemm_bf16(a: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor] = N
     if (out_dtype == torch.bfloat16 and 0 < lim.sums_from <= M <= lim.sums_to and w.shape[0] % 4 == 0
             and gemm_partial_sums_supports(a, w)):
         return sum_stacks(gemm_partial_sums(a, w), bias)
-    if library and out_dtype == torch.float32 and a.is_contiguous() and w.is_contiguous() and _MM_TAKES_OUT_DTYPE:
+    if library and out_dtype == torch.float32 and a.stride(1) == 1 and w.is_contiguous() and _MM_TAKES_OUT_DTYPE:
         y = torch.mm(a, w.t(), out_dtype=torch.float32)
         return y if bias is None else add_bias(y, bias)
     if library and out_dtype == torch.bfloat16:
@@ -1365,15 +1390,15 @@ def selective_scan(x: torch.Tensor, raw_dt: torch.Tensor, bc: torch.Tensor, z: t
                    dt_bias: torch.Tensor, d_skip: torch.Tensor, state: torch.Tensor, state_off: int, ctx, plan=None,
                    write_state: bool = True) -> torch.Tensor:
     """Per channel c and state n over each entry's tokens: dt = softplus(raw_dt + dt_bias), S = exp(dt A) S + dt x B,
-    y = sum_n S C + d_skip x; returns y * silu(z) ([T, inner] of x's dtype).  ``raw_dt`` float32 [T, inner], ``bc`` float32
-    [T, 2 n] (B, then C), ``a_log2`` float32 [inner, n] = A log2(e); ``x``, ``z`` and ``bc`` may be columns of wider rows.  The
+    y = sum_n S C + d_skip x; returns y * silu(z) ([T, inner] of x's dtype).  ``raw_dt`` float32 [T, inner], ``bc`` [T, 2 n] of
+    x's dtype (B, then C), ``a_log2`` float32 [inner, n] = A log2(e); ``x``, ``z`` and ``bc`` may be columns of wider rows.  The
     states are float32 at ``state[slot, state_off + c * n ..]``.  ``plan`` lists the segments the entries' tokens are cut
     into (:func:`~ullm_amd.parts.ssm.plan_scan_segments`; None: every entry is walked in order)."""
     T, inner = x.shape
     n = a_log2.shape[1]
     _need(x.stride(1) == 1 and z.shape == (T, inner) and z.stride(1) == 1 and z.dtype == x.dtype, "x and z must be [T, inner] of one dtype")
     _f32_rows(raw_dt, "raw_dt", T, inner)
-    _f32_rows(bc, "bc", T, 2 * n)
+    _need(bc.shape == (T, 2 * n) and bc.stride(1) == 1 and bc.dtype == x.dtype, "bc must be [T, 2 n] of x's dtype")
     _need(a_log2.dtype == torch.float32 and a_log2.shape == (inner, n) and a_log2.is_contiguous() and n <= SELECTIVE_SCAN_MAX_STATE,
           f"A must be float32 [inner, n <= {SELECTIVE_SCAN_MAX_STATE}]")
     for v, nm in ((dt_bias, "dt_bias"), (d_skip, "d_skip")):

@@ -19,7 +19,7 @@ The input projection's rows are x | z (``inner`` each).  x passes the short conv
 dt | B | C (``dt_rank``, ``state``, ``state`` values); the step sizes are softplus(W_dt dt + bias), one per channel.  Per
 channel c and state n:  S = exp(-exp(A_log) dt) S + dt x B,  y = sum_n S C + D x;  y * silu(z) is projected out.  A
 request's float32 row holds the convolution's last inputs, then the states.  Step sizes, decays and states are 32-bit;
-the projections and the convolution's result are stored in the compute dtype (B, C and the step sizes in 32-bit).
+the projections and the convolution's result are stored in the compute dtype (the step sizes' last product in 32-bit).
 """
 from __future__ import annotations
 
@@ -144,11 +144,12 @@ class SelectiveScan(Mixer):
         get = lambda role: tensors[self._name(role)]                     # noqa: E731
         self.w_in, self.w_out = get("in").contiguous(), get("out").contiguous()
         self.w_conv, self.b_conv = get("conv").t().contiguous(), get("conv_bias").contiguous()
-        # the low-rank step sizes' inner size is padded with zeros to a multiple of eight: whole 16-byte pieces
+        # the low-rank step sizes' inner size and the row dt | B | C are padded with zeros to multiples of eight: whole
+        # 16-byte pieces
         r, pad = self.dt_rank, -self.dt_rank % 8
         x, dt = get("x"), get("dt")
-        self.w_dt_low = torch.cat((x[:r], x.new_zeros((pad, self.inner)))).contiguous()
-        self.w_bc = x[r:].contiguous()
+        self.w_x = torch.cat((x[:r], x.new_zeros((pad, self.inner)), x[r:], x.new_zeros((-2 * self.state % 8, self.inner)))).contiguous()
+        self.rank8 = r + pad
         self.w_dt = torch.cat((dt, dt.new_zeros((self.inner, pad))), dim=1).contiguous()
         self.dt_bias, self.d_skip = get("dt_bias").contiguous(), get("d").contiguous()
         # A log2(e), rounded to 32-bit once: a decay is then one exponent of two
@@ -158,8 +159,8 @@ class SelectiveScan(Mixer):
         n, rows = self.inner, cache.state.view(cache.state.shape[0], -1)
         proj = linear(x, self.w_in)                                      # x | z
         u = ops.short_conv(proj[:, :n], self.w_conv, self.b_conv, rows, 0, ctx, ops.CONV_SILU, ctx.dtype, write_state=cache.owner)
-        bc = linear(u, self.w_bc, out_dtype=torch.float32)
-        dt = linear(linear(u, self.w_dt_low), self.w_dt, out_dtype=torch.float32)
-        y = ops.selective_scan(u, dt, bc, proj[:, n:], self.a_log2, self.dt_bias, self.d_skip, rows, self.carry, ctx,
+        low = linear(u, self.w_x)                                        # dt | B | C
+        dt = linear(low[:, :self.rank8], self.w_dt, out_dtype=torch.float32)
+        y = ops.selective_scan(u, dt, low[:, self.rank8:self.rank8 + 2 * self.state], proj[:, n:], self.a_log2, self.dt_bias, self.d_skip, rows, self.carry, ctx,
                                ctx.plans["scan segments"], write_state=cache.owner)
         return linear_into_stream(y, self.w_out, ctx)
