@@ -250,7 +250,7 @@ extern "C" int ullm_conv_norm_write(const void* proj, int ld, const float* w, in
                    (uintptr_t)carry % 16 == 0 && ((uintptr_t)w | (uintptr_t)q_gain | (uintptr_t)k_gain) % 16 == 0;
   const int pieces_all = by4 ? C / 4 : C;
   int pieces = 1;
-  while (pieces * 1024 < pieces_all) pieces *= 2;
+  while (pieces * (T_ >= 64 ? 512 : 1024) < pieces_all) pieces *= 2;
   if (pieces > 16) return ULLM_ERR_SHAPE;                    // rows of up to 65536 values (16384 where not by fours)
   const int threads = ((pieces_all + pieces - 1) / pieces + 63) / 64 * 64;
   const bool runs = !single && T_ >= 512;
@@ -259,7 +259,7 @@ extern "C" int ullm_conv_norm_write(const void* proj, int ld, const float* w, in
     q_start, entry_slot, block_table, bt_stride, (TT*)q_out, (TT*)k_pool, (TT*)v_pool, page_size, nq, nkv, hd, T_, single,           \
     pool, pooled_table, pooled_stride, (TT*)pk_pool, (TT*)pv_pool)
 #define GO(TT, TAPS, V, P) GO_R(TT, TAPS, V, P, 1)
-#define GO_P(TT, TAPS, V) do { if (pieces == 1 && runs && V == 4) GO_R(TT, TAPS, V, 1, 4); else if (pieces == 1) GO(TT, TAPS, V, 1); else if (pieces == 2) GO(TT, TAPS, V, 2); \
+#define GO_P(TT, TAPS, V) do { if (pieces <= 4 && runs && V == 4) { if (pieces == 1) GO_R(TT, TAPS, V, 1, 4); else if (pieces == 2) GO_R(TT, TAPS, V, 2, 4); else GO_R(TT, TAPS, V, 4, 4); } else if (pieces == 1) GO(TT, TAPS, V, 1); else if (pieces == 2) GO(TT, TAPS, V, 2); \
     else if (pieces == 4) GO(TT, TAPS, V, 4); else if (pieces == 8) GO(TT, 0, V, 8); else GO(TT, 0, V, 16); } while (0)
   // up to 4 taps with up to 4 pieces a thread the inputs are kept in registers; else every tap is read where it lies,
   // and the state is moved on by a kernel of its own

@@ -51,6 +51,9 @@ def load_model(model_dir: str, dtype: str, device: str, context_len: int, strict
     config_dict = read_config_json(model_dir)
     cfg, model = build_model(config_dict)
     env = make_env(dtype, device, context_within_model(cfg, context_len, strict_context))
+    # what the model is sure to launch is compiled side by side where it is not built yet
+    kernel_build.prepare(["elementwise", "gemm_skinny" if env.dtype == torch.bfloat16 else "gemm_simple"]
+                         + [f for part in model.parts() for f in part.kernel_families(env.dtype)])
     load_weights(model, model_dir, env)
     return cfg, model, env
 

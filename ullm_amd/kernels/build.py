@@ -163,6 +163,28 @@ def build_all(force: bool = True, verbose: bool = True, jobs: int = 4) -> Dict[s
     return results
 
 
+def prepare(wanted, jobs: int = 8) -> None:
+    """Compile the families of ``wanted`` that have no library yet, side by side (a fresh checkout's first run)."""
+    missing = [f for f in dict.fromkeys(wanted) if not os.path.isfile(lib_path(f))]
+    errors: List[str] = []
+
+    def work(queue):
+        while queue:
+            try:
+                compile_family(queue.pop(0))
+            except KernelBuildError as e:
+                errors.append(str(e))
+            except IndexError:
+                return
+    threads = [threading.Thread(target=work, args=(missing,)) for _ in range(min(jobs, len(missing)))]
+    for t in threads:
+        t.start()
+    for t in threads:
+        t.join()
+    if errors:
+        raise KernelBuildError("\n\n".join(errors))
+
+
 def load(family: str) -> ctypes.CDLL:
     """The loaded library of a family, building it first if need be."""
     lib = _loaded.get(family)

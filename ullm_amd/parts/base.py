@@ -242,6 +242,11 @@ class Part:
     # {name: function(StepShape) -> StepPlan}: per-step work lists this part's kernels want (see StepPlan)
     step_planners: Dict[str, Callable] = {}
 
+    def kernel_families(self, dtype: torch.dtype) -> Tuple[str, ...]:
+        """Kernel families the part is sure to launch in this compute dtype: a loader may compile them side by side ahead
+        of the first step (a family that no part names is compiled when it is first used)."""
+        return ()
+
     def weights(self) -> List[WeightDecl]:
         return []
 

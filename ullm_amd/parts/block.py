@@ -171,6 +171,9 @@ class PostNormBlock(Block):
     def children(self):
         return [p for p in (self.mixer, self.mixer_post, self.ffn, self.ffn_post) if p is not None]
 
+    def kernel_families(self, dtype):
+        return ("postnorm", "short_conv") if self.taps else ("postnorm",)
+
     def cache_need(self):
         if not self.taps:
             return self._mixer_needs or None

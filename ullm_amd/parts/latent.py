@@ -63,6 +63,9 @@ class LatentAttention(Mixer):
     def children(self):
         return [self.position] if self.position is not None else []
 
+    def kernel_families(self, dtype):
+        return ("latent", "attention_mfma" if dtype == torch.bfloat16 and self.hd <= 256 else "attention_generic")
+
     def cache_need(self):
         return KVNeed(1, self.hd, self.window)
 

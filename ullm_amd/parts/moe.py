@@ -82,6 +82,9 @@ class RoutedExperts(FeedForward):
         self.names = {**DEFAULT_NAMES, **(names or {})}
         self.w_router = self.correction = self.w_gate_up = self.w_down = self.w_shared_gate_up = self.w_shared_down = None
 
+    def kernel_families(self, dtype):
+        return ("moe",)
+
     # ------------------------------------------------------------------ weights
     def _expert(self, index: int, role: str) -> str:
         return f"{self.prefix}.{self.names['expert'].format(index=index)}.{self.names[role]}"

@@ -63,6 +63,9 @@ class PooledAttention(GQAttention):
         if self.pool:
             self.step_planners[f"blocks of {self.pool}"] = block_planner(self.pool)
 
+    def kernel_families(self, dtype):
+        return ("pooled", "attention_pooled") if dtype == torch.bfloat16 and not self.softmax else ("pooled",)
+
     def cache_need(self):
         needs = [KVNeed(self.nkv, self.hd, max(self.window, self.pool))]
         if self.pool:

@@ -128,6 +128,9 @@ class SelectiveScan(Mixer):
     def _name(self, role: str) -> str:
         return f"{self.prefix}.{self.names[role]}"
 
+    def kernel_families(self, dtype):
+        return ("short_conv", "selective_scan")
+
     def cache_need(self):
         return StateNeed((self.carry + self.inner * self.state,), torch.float32, graph_safe=True)
 
