@@ -22,7 +22,8 @@ def silu(z):
 
 
 def causal_conv(u, w):
-    """u [T, channels], w [channels, taps]: y_t = sum_j w[:, j] u_(t - taps + 1 + j), zeros before the first token."""
+    """u [T, channels], w [channels, taps]: every channel's taps over its own past; the last tap is the token's own input, and
+    what lies ahead of the first token counts as zero."""
     T, taps = u.shape[0], w.shape[1]
     y = torch.zeros_like(u)
     for j in range(taps):
@@ -115,7 +116,7 @@ def pooled_sigmoid_attention(h, w, p, m, eps):
 # ----------------------------------------------------------------------------- selective scan
 
 def selective_scan(x, dt, A, B, C, D):
-    """Per channel c and state n: S <- exp(dt_c A[c, n]) S + dt_c x_c B_n; y_c = sum_n S[c, n] C_n + D_c x_c."""
+    """A row of states per channel: it decays by exp(dt A), takes in dt x B, is read out with C, and D passes x by."""
     T, inner = x.shape
     S = torch.zeros_like(A)
     y = torch.zeros_like(x)

@@ -255,16 +255,21 @@ extern "C" int ullm_latent_query(const void* qa, long long qa_st, long long qa_s
 
 // ------------------------------------------------------------------ a gate per value
 // y[t, h, n] = x[t, h, n] * sigmoid(gate[t, h * N + n]) for x with strides (x_st, x_sh, 1), y contiguous [T, heads * N].
-template <typename T>
+template <typename T, int V>
 __global__ void __launch_bounds__(256)
 value_gate_kernel(const T* __restrict__ x, long long x_st, long long x_sh, const T* __restrict__ gate, long long gate_ld,
                   T* __restrict__ y, int N, int width, size_t total) {
-  const size_t e = (size_t)blockIdx.x * 256 + threadIdx.x;
+  const size_t e = V * ((size_t)blockIdx.x * 256 + threadIdx.x);
   if (e >= total) return;
   const size_t t = e / width;
   const int o = (int)(e - t * width), h = o / N, n = o - h * N;
-  const float g = ld_f32(gate + t * gate_ld + o);
-  st_f32(y + e, ld_f32(x + t * x_st + (size_t)h * x_sh + n) * (1.f / (1.f + expf(-g))));
+  struct alignas(V * sizeof(T)) Piece { T v[V]; };
+  const Piece g = *reinterpret_cast<const Piece*>(gate + t * gate_ld + o);
+  const Piece a = *reinterpret_cast<const Piece*>(x + t * x_st + (size_t)h * x_sh + n);
+  Piece r;
+#pragma unroll
+  for (int u = 0; u < V; ++u) st_f32(&r.v[u], ld_f32(&a.v[u]) * (1.f / (1.f + expf(-ld_f32(&g.v[u])))));
+  *reinterpret_cast<Piece*>(y + e) = r;
 }
 
 extern "C" int ullm_value_gate(const void* x, long long x_st, long long x_sh, const void* gate, long long gate_ld, void* y, int T_,
@@ -272,11 +277,15 @@ extern "C" int ullm_value_gate(const void* x, long long x_st, long long x_sh, co
   if (T_ <= 0) return 0;
   if (heads < 1 || N < 1 || gate_ld < (long long)heads * N) return ULLM_ERR_SHAPE;
   const size_t total = (size_t)T_ * heads * N;
-#define GO(TT) hipLaunchKernelGGL(value_gate_kernel<TT>, dim3((unsigned)((total + 255) / 256)), dim3(256), 0, stream, (const TT*)x, x_st, \
+  const size_t four = 4 * (dtype == ULLM_F32 ? 4 : 2);
+  const bool by4 = N % 4 == 0 && x_st % 4 == 0 && x_sh % 4 == 0 && gate_ld % 4 == 0 && ((uintptr_t)x | (uintptr_t)gate | (uintptr_t)y) % four == 0;
+#define GO_V(TT, V) hipLaunchKernelGGL((value_gate_kernel<TT, V>), dim3((unsigned)((total / V + 255) / 256)), dim3(256), 0, stream, (const TT*)x, x_st, \
     x_sh, (const TT*)gate, gate_ld, (TT*)y, N, heads * N, total)
+#define GO(TT) do { if (by4) GO_V(TT, 4); else GO_V(TT, 1); } while (0)
   if (dtype == ULLM_F32) GO(float);
   else if (dtype == ULLM_BF16) GO(bf16_t);
   else return ULLM_ERR_DTYPE;
 #undef GO
+#undef GO_V
   ULLM_LAUNCH_CHECK();
 }

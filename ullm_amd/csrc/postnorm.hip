@@ -3,8 +3,8 @@
 //
 //   y = a * branch (+ b * second),  stream += y / sqrt(mean(y^2) + eps) * gain
 //   out = stream                                              in the compute dtype, or
-//   out = stream + sum_j w[j] * stream(token - taps + 1 + j)  for steps of single tokens, with the rows before the token in
-//                                                             its state row, which is moved on
+//   out = stream + conv(stream)                               for steps of single tokens: the last taps rows per channel,
+//                                                             those before the token's from its state row, which moves on
 //
 // A branch may be a stack of partial sums [S, T, H], added slice by slice.  Everything is 32-bit; a row's sums have a
 // fixed order.

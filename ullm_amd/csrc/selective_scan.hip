@@ -1,7 +1,7 @@
 // A selective scan with a state per channel (the Mamba form).  Per channel c and state n of an entry's tokens in order:
 //   dt = softplus(raw[t, c] + dt_bias[c])
-//   S[c, n] = exp(dt * A[c, n]) * S[c, n] + dt * x[t, c] * B[t, n]
-//   y[t, c] = sum_n S[c, n] * C[t, n] + D[c] * x[t, c],   stored: y * silu(z[t, c])
+//   S[c, :] = exp(dt * A[c, :]) * S[c, :] + (dt * x[t, c]) * B[t, :]
+//   y       = S[c, :] . C[t, :] + D[c] * x[t, c],   stored: y * silu(z[t, c])
 // A is handed over as A * log2(e), so that a decay is one exponent of two.  The states are float32 and come from and
 // go to the entry's state row (state[slot, off + c * N + n]).  Everything is 32-bit; x, z and the result are stored in
 // the compute dtype (B and C too: they are a projection's values).

@@ -51,10 +51,10 @@ __device__ __forceinline__ void conv_store(bf16_t* p, const float* v) {
 __device__ __forceinline__ float conv_silu_of(float z) { return z / (1.f + expf(-z)); }
 
 // grid (runs of `tok` tokens, channel pieces).  A thread owns V neighbouring channels, keeps their weights and the last
-// taps-1 inputs in registers and walks its run; at the run's start and at every entry's first token the inputs before
-// come from the rows before or from the state row.  `update`: every entry brings one token, and the thread that has
-// used its channels' state moves it on itself.
-template <typename TI, typename TO, int TAPS, int V>
+// taps-1 inputs in registers and walks its run, RUN tokens' rows asked for at a time; at the run's start and at every
+// entry's first token the inputs before come from the rows before or from the state row.  `update`: every entry brings
+// one token, and the thread that has used its channels' state moves it on itself.
+template <typename TI, typename TO, int TAPS, int V, int RUN>
 __global__ void __launch_bounds__(256)
 short_conv_kernel(const TI* __restrict__ in, int in_stride, const float* __restrict__ w, const float* __restrict__ bias,
                   float* __restrict__ carry, long long carry_stride, const int* __restrict__ token_entry,
@@ -69,34 +69,43 @@ short_conv_kernel(const TI* __restrict__ in, int in_stride, const float* __restr
 #pragma unroll
   for (int u = 0; u < V; ++u) b0.v[u] = bias ? bias[c + u] : 0.f;
   const int t0 = blockIdx.x * tok;
-  for (int t = t0; t < t0 + tok && t < T_; ++t) {
-    const int b = token_entry[t], first = q_start[b], i = t - first;
-    if (t == t0 || i == 0) {
-      const float* old = carry + (size_t)entry_slot[b] * carry_stride + c;
+  const int stop = t0 + tok < T_ ? t0 + tok : T_;
+  for (int g0 = t0; g0 < stop; g0 += RUN) {
+    ConvPiece<V> rows[RUN];
 #pragma unroll
-      for (int k = 0; k < TAPS - 1; ++k) {
-        const int l = i - (TAPS - 1) + k;
-        hist[k] = l >= 0 ? conv_load<V>(in + (size_t)(first + l) * in_stride + c)
-                         : conv_load<V>(old + (size_t)(l + TAPS - 1) * channels);
+    for (int r = 0; r < RUN; ++r) rows[r] = conv_load<V>(in + (size_t)(g0 + r < stop ? g0 + r : stop - 1) * in_stride + c);
+#pragma unroll
+    for (int r = 0; r < RUN; ++r) {
+      const int t = g0 + r;
+      if (t >= stop) break;
+      const int b = token_entry[t], first = q_start[b], i = t - first;
+      if (t == t0 || i == 0) {
+        const float* old = carry + (size_t)entry_slot[b] * carry_stride + c;
+#pragma unroll
+        for (int k = 0; k < TAPS - 1; ++k) {
+          const int l = i - (TAPS - 1) + k;
+          hist[k] = l >= 0 ? conv_load<V>(in + (size_t)(first + l) * in_stride + c)
+                           : conv_load<V>(old + (size_t)(l + TAPS - 1) * channels);
+        }
       }
-    }
-    hist[TAPS - 1] = conv_load<V>(in + (size_t)t * in_stride + c);
-    float acc[V];
+      hist[TAPS - 1] = rows[r];
+      float acc[V];
 #pragma unroll
-    for (int u = 0; u < V; ++u) acc[u] = b0.v[u];
+      for (int u = 0; u < V; ++u) acc[u] = b0.v[u];
 #pragma unroll
-    for (int j = 0; j < TAPS; ++j)
+      for (int j = 0; j < TAPS; ++j)
 #pragma unroll
-      for (int u = 0; u < V; ++u) acc[u] += wt[j].v[u] * hist[j].v[u];
+        for (int u = 0; u < V; ++u) acc[u] += wt[j].v[u] * hist[j].v[u];
 #pragma unroll
-    for (int u = 0; u < V; ++u) acc[u] = mode == CONV_SILU ? conv_silu_of(acc[u]) : hist[TAPS - 1].v[u] + acc[u];
-    conv_store<V>(out + (size_t)t * channels + c, acc);
+      for (int u = 0; u < V; ++u) acc[u] = mode == CONV_SILU ? conv_silu_of(acc[u]) : hist[TAPS - 1].v[u] + acc[u];
+      conv_store<V>(out + (size_t)t * channels + c, acc);
 #pragma unroll
-    for (int k = 0; k < TAPS - 1; ++k) hist[k] = hist[k + 1];
-    if (update) {
-      float* row = carry + (size_t)entry_slot[b] * carry_stride + c;
+      for (int k = 0; k < TAPS - 1; ++k) hist[k] = hist[k + 1];
+      if (update) {
+        float* row = carry + (size_t)entry_slot[b] * carry_stride + c;
 #pragma unroll
-      for (int k = 0; k < TAPS - 1; ++k) conv_store<V>(row + (size_t)k * channels, hist[k].v);
+        for (int k = 0; k < TAPS - 1; ++k) conv_store<V>(row + (size_t)k * channels, hist[k].v);
+      }
     }
   }
 }
@@ -132,11 +141,12 @@ static int launch_conv(const void* in, int in_stride, const float* w, const floa
   bool moved = false;
   if (taps <= 4) {
     // a block walks several tokens where the step has many: weights and the overlap with the rows before cost less
-    const int tok = single ? 1 : (T_ >= 2048 ? 16 : (T_ >= 256 ? 4 : 1));
+    const int tok = single ? 1 : (T_ >= 1024 ? 8 : (T_ >= 256 ? 4 : 1));
     moved = single && update;
-#define GO(TAPS, V) hipLaunchKernelGGL((short_conv_kernel<TI, TO, TAPS, V>), dim3((T_ + tok - 1) / tok, (channels / V + 255) / 256), \
+#define GO_R(TAPS, V, R) hipLaunchKernelGGL((short_conv_kernel<TI, TO, TAPS, V, R>), dim3((T_ + tok - 1) / tok, (channels / V + 255) / 256), \
     dim3(256), 0, stream, (const TI*)in, in_stride, w, bias, carry, carry_stride, token_entry, q_start, entry_slot, (TO*)out, T_,     \
     channels, mode, tok, moved ? 1 : 0)
+#define GO(TAPS, V) do { if (tok >= 4) GO_R(TAPS, V, 4); else GO_R(TAPS, V, 1); } while (0)
 #define GO_V(TAPS) do { if (by4) GO(TAPS, 4); else GO(TAPS, 1); } while (0)
     if (taps == 1) GO_V(1);
     else if (taps == 2) GO_V(2);
@@ -144,6 +154,7 @@ static int launch_conv(const void* in, int in_stride, const float* w, const floa
     else GO_V(4);
 #undef GO_V
 #undef GO
+#undef GO_R
   } else {
     hipLaunchKernelGGL((short_conv_general_kernel<TI, TO>), dim3(T_, (channels + 255) / 256), dim3(256), 0, stream, (const TI*)in,
                        in_stride, w, bias, carry, carry_stride, token_entry, q_start, entry_slot, (TO*)out, channels, taps, mode);

@@ -4,9 +4,9 @@ Grouped-query attention without positions.  q, k and v pass a short causal convo
 behind their projections; q and k are then RMS-normed over the whole projection, all heads at once, with a gain per value.
 Scores q . k * scale are soft-capped (``softcap``; 0: not) and a number per head is added; the weight of a visible key is
 the sigmoid of that, and the weights are not normalised over the keys (``weights="softmax"``: the softmax instead).
-Visible to position i are the last ``window`` tokens, itself included, and one key and value for every block of ``pool``
-consecutive tokens (from position 0 on) that lies wholly before that window: the means of the block's keys and values as
-the cache holds them.  ``pool`` 0: the window alone; ``window`` 0: every earlier token.
+A query sees the last ``window`` tokens, its own included.  The tokens are also counted off in blocks of ``pool`` from
+position 0 on, and every block that has ended ahead of the query's window stands in with one row: its keys averaged and
+its values averaged, from the rows in the pages.  ``pool`` 0: the window alone; ``window`` 0: every earlier token.
 
 What a request keeps: the window's keys and values in pages (a page lives until neither the window nor the block being
 filled needs it), the blocks' means in pages of their own with one row per block, and the convolution's last inputs in
