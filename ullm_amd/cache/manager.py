@@ -5,9 +5,10 @@ the device pools the ids index are owned by the model runner.
 Against the reference (ullm/core/kv_cache.py:326-398, ullm/core/req_state.py:6-75): its "page" is a
 single token and all layers share one slot id space; a request's row in fixed arrays is an index
 from a pool of ``max_bs``.  Here
-  * layers with the same needs (kv heads, head size, window) form a *group* with pages of its own
+  * layers with the same needs (kv heads, head size, window or chunk) form a *group* with pages of its own
     and one block table per request;
-  * a group with a window gives pages back as soon as the window has passed them;
+  * a group with a window gives pages back as soon as the window has passed them, a group whose queries see
+    their own chunk of positions alone as soon as the next chunk begins;
   * a group may keep one row for every so many tokens (``tokens_per_row``): its pages hold page_size rows
     and it takes one only when that many tokens are complete;
   * pages are handed out per portion (``reserve``) and a request's progress is recorded after the
@@ -37,6 +38,13 @@ class CacheGroupSpec:
     # per pool; None = one key row and one value row per kv head
     rows: Optional[tuple] = None
     tokens_per_row: int = 1       # one row per this many tokens, written when the last of them is in
+    chunk: int = 0                # > 0: a query sees the keys of its own chunk of this many positions alone
+
+    def first_needed(self, computed: int) -> int:
+        """The first position that a query at ``computed`` or later can see."""
+        if self.chunk > 0:
+            return computed // self.chunk * self.chunk
+        return max(0, computed - self.window + 1) if self.window > 0 else 0
 
     def bytes_per_token(self, itemsize: int) -> int:
         rows = self.rows if self.rows is not None else ((self.num_kv_heads, self.head_dim, None),) * 2
@@ -87,7 +95,7 @@ class CacheManager:
         # no page: a step gathers its rows from here instead of converting Python lists
         self._rows = [np.full((max_requests, 16), -1, dtype=np.int32) for _ in groups]
         self.requests: Dict[str, RequestCache] = {}
-        shareable = all(g.window == 0 and g.tokens_per_row == 1 for g in groups) and len(groups) > 0
+        shareable = all(g.window == 0 and g.chunk == 0 and g.tokens_per_row == 1 for g in groups) and len(groups) > 0
         self.prefix_tree: Optional[PrefixTree] = (
             PrefixTree(page_size, self.allocators) if enable_prefix_cache and shareable else None)
 
@@ -174,8 +182,8 @@ class CacheManager:
         return True
 
     def commit(self, rc: RequestCache, n_new: int) -> None:
-        """Record that ``n_new`` more tokens are in the cache; windowed groups give back the pages
-        no later query can reach: page i is dead once (i+1)*page_size <= num_computed - window + 1."""
+        """Record that ``n_new`` more tokens are in the cache; groups with a window or chunks give back the pages
+        no later query can reach: page i is dead once (i+1)*page_size <= the first position the next query sees."""
         if rc.released:
             raise PageError(f"request {rc.request_id!r} was released")
         P = self.page_size
@@ -184,8 +192,8 @@ class CacheManager:
                 raise PageError(f"request {rc.request_id!r} computed past its reserved pages")
         rc.num_computed += n_new
         for g, spec in enumerate(self.groups):
-            if spec.window > 0:
-                dead_upto = (rc.num_computed - spec.window + 1) // P   # pages [first_live, dead_upto) die
+            if spec.window > 0 or spec.chunk > 0:
+                dead_upto = spec.first_needed(rc.num_computed) // P    # pages [first_live, dead_upto) die
                 table = rc.tables[g]
                 for i in range(rc.first_live[g], min(dead_upto, len(table))):
                     if table[i] >= 0:

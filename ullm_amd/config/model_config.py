@@ -985,3 +985,159 @@ def _nadevik_experts(f) -> NadevikExperts:
     if not 1 <= e.top <= e.experts // e.groups * e.keep or e.ff < 1 or not e.limit > 0:
         raise ConfigError(f"top = {e.top} of {e.experts // e.groups * e.keep} experts in the kept groups; sizes and 'limit' must be positive")
     return e
+
+
+# ----------------------------------------------------------------------------------------- Risolorn
+
+@dataclass(frozen=True)
+class RisolornDelta:
+    """The gated delta rule: convolved q, k and v, unit queries and keys, one decay and one write strength per head."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    conv: int                       # taps of the convolutions behind q, k and v
+
+
+@dataclass(frozen=True)
+class RisolornMemory:
+    """A matrix memory with exponential gates under a soft cap."""
+    heads: int
+    dim: int
+    vdim: int
+    gate_cap: float
+
+
+@dataclass(frozen=True)
+class RisolornAttention:
+    """Grouped-query attention with biases, a partial rotation, sinks, and keys of the query's own chunk alone."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    chunk: int                      # positions of a chunk; 0: every earlier key is seen
+    rot_dims: int                   # 0: no rotation
+    rot_base: float
+    rot_scaling: Optional[RotaryScaling]
+
+
+@dataclass(frozen=True)
+class RisolornExperts:
+    experts: int
+    top: int
+    groups: int                     # experts form this many equal groups of neighbours
+    keep: int                       # and only the best this many are chosen from
+    ff: int
+
+
+@dataclass(frozen=True)
+class RisolornLayer:
+    type: str                       # "delta" | "mlstm" | "attention"
+    mixer: object
+    mlp: Optional[RisolornExperts]
+
+
+@dataclass(frozen=True)
+class RisolornConfig:
+    """Keys of a Risolorn config.json: layers listed one by one, each a mixer of three kinds beside a routed feed-forward
+    (or none) on one squashed input; a scaled embedding, a head of its own and a scale on the logits."""
+    architecture: str
+    vocab_size: int
+    hidden_size: int
+    layers: tuple                   # of RisolornLayer
+    norm_eps: float
+    embedding_scale: float
+    logit_scale: float
+
+    @classmethod
+    def from_dict(cls, d: Mapping[str, Any]) -> "RisolornConfig":
+        norm, emb = d.get("norm") or {}, d.get("embedding") or {}
+        raw_layers = d.get("layers")
+        if not isinstance(raw_layers, (list, tuple)) or not raw_layers:
+            raise ConfigError("config.json: key 'layers' must be a non-empty list")
+        readers = {"attention": _risolorn_attention, "delta": _risolorn_delta, "mlstm": _risolorn_memory}
+        layers = []
+        for i, L in enumerate(raw_layers):
+            try:
+                if not isinstance(L, Mapping):
+                    raise ConfigError("a layer must be an object")
+                kind, m = _take(L, "type", str), L.get("mixer")
+                if kind not in readers:
+                    raise ConfigError(f"type {kind!r}; known: {sorted(readers)}")
+                if not isinstance(m, Mapping):
+                    raise ConfigError("no 'mixer' object")
+                mlp = L.get("mlp")
+                layers.append(RisolornLayer(kind, readers[kind](m), None if mlp is None else _risolorn_experts(mlp)))
+            except ConfigError as e:
+                raise ConfigError(f"{e} (layer {i})") from None
+        cfg = cls(architecture=_take(d, "architecture", str, "Risolorn"), vocab_size=_take(d, "vocab", int),
+                  hidden_size=_take(d, "width", int), layers=tuple(layers), norm_eps=_take(norm, "eps", float),
+                  embedding_scale=_take(emb, "scale", float, 1.0), logit_scale=_take(d, "logit_scale", float, 1.0))
+        if cfg.vocab_size < 1 or cfg.hidden_size < 1 or cfg.norm_eps < 0:
+            raise ConfigError("config.json: 'vocab' and 'width' must be positive, 'norm.eps' not negative")
+        return cfg
+
+    @property
+    def num_hidden_layers(self) -> int:
+        return len(self.layers)
+
+
+def _risolorn_heads(m: Mapping) -> dict:
+    heads, dim = _take(m, "heads", int), _take(m, "dim", int)
+    s = dict(heads=heads, kv_heads=_take(m, "kv_heads", int, heads), dim=dim, vdim=_take(m, "vdim", int, dim))
+    if min(s.values()) < 1 or heads % s["kv_heads"]:
+        raise ConfigError(f"{heads} heads over {s['kv_heads']} key heads of sizes {dim} and {s['vdim']}")
+    return s
+
+
+def _risolorn_delta(m: Mapping) -> RisolornDelta:
+    r = RisolornDelta(**_risolorn_heads(m), conv=_take(m, "conv", int))
+    if r.conv < 1:
+        raise ConfigError(f"'conv' = {r.conv} taps: at least the current token's")
+    return r
+
+
+def _risolorn_memory(m: Mapping) -> RisolornMemory:
+    s = _risolorn_heads(m)
+    if s.pop("kv_heads") != s["heads"]:
+        raise ConfigError("an mlstm mixer has keys for every head of its own")
+    r = RisolornMemory(**s, gate_cap=_take(m, "gate_cap", float))
+    if not r.gate_cap > 0:
+        raise ConfigError(f"'gate_cap' = {r.gate_cap} must be positive")
+    return r
+
+
+def _risolorn_attention(m: Mapping) -> RisolornAttention:
+    s = _risolorn_heads(m)
+    rot, mask = m.get("rot") or {}, m.get("mask") or {}
+    sc, scaling = rot.get("scaling"), None
+    if sc is not None:
+        if not isinstance(sc, Mapping):
+            raise ConfigError("'rot.scaling' must be an object")
+        scaling = RotaryScaling(factor=_take(sc, "factor", float), original=_take(sc, "original", float),
+                                fast=_take(sc, "fast", float), slow=_take(sc, "slow", float))
+        if min(scaling.factor, scaling.original, scaling.fast, scaling.slow) <= 0:
+            raise ConfigError("'rot.scaling': factor, original, fast and slow must be positive")
+    a = RisolornAttention(**s, scale=_take(m, "scale", float, s["dim"] ** -0.5), chunk=_take(mask, "size", int, 0),
+                          rot_dims=_take(rot, "dims", int, 0), rot_base=_take(rot, "base", float, 10000.0), rot_scaling=scaling)
+    if a.chunk < 0 or a.rot_base <= 0 or (scaling is not None and a.rot_base == 1.0):
+        raise ConfigError(f"'mask.size' = {a.chunk} must not be negative and 'rot.base' = {a.rot_base} positive (not 1 under a scaling)")
+    if a.rot_dims < 0 or a.rot_dims % 2 or a.rot_dims > a.dim:
+        raise ConfigError(f"'rot.dims' = {a.rot_dims} must be even and at most 'dim' = {a.dim}")
+    return a
+
+
+def _risolorn_experts(f) -> RisolornExperts:
+    if not isinstance(f, Mapping) or _take(f, "kind", str) != "moe":
+        raise ConfigError("'mlp' must be null or an object of kind 'moe'")
+    router, expert = f.get("router") or {}, f.get("expert") or {}
+    groups = router.get("groups") or {}
+    count = _take(groups, "count", int, 1)
+    e = RisolornExperts(experts=_take(router, "experts", int), top=_take(router, "top", int), groups=count,
+                        keep=_take(groups, "keep", int, count), ff=_take(expert, "ff", int))
+    if e.experts < 1 or e.groups < 1 or e.experts % e.groups or not 1 <= e.keep <= e.groups:
+        raise ConfigError(f"{e.experts} experts in {e.groups} equal groups of which {e.keep} are kept")
+    if not 1 <= e.top <= e.experts // e.groups * e.keep or e.ff < 1:
+        raise ConfigError(f"top = {e.top} of {e.experts // e.groups * e.keep} experts in the kept groups of size {e.ff}")
+    return e

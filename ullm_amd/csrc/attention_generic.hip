@@ -1,5 +1,5 @@
 // Paged grouped-query attention, general form: any head size up to 1024, any number of heads and
-// groups, any page size, any mix of prompt portions and single decoded tokens, optional window.
+// groups, any page size, any mix of prompt portions and single decoded tokens, optional window or chunk (a negative `window`).
 // One block per (token, query head); keys are visited in tiles of the block size in a fixed order
 // that depends only on the token's own position, so the result for a token is the same however
 // the batch was cut.  Scores, running maximum, sum and output are 32-bit.  Optionally a bias by
@@ -33,7 +33,7 @@ paged_attention_generic_kernel(const T* __restrict__ q, int q_stride, T* __restr
   const int kvh = h / (nq / nkv);
   const int pos = positions[t];
   const int* bt = block_table + (size_t)token_entry[t] * bt_stride;
-  const int lo = (window > 0 && pos - window + 1 > 0) ? pos - window + 1 : 0;
+  const int lo = first_seen_key(pos, window);
   const int hi = pos;
   const T* qp = q + (size_t)t * q_stride + (size_t)h * hd;
   for (int i = tid; i < hd; i += ATT_THREADS) q_s[i] = ld_f32(qp + i) * scale;
@@ -112,7 +112,7 @@ extern "C" int ullm_paged_attention_generic(
     const float* sink, int dtype, hipStream_t stream) {
   if (T_ <= 0) return 0;
   if (bias && bias_rows <= 0) return ULLM_ERR_SHAPE;
-  if (hd <= 0 || hd > ATT_MAX_HD || nq <= 0 || nkv <= 0 || nq % nkv != 0 || page_size <= 0 || window < 0)
+  if (hd <= 0 || hd > ATT_MAX_HD || nq <= 0 || nkv <= 0 || nq % nkv != 0 || page_size <= 0)
     return ULLM_ERR_SHAPE;
   dim3 grid(T_, nq), block(ATT_THREADS);
 #define GO(TT) hipLaunchKernelGGL(paged_attention_generic_kernel<TT>, grid, block, 0, stream, \

@@ -16,7 +16,7 @@
 // output is rescaled only then: the result is the same sum, and most tiles skip the rescaling.
 //
 // Semantics as in the general kernel: causal with the queries at the end of the keys, optional
-// window, query head h reads kv head h / (nq / nkv) (ullm/layers/attention.py:76-104,271,298-309).
+// window or chunk (a negative `window`: see first_seen_key), query head h reads kv head h / (nq / nkv) (ullm/layers/attention.py:76-104,271,298-309).
 #include "common.h"
 #include <type_traits>
 #include "no_alloc.h"
@@ -558,7 +558,7 @@ attention_decode_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t* __re
   }();
   queries.fetch_early();
   const int pos = positions[t];
-  const int lo = (window > 0 && pos - window + 1 > 0) ? pos - window + 1 : 0;
+  const int lo = first_seen_key(pos, window);
   const int first = lo & ~31;
   const int tiles = (pos + 1 - first + 31) / 32;
   const int share = 32 * ((tiles + num_splits * WAVES - 1) / (num_splits * WAVES));
@@ -1046,7 +1046,7 @@ attention_prefill_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t* __r
     const bool ok = head_ok && 16 * qg + c < count;
     tok[qg] = first + (16 * qg + c < count ? 16 * qg + c : 0);
     const int pos = positions[tok[qg]];
-    clo[qg] = (window > 0 && pos - window + 1 > 0) ? pos - window + 1 : 0;
+    clo[qg] = first_seen_key(pos, window);
     chi[qg] = ok ? pos : -1;
     const bf16_t* qp = q + (size_t)tok[qg] * q_stride + (size_t)head * HD + 8 * g;
 #pragma unroll
@@ -1065,8 +1065,8 @@ attention_prefill_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t* __r
   const int last_pos = positions[first + count - 1];
   const int first_pos = positions[first];
   // keys every column of the tile sees without a test: from the last column's window start up to the first column
-  const int open_lo = (window > 0 && last_pos - window + 1 > 0) ? last_pos - window + 1 : 0;
-  const int key_begin = ((window > 0 && first_pos - window + 1 > 0) ? first_pos - window + 1 : 0) & ~31;
+  const int open_lo = first_seen_key(last_pos, window);
+  const int key_begin = first_seen_key(first_pos, window) & ~31;
   const int key_end = last_pos + 1;
   // this half's share of the 32-key tiles
   const int steps = ((key_end - key_begin + 31) / 32 + KS - 1) / KS;
@@ -1413,7 +1413,7 @@ attention_prefill_dma_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t*
     const bool ok = head_ok && 16 * qg + c < count;
     tok[qg] = first + (16 * qg + c < count ? 16 * qg + c : 0);
     const int pos = positions[tok[qg]];
-    clo[qg] = (window > 0 && pos - window + 1 > 0) ? pos - window + 1 : 0;
+    clo[qg] = first_seen_key(pos, window);
     chi[qg] = ok ? pos : -1;
     const bf16_t* qp = q + (size_t)tok[qg] * q_stride + (size_t)head * HD + 8 * g;
 #pragma unroll
@@ -1431,8 +1431,8 @@ attention_prefill_dma_kernel(const bf16_t* __restrict__ q, int q_stride, bf16_t*
   }
   const int last_pos = positions[first + count - 1];
   const int first_pos = positions[first];
-  const int open_lo = (window > 0 && last_pos - window + 1 > 0) ? last_pos - window + 1 : 0;
-  const int key_begin = ((window > 0 && first_pos - window + 1 > 0) ? first_pos - window + 1 : 0) & ~31;
+  const int open_lo = first_seen_key(last_pos, window);
+  const int key_begin = first_seen_key(first_pos, window) & ~31;
   const int key_end = last_pos + 1;
   const int steps = ((key_end - key_begin + 31) / 32 + KS - 1) / KS;    // this half's share of the 32-key tiles
   const int my_begin = key_begin + half * steps * 32;
@@ -1595,7 +1595,7 @@ static int decode_launch(
   if (!ullm_attention_mfma_supports(hd, page_size, nq, nkv)) return ULLM_ERR_UNSUPPORTED;
   if (waves != 1 && waves != 4 && waves != 8) return ULLM_ERR_UNSUPPORTED;
   if (hd == 256 && waves == 8) waves = 4;                // shared memory of the merge
-  if (num_splits < 1 || num_splits > 65535 || window < 0) return ULLM_ERR_SHAPE;
+  if (num_splits < 1 || num_splits > 65535) return ULLM_ERR_SHAPE;
   if (num_splits > 1 && !workspace) return ULLM_ERR_SHAPE;
   const int G = nq / nkv, groups = (G + 15) / 16;
   if (n_items > 65535 || nkv * groups > 65535) return ULLM_ERR_SHAPE;
@@ -1843,7 +1843,7 @@ static int prefill_any(
   if (!ullm_attention_mfma_supports(hd, page_size, nq, nkv)) return ULLM_ERR_UNSUPPORTED;
   const bool staged = halves >= 10;                       // 10, 11, 12: as 0, 1, 2 with the kernel that stages tiles in registers
   if (staged) halves -= 10;
-  if (window < 0 || halves < 0 || halves > 2) return ULLM_ERR_SHAPE;
+  if (halves < 0 || halves > 2) return ULLM_ERR_SHAPE;
   const int chunks = (nq / nkv + PREFILL_WAVES - 1) / PREFILL_WAVES;
   const long long blocks = (long long)n_tiles * nkv * chunks;
   if (blocks > 0x7fffffffLL) return ULLM_ERR_SHAPE;
@@ -1853,9 +1853,10 @@ static int prefill_any(
     const long long units = compute_units();
     bool enough;
     if (keys_total > 0 && keys_max > 0) {
-      if (window > 0) {
-        if (keys_max > window + 32) keys_max = window + 32;
-        if (keys_total > (long long)n_tiles * (window + 32)) keys_total = (long long)n_tiles * (window + 32);
+      if (window != 0) {
+        const int reach = (window > 0 ? window : -window) + 32;
+        if (keys_max > reach) keys_max = reach;
+        if (keys_total > (long long)n_tiles * reach) keys_total = (long long)n_tiles * reach;
       }
       enough = (double)keys_total * nkv * chunks / (2.0 * units) >= 0.6 * keys_max;
     } else {

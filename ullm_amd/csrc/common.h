@@ -113,6 +113,13 @@ __device__ __forceinline__ float max_with_lane_xor32(float v) {
 #endif
 }
 
+// The first key that position `pos` sees.  window > 0: the last `window` keys, its own included; window < 0: the keys of its
+// own chunk, chunks of -window positions counted from position 0; 0: every earlier key.  It never falls as pos rises.
+__device__ __forceinline__ int first_seen_key(int pos, int window) {
+  if (window < 0) return pos - pos % -window;
+  return (window > 0 && pos - window + 1 > 0) ? pos - window + 1 : 0;
+}
+
 __device__ __forceinline__ float wave_sum(float v) {
 #pragma unroll
   for (int m = WAVE / 2; m > 0; m >>= 1) v += __shfl_xor(v, m, WAVE);

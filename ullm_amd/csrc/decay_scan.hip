@@ -471,7 +471,8 @@ extern "C" int ullm_token_shift(const void* x, const float* mu, float* state, lo
 // ------------------------------------------------------------------ norm of the outputs, gain and gate
 // The row o [width] is cut into `parts` equal parts (the heads, or one part); each is divided by its root mean
 // square (eps inside the root), multiplied by gain[c % gain_len] (a gain per value channel shared by the heads, or
-// one per column) and by silu or sigmoid of the gate's raw value g[t, c].  Parts of up to 1024 values: a wave per
+// one per column) and by silu or sigmoid of the gate's raw value g[t, c].  With `den` the part is first divided by
+// max(|den[t, part]|, least[t, part]) + 1e-6 (a memory's normaliser and the least it counts).  Parts of up to 1024 values: a wave per
 // (token, part), every lane's values in registers between the sum of squares and the scaling; longer parts: a block.
 #define NORM_PER_LANE 16
 // `slices` > 1: o is [slices, T, width] and a value is the sum of its slices, added in their order.
@@ -481,11 +482,20 @@ __device__ __forceinline__ float sum_slices(const float* p, int slices, size_t s
   return v;
 }
 
+struct Divisor {
+  const float* den;         // [T, parts] or null
+  const float* least;       // rows least_ld apart
+  int least_ld;
+};
+__device__ __forceinline__ float over_divisor(const Divisor& d, int t, int part, int parts) {
+  return d.den ? 1.f / (fmaxf(fabsf(d.den[(size_t)t * parts + part]), d.least[(size_t)t * d.least_ld + part]) + 1e-6f) : 1.f;
+}
+
 template <typename TO>
 __global__ void __launch_bounds__(256)
 gated_unit_norm_wave_kernel(const float* __restrict__ o, const float* __restrict__ g, int g_ld, const float* __restrict__ gain,
                             int gain_len, float eps, int gate_kind, TO* __restrict__ out, int T_, int width, int parts,
-                            int slices) {
+                            int slices, const Divisor divisor) {
   const int lane = threadIdx.x % WAVE;
   const long long item = (long long)blockIdx.x * (256 / WAVE) + threadIdx.x / WAVE;
   if (item >= (long long)T_ * parts) return;
@@ -493,11 +503,12 @@ gated_unit_norm_wave_kernel(const float* __restrict__ o, const float* __restrict
   const int size = width / parts;
   const float* src = o + (size_t)t * width + (size_t)part * size;
   float v[NORM_PER_LANE], z[NORM_PER_LANE];
+  const float over = over_divisor(divisor, t, part, parts);
   float sq = 0.f;
 #pragma unroll
   for (int i = 0; i < NORM_PER_LANE; ++i) {
     const int c = lane + WAVE * i;
-    v[i] = c < size ? sum_slices(src + c, slices, (size_t)T_ * width) : 0.f;
+    v[i] = c < size ? sum_slices(src + c, slices, (size_t)T_ * width) * over : 0.f;
     z[i] = c < size ? g[(size_t)t * g_ld + part * size + c] : 0.f;
     sq += v[i] * v[i];
   }
@@ -517,15 +528,16 @@ template <typename TO>
 __global__ void __launch_bounds__(1024)
 gated_unit_norm_block_kernel(const float* __restrict__ o, const float* __restrict__ g, int g_ld, const float* __restrict__ gain,
                              int gain_len, float eps, int gate_kind, TO* __restrict__ out, int T_, int width, int parts,
-                             int slices) {
+                             int slices, const Divisor divisor) {
   __shared__ float scratch[16];
   const int t = blockIdx.x / parts, part = blockIdx.x % parts;
   const int size = width / parts;
   const float* src = o + (size_t)t * width + (size_t)part * size;
   const size_t stride = (size_t)T_ * width;
+  const float over = over_divisor(divisor, t, part, parts);
   float sq = 0.f;
   for (int c = threadIdx.x; c < size; c += blockDim.x) {
-    const float x = sum_slices(src + c, slices, stride);
+    const float x = sum_slices(src + c, slices, stride) * over;
     sq += x * x;
   }
   const float r = 1.f / sqrtf(block_sum(sq, scratch) / (float)size + eps);
@@ -533,37 +545,39 @@ gated_unit_norm_block_kernel(const float* __restrict__ o, const float* __restric
     const int col = part * size + c;
     const float z = g[(size_t)t * g_ld + col];
     const float gate = gate_kind == GATE_SIGMOID ? 1.f / (1.f + expf(-z)) : exact_silu(z);
-    st_f32(out + (size_t)t * width + col, sum_slices(src + c, slices, stride) * r * gain[col % gain_len] * gate);
+    st_f32(out + (size_t)t * width + col, sum_slices(src + c, slices, stride) * over * r * gain[col % gain_len] * gate);
   }
 }
 
 extern "C" int ullm_gated_unit_norm(const float* o, const float* g, int g_ld, const float* gain, int gain_len, float eps,
-                                    int gate_kind, void* out, int T_, int width, int parts, int slices, int out_dtype,
-                                    hipStream_t stream) {
+                                    int gate_kind, void* out, int T_, int width, int parts, int slices, const float* den,
+                                    const float* least, int least_ld, int out_dtype, hipStream_t stream) {
   if (T_ <= 0) return 0;
   if (width < 1 || parts < 1 || width % parts || gain_len < 1 || width % gain_len || slices < 1) return ULLM_ERR_SHAPE;
   if (gate_kind != GATE_SILU && gate_kind != GATE_SIGMOID) return ULLM_ERR_UNSUPPORTED;
   if (out_dtype != ULLM_F32 && out_dtype != ULLM_BF16) return ULLM_ERR_DTYPE;
+  if (den && !least) return ULLM_ERR_SHAPE;
+  const Divisor divisor = {den, least, least_ld};
   const int size = width / parts;
   if (size <= WAVE * NORM_PER_LANE) {
     const long long items = (long long)T_ * parts;
     const dim3 grid((unsigned)((items + 3) / 4));
     if (out_dtype == ULLM_F32)
       hipLaunchKernelGGL(gated_unit_norm_wave_kernel<float>, grid, dim3(256), 0, stream, o, g, g_ld, gain, gain_len, eps,
-                         gate_kind, (float*)out, T_, width, parts, slices);
+                         gate_kind, (float*)out, T_, width, parts, slices, divisor);
     else
       hipLaunchKernelGGL(gated_unit_norm_wave_kernel<bf16_t>, grid, dim3(256), 0, stream, o, g, g_ld, gain, gain_len, eps,
-                         gate_kind, (bf16_t*)out, T_, width, parts, slices);
+                         gate_kind, (bf16_t*)out, T_, width, parts, slices, divisor);
   } else {
     int threads = 256;
     while (threads < size / 4 && threads < 1024) threads *= 2;
     const dim3 grid((unsigned)((long long)T_ * parts));
     if (out_dtype == ULLM_F32)
       hipLaunchKernelGGL(gated_unit_norm_block_kernel<float>, grid, dim3(threads), 0, stream, o, g, g_ld, gain, gain_len, eps,
-                         gate_kind, (float*)out, T_, width, parts, slices);
+                         gate_kind, (float*)out, T_, width, parts, slices, divisor);
     else
       hipLaunchKernelGGL(gated_unit_norm_block_kernel<bf16_t>, grid, dim3(threads), 0, stream, o, g, g_ld, gain, gain_len, eps,
-                         gate_kind, (bf16_t*)out, T_, width, parts, slices);
+                         gate_kind, (bf16_t*)out, T_, width, parts, slices, divisor);
   }
   ULLM_LAUNCH_CHECK();
 }

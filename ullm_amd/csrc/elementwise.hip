@@ -1128,6 +1128,58 @@ add_norm_general_kernel(const TB* __restrict__ branch, float* __restrict__ resid
   for (int c = threadIdx.x; c < H; c += blockDim.x) st_f32(out + c, ((row[c] - mean) * rs) * gain[c]);
 }
 
+// ------------------------------------------------------------------ add + squash
+// For output row r (input row i = rows ? rows[r] : r):
+//   s = residual[i] + mult * sum over slices of float(branch[slice, i])   (slices 0: nothing is added)
+//   if write_res: residual[i] = s;   y[r] = tanh(alpha * s) * gain + shift
+// No statistics of the row: a thread per piece of V neighbouring columns, rows side by side in a block.
+template <typename TB, typename TY, int V>
+__global__ void __launch_bounds__(256)
+add_tanh_kernel(const TB* __restrict__ branch, int slices, float mult, float* __restrict__ residual,
+                const float* __restrict__ alpha, const float* __restrict__ gain, const float* __restrict__ shift,
+                TY* __restrict__ y, const int* __restrict__ rows, int n_rows, long long slice_stride, int H, int write_res) {
+  const int pieces = H / V;
+  const size_t e = (size_t)blockIdx.x * 256 + threadIdx.x;
+  if (e >= (size_t)n_rows * pieces) return;
+  const int r = (int)(e / pieces), c = V * (int)(e % pieces);
+  const size_t at = (size_t)(rows ? rows[r] : r) * H + c;
+  float s[V], b[V], g[V], h[V];
+  const float a = *alpha;
+#pragma unroll
+  for (int j = 0; j < V; ++j) s[j] = residual[at + j], g[j] = gain[c + j], h[j] = shift[c + j], b[j] = 0.f;
+  for (int k = 0; k < slices; ++k) {
+#pragma unroll
+    for (int j = 0; j < V; ++j) b[j] += ld_f32(branch + (size_t)k * slice_stride + at + j);
+  }
+#pragma unroll
+  for (int j = 0; j < V; ++j) {
+    s[j] += mult * b[j];
+    if (write_res && slices) residual[at + j] = s[j];
+    st_f32(y + (size_t)r * H + c + j, tanhf(a * s[j]) * g[j] + h[j]);
+  }
+}
+
+extern "C" int ullm_add_tanh(const void* branch, int slices, float mult, float* residual, const float* alpha, const float* gain,
+                             const float* shift, void* y, const int* rows, int n_rows, int T_, int H, int branch_dtype,
+                             int y_dtype, int write_res, hipStream_t stream) {
+  if (n_rows <= 0) return 0;
+  if (H <= 0 || slices < 0 || (slices && !branch)) return ULLM_ERR_SHAPE;
+  const bool vec = H % 4 == 0 && ((uintptr_t)branch | (uintptr_t)residual | (uintptr_t)gain | (uintptr_t)shift | (uintptr_t)y) % 16 == 0;
+  const size_t work = (size_t)n_rows * (vec ? H / 4 : H);
+  const dim3 grid((unsigned)((work + 255) / 256));
+#define GO_V(TB, TY, V) hipLaunchKernelGGL((add_tanh_kernel<TB, TY, V>), grid, dim3(256), 0, stream, (const TB*)branch, slices, mult, \
+    residual, alpha, gain, shift, (TY*)y, rows, n_rows, (long long)T_ * H, H, write_res)
+#define GO(TB, TY) do { if (vec) GO_V(TB, TY, 4); else GO_V(TB, TY, 1); } while (0)
+  if (branch_dtype == ULLM_F32 && y_dtype == ULLM_F32) GO(float, float);
+  else if (branch_dtype == ULLM_BF16 && y_dtype == ULLM_BF16) GO(bf16_t, bf16_t);
+  else if (branch_dtype == ULLM_F32 && y_dtype == ULLM_BF16) GO(float, bf16_t);
+  else if (branch_dtype == ULLM_BF16 && y_dtype == ULLM_F32) GO(bf16_t, float);
+  else return ULLM_ERR_DTYPE;
+#undef GO
+#undef GO_V
+  ULLM_LAUNCH_CHECK();
+}
+
 // Two block sums with one pair of barriers.
 __device__ __forceinline__ void block_sum2(float& a, float& b, float* scratch /* 32 floats */) {
   const int lane = threadIdx.x & (WAVE - 1), wave = threadIdx.x / WAVE;

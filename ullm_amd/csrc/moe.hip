@@ -43,13 +43,13 @@ union Pack8 {
 // mode ROUTE_SIGMOID: every score is the sigmoid of its own logit; choice and weights as for ROUTE_SOFTMAX_ALL.
 // Every weight is multiplied by `weight_scale`.  `raw`: the weights are the chosen scores as they are, not over their sum
 // (not with ROUTE_TOP_LOGITS).  groups > 1: the outputs form that many equal groups of neighbours (at most 64), a group
-// counts as much as the largest choice score in it, and only outputs of the `keep` best groups (ties: the lower
-// index) can be chosen.
+// counts as much as the `group_top` (1 or 2) largest choice scores in it together, and only outputs of the `keep` best
+// groups (ties: the lower index) can be chosen.
 enum { ROUTE_SOFTMAX_ALL = 0, ROUTE_TOP_LOGITS = 1, ROUTE_SIGMOID = 2 };
 __device__ __forceinline__ void route_from_logits(float* z, float* s_choice, float* s_pick,
                                                   const float* __restrict__ correction, int n_router, int top,
                                                   int* __restrict__ ids, float* __restrict__ weights, int lane,
-                                                  int mode, float weight_scale, int groups, int keep, int raw) {
+                                                  int mode, float weight_scale, int groups, int keep, int raw, int group_top) {
   if (mode == ROUTE_TOP_LOGITS) {
     for (int e = lane; e < n_router; e += 64) {
       const float v = z[e] + (correction ? correction[e] : 0.f);
@@ -83,9 +83,14 @@ __device__ __forceinline__ void route_from_logits(float* z, float* s_choice, flo
   __builtin_amdgcn_wave_barrier();
   if (groups > 1) {
     const int size = n_router / groups;
-    float mine = -INFINITY;
+    float mine = -INFINITY, next = -INFINITY;            // the group's two largest choice scores
     if (lane < groups)
-      for (int j = 0; j < size; ++j) mine = fmaxf(mine, s_choice[lane * size + j]);
+      for (int j = 0; j < size; ++j) {
+        const float c = s_choice[lane * size + j];
+        next = fmaxf(next, fminf(mine, c));
+        mine = fmaxf(mine, c);
+      }
+    if (group_top == 2 && size > 1) mine += next;
     int rank = 0;                                        // how many groups come before this lane's
     for (int o = 0; o < groups; ++o) {
       const float other = __shfl(mine, o, 64);
@@ -140,31 +145,31 @@ __device__ __forceinline__ void route_from_logits(float* z, float* s_choice, flo
 
 __global__ void __launch_bounds__(64)
 moe_route_kernel(const float* __restrict__ logits, int ld, const float* __restrict__ correction, int n_router, int top,
-                 int* __restrict__ ids, float* __restrict__ weights, int mode, float weight_scale, int groups, int keep, int raw) {
+                 int* __restrict__ ids, float* __restrict__ weights, int mode, float weight_scale, int groups, int keep, int raw, int group_top) {
   __shared__ float s_soft[MOE_MAX_ROUTER], s_choice[MOE_MAX_ROUTER];
   __shared__ float s_pick[MOE_MAX_TOP];
   const int t = blockIdx.x, lane = threadIdx.x;
   for (int e = lane; e < n_router; e += 64) s_soft[e] = logits[(size_t)t * ld + e];
   __syncthreads();
   route_from_logits(s_soft, s_choice, s_pick, correction, n_router, top, ids + (size_t)t * top, weights + (size_t)t * top, lane,
-                    mode, weight_scale, groups, keep, raw);
+                    mode, weight_scale, groups, keep, raw, group_top);
 }
 
-static bool bad_groups(int n_router, int top, int mode, int groups, int keep, int raw) {
+static bool bad_groups(int n_router, int top, int mode, int groups, int keep, int raw, int group_top) {
   return groups < 1 || groups > 64 || keep < 1 || keep > groups || n_router % groups || top > n_router / groups * keep ||
-         (raw && mode == ROUTE_TOP_LOGITS);
+         (raw && mode == ROUTE_TOP_LOGITS) || (group_top != 1 && group_top != 2);
 }
 
 extern "C" int ullm_moe_route(const float* logits, int ld, const float* correction, int T_, int n_router, int top,
                               int* ids, float* weights, int mode, float weight_scale, int groups, int keep, int raw,
-                              hipStream_t stream) {
+                              int group_top, hipStream_t stream) {
   if (T_ <= 0) return 0;
-  if (bad_groups(n_router, top, mode, groups, keep, raw)) return ULLM_ERR_SHAPE;
+  if (bad_groups(n_router, top, mode, groups, keep, raw, group_top)) return ULLM_ERR_SHAPE;
   if (n_router < 1 || n_router > MOE_MAX_ROUTER || top < 1 || top > MOE_MAX_TOP || top > n_router || ld < n_router)
     return ULLM_ERR_SHAPE;
   if (mode < ROUTE_SOFTMAX_ALL || mode > ROUTE_SIGMOID) return ULLM_ERR_UNSUPPORTED;
   hipLaunchKernelGGL(moe_route_kernel, dim3(T_), dim3(64), 0, stream, logits, ld, correction, n_router, top, ids, weights,
-                     mode, weight_scale, groups, keep, raw);
+                     mode, weight_scale, groups, keep, raw, group_top);
   ULLM_LAUNCH_CHECK();
 }
 
@@ -177,7 +182,7 @@ template <typename T, int TPB>
 __global__ void __launch_bounds__(TPB == 1 ? 1024 : 256)
 moe_router_kernel(const T* __restrict__ x, int ldx, const float* __restrict__ w, const float* __restrict__ correction,
                   int n_tokens, int H, int n_router, int top, int* __restrict__ ids, float* __restrict__ weights, int mode,
-                  float weight_scale, int groups, int keep, int raw) {
+                  float weight_scale, int groups, int keep, int raw, int group_top) {
   extern __shared__ __attribute__((aligned(16))) float xrow[];          // [TPB][H]
   constexpr int RCAP = TPB == 1 ? MOE_MAX_ROUTER : 256;                // router outputs the variant takes
   __shared__ float z[TPB][RCAP], s_choice[TPB][RCAP];
@@ -240,14 +245,14 @@ moe_router_kernel(const T* __restrict__ x, int ldx, const float* __restrict__ w,
   __syncthreads();
   if (wave < TPB && t0 + wave < n_tokens)
     route_from_logits(z[wave], s_choice[wave], s_pick[wave], correction, n_router, top, ids + (size_t)(t0 + wave) * top,
-                      weights + (size_t)(t0 + wave) * top, lane, mode, weight_scale, groups, keep, raw);
+                      weights + (size_t)(t0 + wave) * top, lane, mode, weight_scale, groups, keep, raw, group_top);
 }
 
 extern "C" int ullm_moe_router(const void* x, int ldx, const float* w, const float* correction, int T_, int H,
                                int n_router, int top, int* ids, float* weights, int mode, float weight_scale, int groups, int keep,
-                               int raw, int dtype, hipStream_t stream) {
+                               int raw, int group_top, int dtype, hipStream_t stream) {
   if (T_ <= 0) return 0;
-  if (bad_groups(n_router, top, mode, groups, keep, raw)) return ULLM_ERR_SHAPE;
+  if (bad_groups(n_router, top, mode, groups, keep, raw, group_top)) return ULLM_ERR_SHAPE;
   if (mode < ROUTE_SOFTMAX_ALL || mode > ROUTE_SIGMOID) return ULLM_ERR_UNSUPPORTED;
   if (n_router < 1 || n_router > MOE_MAX_ROUTER || top < 1 || top > MOE_MAX_TOP || top > n_router || H < 1 || ldx < H ||
       (size_t)H * sizeof(float) > 48 * 1024)
@@ -259,7 +264,7 @@ extern "C" int ullm_moe_router(const void* x, int ldx, const float* w, const flo
   // a token a block: sixteen waves, so that up to 64 router outputs are summed in one round of trips to memory
   dim3 grid(four ? (T_ + 3) / 4 : T_), block(four ? 256 : 1024);
 #define GO(TT, N) hipLaunchKernelGGL((moe_router_kernel<TT, N>), grid, block, lds, stream, (const TT*)x, ldx, w, correction, T_, H, \
-    n_router, top, ids, weights, mode, weight_scale, groups, keep, raw)
+    n_router, top, ids, weights, mode, weight_scale, groups, keep, raw, group_top)
   if (dtype == ULLM_F32) { if (four) GO(float, 4); else GO(float, 1); }
   else if (dtype == ULLM_BF16) { if (four) GO(bf16_t, 4); else GO(bf16_t, 1); }
   else return ULLM_ERR_DTYPE;

@@ -31,7 +31,8 @@ HIPCC_FLAGS = [
     "-Wno-unused-command-line-argument",
 ]
 HEADERS = ["common.h"]
-FAMILY_HEADERS = {"attention_mfma": ["no_alloc.h"], "short_conv": ["short_conv.h"], "pooled": ["short_conv.h"]}     # headers only this family includes
+FAMILY_HEADERS = {"attention_mfma": ["no_alloc.h"], "short_conv": ["short_conv.h"], "pooled": ["short_conv.h"],
+                  "matrix_memory": ["short_conv.h"]}     # headers only this family includes
 
 _lock = threading.Lock()
 _loaded: Dict[str, ctypes.CDLL] = {}

@@ -430,6 +430,32 @@ def add_norm_general(branch: Optional[torch.Tensor], residual: torch.Tensor, gai
     return out
 
 
+def add_tanh(branch: Optional[torch.Tensor], residual: torch.Tensor, alpha: torch.Tensor, gain: torch.Tensor, shift: torch.Tensor,
+             out_dtype: torch.dtype, rows: Optional[torch.Tensor] = None, mult: float = 1.0) -> torch.Tensor:
+    """residual (float32 [T, H], in place unless ``rows``) += mult * branch ([T, H], or a stack [S, T, H] of partial sums
+    added in order, or None: nothing); returns tanh(alpha * sum) * gain + shift in ``out_dtype`` (``alpha`` float32, one value
+    on the device; ``gain`` and ``shift`` float32 [H]), for the tokens ``rows`` lists only where it is given."""
+    T, H = residual.shape
+    _need(residual.dtype == torch.float32 and residual.is_contiguous(), "residual must be contiguous float32")
+    for g, n, nm in ((alpha, 1, "alpha"), (gain, H, "gain"), (shift, H, "shift")):
+        _need(g.dtype == torch.float32 and g.numel() == n and g.is_contiguous(), f"{nm} must be float32 with {n} values")
+    slices = 0
+    if branch is not None:
+        _need(branch.shape[-2:] == (T, H) and branch.dim() in (2, 3) and branch.is_contiguous(),
+              "branch must be contiguous [T, H] or a stack [S, T, H]")
+        slices = branch.shape[0] if branch.dim() == 3 else 1
+    n = T
+    if rows is not None:
+        _i32(rows, "rows")
+        n = rows.numel()
+    out = torch.empty((n, H), dtype=out_dtype, device=residual.device)
+    _check(build.load("elementwise").ullm_add_tanh(
+        _p(branch), _c_int(slices), _c_float(mult), _p(residual), _p(alpha), _p(gain), _p(shift), _p(out), _p(rows), _c_int(n), _c_int(T),
+        _c_int(H), _c_int(_dt(branch) if branch is not None else F32), _c_int(_dt(out)), _c_int(0 if rows is not None else 1), _stream()),
+        "add_tanh")
+    return out
+
+
 def post_add(branch: torch.Tensor, residual: torch.Tensor, gain: torch.Tensor, eps: float, out_dtype: Optional[torch.dtype],
              second: Optional[torch.Tensor] = None, a: float = 1.0, b: float = 1.0, conv=None) -> Optional[torch.Tensor]:
     """residual (float32 [T, H], in place) += the RMS norm of a * branch (+ b * second) times ``gain``; returns the new rows in
@@ -742,10 +768,11 @@ def token_shift(x: torch.Tensor, mu: torch.Tensor, state: torch.Tensor, state_of
 
 
 def gated_unit_norm(o: torch.Tensor, gate: torch.Tensor, gain: torch.Tensor, eps: float, parts: int, gate_kind: int,
-                    out_dtype: torch.dtype) -> torch.Tensor:
+                    out_dtype: torch.dtype, den: Optional[torch.Tensor] = None, least: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Rows ``o`` (float32 [T, width], or [slices, T, width] whose slices are added first, in their order) cut into ``parts`` equal parts, each divided by its root mean square (eps inside
     the root), times ``gain`` (float32; as long as a part, shared by the parts, or as long as the row) and times
-    silu or sigmoid (``gate_kind``) of ``gate`` (float32 [T, width], may be a column range of wider rows)."""
+    silu or sigmoid (``gate_kind``) of ``gate`` (float32 [T, width], may be a column range of wider rows).  With ``den`` and
+    ``least`` (float32 [T, parts]) every part is first divided by max(|den|, least) + 1e-6."""
     slices = 1
     if o.dim() == 3:
         slices = o.shape[0]
@@ -755,11 +782,117 @@ def gated_unit_norm(o: torch.Tensor, gate: torch.Tensor, gain: torch.Tensor, eps
     _need(parts >= 1 and width % parts == 0, f"{width} values do not cut into {parts} equal parts")
     _need(gain.dtype == torch.float32 and gain.is_contiguous() and gain.numel() in (width // parts, width),
           "gain must be float32, as long as a part or as the row")
+    if den is not None:
+        _f32_rows(den, "den", T, parts)
+        _f32_rows(least, "least", T, parts)
+        _need(den.is_contiguous(), "den must be contiguous")
     out = torch.empty((T, width), dtype=out_dtype, device=o.device)
     _check(build.load("decay_scan").ullm_gated_unit_norm(
         _p(o), _p(gate), _c_int(gate.stride(0)), _p(gain), _c_int(gain.numel()), _c_float(eps), _c_int(gate_kind), _p(out),
-        _c_int(T), _c_int(width), _c_int(parts), _c_int(slices), _c_int(_dt(out)), _stream()), "gated_unit_norm")
+        _c_int(T), _c_int(width), _c_int(parts), _c_int(slices), _p(den), _p(least),
+        _c_int(least.stride(0) if least is not None else 0), _c_int(_dt(out)), _stream()), "gated_unit_norm")
     return out
+
+
+# ---------------------------------------------------------------------------------- matrix memories with a decay per token
+
+MEMORY_DELTA, MEMORY_SUM = 0, 1          # how a matrix memory takes a token in
+MEMORY_MAX_KEYS = 512                    # key channels a head; a convolved head's value channels too
+
+
+def _check_step(q_start, entry_slot, n_entries: int) -> None:
+    _i32(q_start, "q_start", n_entries + 1)
+    _i32(entry_slot, "entry_slot", n_entries)
+
+
+def matrix_memory(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, keep: torch.Tensor, take: torch.Tensor, rule: int,
+                  state: torch.Tensor, state_off: int, ctx, heads: int, kv_heads: int, key_dim: int, value_dim: int,
+                  q_scale: float = 1.0, norm_off: int = 0, write_state: bool = True):
+    """A recurrence per head over each entry's tokens, with the head's memory S [key_dim, value_dim] (float32, at
+    ``state[slot, state_off + head * key_dim * value_dim ..]``) and one decay ``keep`` and one strength ``take`` per token and
+    head (float32 [T, heads], columns of wider rows).  MEMORY_DELTA: S <- keep S, u = take (v - S^T k), S <- S + k u^T.
+    MEMORY_SUM: S <- keep S + k (take v)^T, and the same with v = 1 for the normaliser n [key_dim] at ``norm_off + head * key_dim``.
+    ``q``, ``k`` (float32 [T, kv_heads * key_dim], head h takes kv head h // (heads // kv_heads)) and ``v`` (float32 [T, heads *
+    value_dim]) may be column ranges of wider rows; q is multiplied by ``q_scale``.  Returns (S^T q float32 [T, heads * value_dim],
+    n . q float32 [T, heads] or None), both after the token's update."""
+    T = q.shape[0]
+    _need(heads % kv_heads == 0, f"{heads} heads are not a multiple of {kv_heads} key heads")
+    _f32_rows(q, "q", T, kv_heads * key_dim)
+    _f32_rows(k, "k", T, kv_heads * key_dim)
+    _f32_rows(v, "v", T, heads * value_dim)
+    _f32_rows(keep, "keep", T, heads)
+    _f32_rows(take, "take", T, heads)
+    _need(keep.stride(0) == take.stride(0), "keep and take must be columns of rows equally far apart")
+    _need(1 <= key_dim <= MEMORY_MAX_KEYS, f"{key_dim} key channels a head: at most {MEMORY_MAX_KEYS}")
+    _check_step_state(state, state_off, heads * key_dim * value_dim, "the memories")
+    if rule == MEMORY_SUM:
+        _check_step_state(state, norm_off, heads * key_dim, "the normalisers")
+    _check_step(ctx.q_start, ctx.entry_slot, ctx.num_entries)
+    _need(not ctx.decode_only or T == ctx.num_entries, "a step of single tokens has as many tokens as entries")
+    ll = ctypes.c_longlong
+    out = torch.empty((T, heads * value_dim), dtype=torch.float32, device=q.device)
+    norm = torch.empty((T, heads), dtype=torch.float32, device=q.device) if rule == MEMORY_SUM else None
+    _check(build.load("matrix_memory").ullm_matrix_memory(
+        _p(q), _c_int(q.stride(0)), _p(k), _c_int(k.stride(0)), _p(v), _c_int(v.stride(0)), _p(keep), _p(take), _c_int(keep.stride(0)),
+        _c_int(rule), _c_float(q_scale), _p(state), ll(state.stride(0)), ll(state_off), ll(norm_off), _p(ctx.q_start),
+        _p(ctx.entry_slot), _p(out), _p(norm), _c_int(ctx.num_entries), _c_int(heads), _c_int(kv_heads), _c_int(key_dim),
+        _c_int(value_dim), _c_int(1 if write_state else 0), _c_int(1 if ctx.decode_only else 0), _stream()), "matrix_memory")
+    return out, norm
+
+
+def delta_prepare(x: torch.Tensor, weight: torch.Tensor, raw_b: torch.Tensor, raw_a: torch.Tensor, a_rate: torch.Tensor,
+                  dt_bias: torch.Tensor, state: torch.Tensor, state_off: int, ctx, heads: int, kv_heads: int, key_dim: int,
+                  value_dim: int, q_scale: float, write_state: bool = True):
+    """Ahead of the delta rule.  ``x`` (float32 [T, channels], columns of wider rows) holds q (kv_heads * key_dim) | k (the same) |
+    v (heads * value_dim); each channel passes a causal convolution over time (``weight`` float32 [taps, channels], the last
+    row is the current token's; the inputs before an entry's first token lie in ``state[slot, state_off ..]``, oldest first) and
+    silu; q and k are then divided by sqrt(sum of squares + 1e-6) per head, and q is multiplied by ``q_scale``.  Returns (the
+    rows float32 [T, channels], gates float32 [T, 2, heads]: exp(-a_rate softplus(raw_a + dt_bias)) and sigmoid(raw_b)); the raw
+    values are columns of rows as far apart as x's."""
+    T, channels = x.shape
+    taps = weight.shape[0]
+    _f32_rows(x, "x", T, 2 * kv_heads * key_dim + heads * value_dim)
+    for t, nm in ((raw_b, "raw_b"), (raw_a, "raw_a")):
+        _f32_rows(t, nm, T, heads)
+        _need(t.stride(0) == x.stride(0), f"{nm} must be columns of the same rows as x")
+    _need(weight.dtype == torch.float32 and weight.shape == (taps, channels) and weight.is_contiguous()
+          and 1 <= taps <= SHORT_CONV_MAX_TAPS, f"weight must be float32 [taps, channels] of at most {SHORT_CONV_MAX_TAPS} taps")
+    for t, nm in ((a_rate, "a_rate"), (dt_bias, "dt_bias")):
+        _need(t.dtype == torch.float32 and t.numel() == heads and t.is_contiguous(), f"{nm} must be float32 [heads]")
+    _need(heads % kv_heads == 0 and max(key_dim, value_dim) <= MEMORY_MAX_KEYS, f"heads of up to {MEMORY_MAX_KEYS} channels")
+    _check_step_state(state, state_off, (taps - 1) * channels, "the convolution's state")
+    _i32(ctx.token_entry, "token_entry", T)
+    _check_step(ctx.q_start, ctx.entry_slot, ctx.num_entries)
+    _need(not ctx.decode_only or T == ctx.num_entries, "a step of single tokens has as many tokens as entries")
+    out = torch.empty((T, channels), dtype=torch.float32, device=x.device)
+    gates = torch.empty((T, 2, heads), dtype=torch.float32, device=x.device)
+    _check(build.load("matrix_memory").ullm_delta_prepare(
+        _p(x), _c_int(x.stride(0)), _p(weight), _p(raw_b), _p(raw_a), _p(a_rate), _p(dt_bias), _p(state[:, state_off:]),
+        ctypes.c_longlong(state.stride(0)), _p(ctx.token_entry), _p(ctx.q_start), _p(ctx.entry_slot), _p(out), _p(gates), _c_int(T),
+        _c_int(ctx.num_entries), _c_int(heads), _c_int(kv_heads), _c_int(key_dim), _c_int(value_dim), _c_int(taps), _c_float(q_scale),
+        _c_int(1 if ctx.decode_only else 0), _c_int(1 if write_state else 0), _stream()), "delta_prepare")
+    return out, gates
+
+
+def exp_gates(raw_i: torch.Tensor, raw_f: torch.Tensor, b_i: torch.Tensor, b_f: torch.Tensor, cap: float, state: torch.Tensor,
+              m_off: int, ctx, write_state: bool = True) -> torch.Tensor:
+    """gates float32 [T, 3, heads] of a memory with exponential gates: with i = cap tanh((raw_i + b_i) / cap), f = log sigmoid(cap
+    tanh((raw_f + b_f) / cap)) and the running maximum m <- max(f + m, i) (from ``state[slot, m_off + head]``, which moves on):
+    keep = exp(f + m_before - m), take = exp(i - m), floor = exp(-m)."""
+    T, heads = raw_i.shape
+    _f32_rows(raw_i, "raw_i", T, heads)
+    _f32_rows(raw_f, "raw_f", T, heads)
+    _need(raw_i.stride(0) == raw_f.stride(0) and cap > 0, "raw_i and raw_f must be columns of the same rows, cap positive")
+    for t, nm in ((b_i, "b_i"), (b_f, "b_f")):
+        _need(t.dtype == torch.float32 and t.numel() == heads and t.is_contiguous(), f"{nm} must be float32 [heads]")
+    _check_step_state(state, m_off, heads, "the running maxima")
+    _check_step(ctx.q_start, ctx.entry_slot, ctx.num_entries)
+    gates = torch.empty((T, 3, heads), dtype=torch.float32, device=raw_i.device)
+    _check(build.load("matrix_memory").ullm_exp_gates(
+        _p(raw_i), _p(raw_f), _c_int(raw_i.stride(0)), _p(b_i), _p(b_f), _c_float(cap), _p(state), ctypes.c_longlong(state.stride(0)),
+        ctypes.c_longlong(m_off), _p(ctx.q_start), _p(ctx.entry_slot), _p(gates), _c_int(ctx.num_entries), _c_int(heads),
+        _c_int(ctx.max_q_len), _c_int(1 if write_state else 0), _stream()), "exp_gates")
+    return gates
 
 
 # ---------------------------------------------------------------------------------- attention
@@ -1113,14 +1246,14 @@ def decode_split(n_items: int, nkv: int, groups: int, max_kv: int, hd: int = 128
     tiles, so short contexts are not cut.  Mostly a block is a single wave (several are resident on a
     SIMD, they start and end independently and one's start overlaps the others' streaming, and their number
     need not be a multiple of the compute units); four waves a block where few pairs have very many keys.
-    With a window a token reads at most the window's keys (and up to 31 before them, to the tile's edge),
+    With a window or a chunk (``window`` < 0) a token reads at most its keys (and up to 31 before them, to the tile's edge),
     however long its context is.  ``units``: the device's compute units, four SIMDs each."""
     pairs = max(1, n_items * nkv * groups)
     simds = 4 * units
     if pairs >= simds:
         return 1, 1
-    if window > 0:
-        max_kv = min(max_kv, window + 31)
+    if window != 0:
+        max_kv = min(max_kv, abs(window) + 31)
     tiles = -(-max_kv // 32)
     if pairs > units:
         # single waves, two to four to a SIMD, so that the launch has no rounds of whole blocks (four-wave blocks,
@@ -1317,7 +1450,8 @@ def paged_attention(q: torch.Tensor, k_pool: torch.Tensor, v_pool: torch.Tensor,
     the one-token entries, one for the tiles of longer entries, both listed in ``plan``: arrays
     ``decode_tokens`` and ``tiles``, numbers ``num_decode``, ``max_decode_kv``, ``num_tiles``,
     ``tile_keys_total``, ``tile_keys_max``); everything else, and float32 always, takes the general
-    kernel.  Every choice computes the same function.  ``bias`` (float32 [nq, rows]) is a bias by distance on the
+    kernel.  Every choice computes the same function.  ``window``: how many keys back a query sees, its own included; 0: all;
+    negative: the keys of its own chunk of ``-window`` positions (all kernels here).  ``bias`` (float32 [nq, rows]) is a bias by distance on the
     scores (``bias_log2``: the same times log2(e), which the matrix-core kernels add to their exponents of two);
     ``gate`` [T, >= nq]: every head's output is multiplied by the sigmoid of its gate; ``sink`` (float32 [nq]):
     exp(sink[head]) joins the softmax's denominator (``sink_log2``: the same times log2(e))."""
@@ -1659,14 +1793,14 @@ MOE_MAX_GROUPS = 64               # groups a router may choose from before it ch
 
 
 def moe_route(logits: torch.Tensor, correction: Optional[torch.Tensor], top: int, mode: int = ROUTE_SOFTMAX_ALL,
-              weight_scale: float = 1.0, groups: int = 1, keep: int = 1, raw: bool = False):
+              weight_scale: float = 1.0, groups: int = 1, keep: int = 1, raw: bool = False, group_top: int = 1):
     """(ids int32 [T, top], weights float32 [T, top]) from router logits float32 [T, R]: the softmax over all R, the
     ``top`` largest of softmax + ``correction`` (float32 [R] or None; ties go to the lower index), and as weights the
     chosen outputs' softmax values over their sum (+ 1e-20).  With ``mode`` ROUTE_TOP_LOGITS: the ``top`` largest of
     logits + ``correction`` (a bias on the logits), weighed by the softmax over those alone.  With ROUTE_SIGMOID the
     scores are the sigmoids of the logits, each on its own; choice and weights as with the softmax.  Every weight is
     multiplied by ``weight_scale``.  ``groups`` > 1: only outputs of the ``keep`` best of that many equal groups of
-    neighbours can be chosen (a group counts as much as the largest choice score in it); ``raw``: the weights are the
+    neighbours can be chosen (a group counts as much as the ``group_top``, 1 or 2, largest choice scores in it together); ``raw``: the weights are the
     chosen scores as they are."""
     T, R = logits.shape
     _need(logits.dtype == torch.float32 and logits.stride(1) == 1, "router logits must be float32 [T, R]")
@@ -1679,7 +1813,7 @@ def moe_route(logits: torch.Tensor, correction: Optional[torch.Tensor], top: int
     weights = torch.empty((T, top), dtype=torch.float32, device=logits.device)
     _check(build.load("moe").ullm_moe_route(_p(logits), _c_int(logits.stride(0)), _p(correction), _c_int(T), _c_int(R),
                                             _c_int(top), _p(ids), _p(weights), _c_int(mode), _c_float(weight_scale),
-                                            _c_int(groups), _c_int(keep), _c_int(1 if raw else 0), _stream()), "moe_route")
+                                            _c_int(groups), _c_int(keep), _c_int(1 if raw else 0), _c_int(group_top), _stream()), "moe_route")
     return ids, weights
 
 
@@ -1687,7 +1821,7 @@ MOE_ROUTER_MAX_WIDTH = 12288      # widest row the fused router kernel keeps in 
 
 
 def moe_router(x: torch.Tensor, w_router: torch.Tensor, correction: Optional[torch.Tensor], top: int,
-               mode: int = ROUTE_SOFTMAX_ALL, weight_scale: float = 1.0, groups: int = 1, keep: int = 1, raw: bool = False):
+               mode: int = ROUTE_SOFTMAX_ALL, weight_scale: float = 1.0, groups: int = 1, keep: int = 1, raw: bool = False, group_top: int = 1):
     """:func:`moe_route` of the 32-bit product of ``x`` [T, H] with ``w_router`` (float32 [R, H]), in one kernel: every
     router output is summed along the row in an order that depends on nothing but the row."""
     T, H = x.shape
@@ -1704,8 +1838,8 @@ def moe_router(x: torch.Tensor, w_router: torch.Tensor, correction: Optional[tor
     weights = torch.empty((T, top), dtype=torch.float32, device=x.device)
     _check(build.load("moe").ullm_moe_router(_p(x), _c_int(x.stride(0)), _p(w_router), _p(correction), _c_int(T), _c_int(H),
                                              _c_int(R), _c_int(top), _p(ids), _p(weights), _c_int(mode), _c_float(weight_scale),
-                                             _c_int(groups), _c_int(keep), _c_int(1 if raw else 0), _c_int(_dt(x)),
-                                             _stream()), "moe_router")
+                                             _c_int(groups), _c_int(keep), _c_int(1 if raw else 0), _c_int(group_top),
+                                             _c_int(_dt(x)), _stream()), "moe_router")
     return ids, weights
 
 

@@ -159,7 +159,7 @@ class Model:
             rows = tuple((r.heads, r.dim, None if r.dtype is None else torch.empty((), dtype=r.dtype).element_size())
                          for r in need.rows) if need.rows else None
             groups.append(CacheGroupSpec(need.num_kv_heads, need.head_dim, need.window, tuple(keys), rows,
-                                         need.tokens_per_row))
+                                         need.tokens_per_row, need.chunk))
         self._group_needs = list(keyed)
         for idx, (layer, cache_id) in enumerate(self.run_order):
             owner_layer = self.run_order[self.cache_owner[cache_id]][0]

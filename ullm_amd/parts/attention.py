@@ -4,7 +4,8 @@ Reference: ullm/models/qwen3.py:49-130 (projection, per-head q/k norm, rotation,
 projection) and ullm/layers/attention.py:279-313 (write k, v to the cache, then attend over it).
 Head size is a parameter of its own (qwen3.py:78: not hidden/heads), the q/k norms and the position
 encoding are optional parts, and a window bounds how far back a query looks (0 = everything; the
-reference never windows).
+reference never windows), or ``chunk`` bounds it to the query's own chunk of so many positions, counted from
+position 0 of the sequence.
 
 Beyond that form the same mixer takes, each as a parameter of its own: a value size that differs from the
 query/key size (``value_dim``), the q/k norm taken over the whole projection instead of per head
@@ -96,9 +97,11 @@ class GQAttention(Mixer):
                  value_dim: Optional[int] = None, qk_norm: str = "head", head_gate: bool = False,
                  own_kv: bool = True, names: Optional[Dict[str, str]] = None, values: str = "own",
                  sink: bool = False, out_bias: bool = False, sink_value: Optional[float] = None,
-                 qk_norm_gain: bool = True):
+                 qk_norm_gain: bool = True, chunk: int = 0):
         if qk_norm not in ("head", "whole"):
             raise ValueError(f"qk_norm={qk_norm!r}: 'head' (per head) or 'whole' (over the whole projection)")
+        if chunk < 0 or (chunk and window):
+            raise ValueError(f"chunk={chunk} with window={window}: a query looks back over a window or its own chunk, not both")
         if values not in ("own", "keys"):
             raise ValueError(f"values={values!r}: 'own' (a value projection) or 'keys' (the keys as projected)")
         self.dim, self.vdim = head_dim, head_dim if value_dim is None else int(value_dim)
@@ -129,7 +132,8 @@ class GQAttention(Mixer):
         self.position = position
         self.qk_norm_eps = qk_norm_eps          # None: no per-head norm
         self.bias = bias
-        self.window = int(window)
+        self.window, self.chunk = int(window), int(chunk)
+        self.reach = -self.chunk if self.chunk else self.window         # what the kernels take as `window`
         self.scale = float(scale) if scale is not None else self.dim ** -0.5   # qwen3.py:81
         self.w_qkv = self.b_qkv = self.w_o = self.b_o = self.q_gain = self.k_gain = None
         self.sinks = self.sinks_log2 = None
@@ -138,7 +142,7 @@ class GQAttention(Mixer):
         return [self.position] if self.position is not None else []
 
     def cache_need(self):
-        return KVNeed(self.nkv, self.hd, self.window)
+        return KVNeed(self.nkv, self.hd, self.window, chunk=self.chunk)
 
     def weights(self) -> List[WeightDecl]:
         if self.general:
@@ -202,7 +206,7 @@ class GQAttention(Mixer):
             ops.attention_decode_fused(
                 qkv, out, self.q_gain, self.k_gain, eps, table, rot, style, cache.k_pool, cache.v_pool,
                 plan.arrays["decode_tokens"], work["num_decode"], ctx.positions, ctx.token_entry, group.block_table,
-                group.page_size, self.nq, self.nkv, self.hd, self.scale, self.window, work["max_decode_kv"],
+                group.page_size, self.nq, self.nkv, self.hd, self.scale, self.reach, work["max_decode_kv"],
                 write_kv=cache.owner)
             return out
         q = torch.empty((T, self.nq * self.hd), dtype=x.dtype, device=x.device)
@@ -211,7 +215,7 @@ class GQAttention(Mixer):
             table, rot, style, ctx.positions, ctx.token_entry, group.block_table,
             cache.k_pool, cache.v_pool, group.page_size, self.nq, self.nkv, self.hd, write_kv=cache.owner)
         return ops.paged_attention(q, cache.k_pool, cache.v_pool, ctx, group, self.nq, self.nkv, self.hd,
-                                   self.scale, self.window, plan)
+                                   self.scale, self.reach, plan)
 
     # ------------------------------------------------------------------ the general path
     def _name(self, role: str) -> str:
@@ -324,7 +328,7 @@ class GQAttention(Mixer):
                                     nq, nkv, hd, has_kv=self.own_kv)
         bias = self.position.score_bias() if self.position is not None else None
         # the bias joins the scores and the gate the heads' outputs inside the attention kernels
-        out = ops.paged_attention(q, cache.k_pool, cache.v_pool, ctx, group, nq, nkv, hd, self.scale, self.window,
+        out = ops.paged_attention(q, cache.k_pool, cache.v_pool, ctx, group, nq, nkv, hd, self.scale, self.reach,
                                   ctx.plans["attention"], bias=bias,
                                   bias_log2=self.position.score_bias_log2() if bias is not None else None,
                                   gate=proj[:, self.gate_off:] if self.head_gate else None,

@@ -70,6 +70,7 @@ class KVNeed:
     window: int = 0               # keys a query looks back over, itself included; 0 = all
     rows: Tuple[CacheRows, ...] = ()
     tokens_per_row: int = 1       # > 1: one row per this many tokens (row b stands for tokens b*n .. b*n + n - 1)
+    chunk: int = 0                # > 0: a query sees the keys of its own chunk of this many positions alone (no window then)
 
     def pools(self) -> Tuple[CacheRows, ...]:
         if self.rows:

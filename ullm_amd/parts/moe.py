@@ -13,7 +13,7 @@ alone; ``routing="sigmoid"`` scores every output by the sigmoid of its own logit
 weighs by the chosen scores over their sum (+ 1e-20); ``weight_scale`` multiplies every weight; ``limit=None`` makes
 every expert the plain gated unit ``silu(g) * u``; ``renormalize=False`` takes the chosen scores as weights as they are;
 ``groups`` and ``keep_groups``: the router's outputs form that many equal groups of neighbours, and only outputs of the
-best ``keep_groups`` (by their largest choice score) can be chosen.
+best ``keep_groups`` can be chosen (a group counts as much as its ``group_top`` largest choice scores together: one or two).
 
 The experts' matrices are stacked ([experts, 2 ff, hidden] with gate rows, then up rows, per expert, and
 [experts, hidden, ff]); the loader puts the checkpoint's per-expert tensors into their rows.  A step groups
@@ -53,7 +53,7 @@ class RoutedExperts(FeedForward):
                  prefix: str, identity: int = 0, alpha: float = 1.702, correction: bool = True,
                  shared_size: int = 0, shared_limit: Optional[float] = None, names: Optional[Dict[str, str]] = None,
                  routing: str = "softmax_all", weight_scale: float = 1.0, renormalize: bool = True, groups: int = 1,
-                 keep_groups: Optional[int] = None):
+                 keep_groups: Optional[int] = None, group_top: int = 1):
         modes = {"softmax_all": ops.ROUTE_SOFTMAX_ALL, "top_logits": ops.ROUTE_TOP_LOGITS, "sigmoid": ops.ROUTE_SIGMOID}
         if routing not in modes:
             raise ValueError(f"routing={routing!r}: one of {sorted(modes)}")
@@ -66,6 +66,9 @@ class RoutedExperts(FeedForward):
                 or top > outputs // self.groups * self.keep_groups:
             raise ValueError(f"{outputs} router outputs in {groups} equal groups (at most {ops.MOE_MAX_GROUPS}) of which "
                              f"{self.keep_groups} are kept, {top} chosen")
+        if group_top not in (1, 2):
+            raise ValueError(f"group_top={group_top}: a group counts as much as its largest choice score or its two largest")
+        self.group_top = int(group_top)
         limit = 0.0 if limit is None else limit            # the kernels read a limit of 0 as the plain unit
         if experts < 0 or identity < 0 or experts + identity < 1:
             raise ValueError(f"{experts} experts and {identity} identity experts: a router needs at least one output")
@@ -124,10 +127,10 @@ class RoutedExperts(FeedForward):
         """(ids int32 [T, top], weights float32 [T, top]) of the rows of x."""
         if self.hidden_size <= ops.MOE_ROUTER_MAX_WIDTH:
             return ops.moe_router(x, self.w_router, self.correction, self.top, self.mode, self.weight_scale,     # the product and the routing in one
-                                  self.groups, self.keep_groups, self.raw)
+                                  self.groups, self.keep_groups, self.raw, self.group_top)
         logits = ops.gemm_simple(x, self.w_router, out_dtype=torch.float32)       # 32-bit sums in a fixed order
         return ops.moe_route(logits, self.correction, self.top, self.mode, self.weight_scale, self.groups, self.keep_groups,
-                             self.raw)
+                             self.raw, self.group_top)
 
     def forward(self, x: torch.Tensor, ctx: StepContext) -> torch.Tensor:
         return self.forward_onto(x, ctx, None, None)

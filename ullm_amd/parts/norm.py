@@ -1,4 +1,4 @@
-"""RMS norm fused with the residual add (reference: ullm/layers/layernorm.py:15-34).
+"""Norms of the residual stream, each fused with the add of what is pending.  RMS norm (reference: ullm/layers/layernorm.py:15-34).
 
 The reference carries the residual in the model dtype and rounds the 32-bit sum once per add
 (layernorm.py:25-26); here the residual stream itself stays 32-bit, so the sum is never rounded.
@@ -93,3 +93,37 @@ class LayerNorm(Norm):
         if out_dtype is None:
             out_dtype = branch.dtype if branch is not None else torch.float32
         return ops.add_norm_general(branch, residual, self.gain, self.eps, ops.NORM_LAYER, out_dtype, rows=rows)
+
+
+@register_part("norm", "dynamic_tanh")
+class DynamicTanh(Norm):
+    """tanh(alpha * x) * gain + shift, in 32-bit: an elementwise squashing in a norm's place, without statistics of the row.
+    ``alpha`` is one learned number, ``gain`` and ``shift`` are as long as the row; the tensors are ``weight_name``,
+    ``<weight_name>.alpha`` and ``<weight_name>.b`` (or what ``alpha_name`` and ``shift_name`` say)."""
+    adds_stacks = True
+
+    def __init__(self, size: int, weight_name: str, alpha_name: Optional[str] = None, shift_name: Optional[str] = None):
+        self.size, self.weight_name = size, weight_name
+        self.alpha_name = alpha_name or f"{weight_name}.alpha"
+        self.shift_name = shift_name or f"{weight_name}.b"
+        self.alpha = self.gain = self.shift = None
+
+    def weights(self) -> List[WeightDecl]:
+        return [WeightDecl(self.weight_name, (self.size,), init="gain", keep_fp32=True),
+                WeightDecl(self.alpha_name, (), init="gain", keep_fp32=True),
+                WeightDecl(self.shift_name, (self.size,), keep_fp32=True)]
+
+    def bind(self, tensors: Dict[str, torch.Tensor], env: PartEnv) -> None:
+        self.gain, self.shift = tensors[self.weight_name].contiguous(), tensors[self.shift_name].contiguous()
+        self.alpha = tensors[self.alpha_name].contiguous()
+
+    def add_norm(self, branch, residual, rows=None, out_dtype=None):
+        mult = 1.0
+        if isinstance(branch, NormedBranch):
+            if branch.post is not None:
+                raise TypeError("dynamic_tanh adds a branch as it is: no norm can stand behind it")
+            mult = branch.mult
+            branch = branch.branch if branch.second is None else branch.joined()
+        if out_dtype is None:
+            out_dtype = branch.dtype if branch is not None and branch.dim() == 2 else torch.float32
+        return ops.add_tanh(branch, residual, self.alpha, self.gain, self.shift, out_dtype, rows=rows, mult=mult)
