@@ -55,7 +55,7 @@ def parse_args():
                     help="instead of the default workload: Pamopel (attention with a distance bias and head gates, a "
                          "layer on another's keys and values, a Mamba-2 layer) beside a Qwen3 stack of the same width, "
                          f"heads, feed-forward, vocabulary and depth, random weights; shapes: {sorted(DESIGN_SHAPES)}")
-    ap.add_argument("--design-model", choices=("both", "all", "pamopel", "qwen3", "ziferax", "dovisun", "kumudra", "nadevik"), default="both",
+    ap.add_argument("--design-model", choices=("both", "all", "pamopel", "qwen3", "ziferax", "dovisun", "kumudra", "nadevik", "risolorn"), default="both",
                     help="with --design: one design only (for profiles), Pamopel and Qwen3 (both), or these, Ziferax "
                          "(a stack of parallel blocks of windowed attention with sinks and a routed feed-forward) and "
                          "Dovisun (parallel blocks of unit-norm attention with a fixed sink or latent attention, dense "
@@ -63,7 +63,8 @@ def parse_args():
                          "stream, gated linear attention, lightning attention and windowed attention beside time "
                          "mixing, four layers passed twice) and Nadevik (norms behind the sublayers, sigmoid attention "
                          "over a window and pooled blocks beside a selective scan, windowed latent attention, experts "
-                         "from the best groups) (all)")
+                         "from the best groups) and Risolorn (parallel blocks behind a dynamic tanh: the gated delta "
+                         "rule, a matrix memory with exponential gates, attention in chunks with sinks) (all)")
     ap.add_argument("--prefill-only", type=int, default=0, metavar="T",
                     help="only time a T-token prompt and print its figures (for profiling)")
     return ap.parse_args()
@@ -235,13 +236,29 @@ def nadevik_config(shape):
                 embedding=dict(scale=float(W) ** 0.5, bigram=dict(buckets=65521, mul_prev=8191, mul_cur=127)))
 
 
+# Risolorn at a design shape: the same width, heads and depth.  Of every four layers one is a matrix memory with exponential
+# gates and two are the gated delta rule (heads of the head size, as many states as Kumudra's lightning layers have; the
+# other stacks' key heads, four taps), one attention (the other stacks' heads, chunks of 1024 positions, sinks, half of each
+# head rotated, stretched).  Every feed-forward is routed, with as many columns a token as the dense stack's (top 4 of 32
+# experts of a sixth of it, in four groups of which three are kept).
+def risolorn_config(shape):
+    (W, H, G, D, F, L), _ = DESIGN_SHAPES[shape]
+    mlp = dict(kind="moe", router=dict(experts=32, top=4, groups=dict(count=4, keep=3)), expert=dict(ff=F // 6))
+    delta = dict(type="delta", mlp=mlp, mixer=dict(heads=H, kv_heads=G, dim=D, vdim=D, conv=4))
+    memory = dict(type="mlstm", mlp=mlp, mixer=dict(heads=H, dim=D, vdim=D, gate_cap=10.0))
+    rot = dict(base=500000.0, dims=D // 2, scaling=dict(factor=8.0, original=4096, fast=32.0, slow=1.0))
+    att = dict(type="attention", mlp=mlp, mixer=dict(heads=H, kv_heads=G, dim=D, vdim=D, scale=D ** -0.5, mask=dict(size=1024), rot=rot))
+    return dict(architecture="Risolorn", vocab=DESIGN_VOCAB, width=W, norm=dict(eps=1e-6), embedding=dict(scale=1.0), logit_scale=0.7,
+                layers=[(memory, delta, att, delta)[i % 4] for i in range(L)])
+
+
 def design_run(args):
     """Decode at batch 1 / 8 / 64 (1024-token prompts) and one 2048-token prompt, for the designs of a shape."""
     out = {"metric": f"decode and prefill tok/s, designs beside Qwen3 at shape {args.design}, random weights",
            "unit": "tokens/s", "dtype": args.dtype, "data": "synthetic", "shape": args.design, "designs": {}}
     configs = design_configs(args.design) + (ziferax_config(args.design), dovisun_config(args.design), kumudra_config(args.design),
-                                             nadevik_config(args.design))
-    for label, config in zip(("pamopel", "qwen3", "ziferax", "dovisun", "kumudra", "nadevik"), configs):
+                                             nadevik_config(args.design), risolorn_config(args.design))
+    for label, config in zip(("pamopel", "qwen3", "ziferax", "dovisun", "kumudra", "nadevik", "risolorn"), configs):
         if args.design_model not in ("both", "all", label) or (label not in ("pamopel", "qwen3") and args.design_model == "both"):
             continue
         m = Sized(label, args.dtype, 4096, eager=args.eager, config=config)

@@ -232,6 +232,7 @@ def test_parts_are_found_by_name_and_unknown_names_fail():
     assert "toy_running_mean" in registered_parts("mixer") and "gqa_attention" in registered_parts("mixer")
     assert "toy_keys_only" in registered_parts("mixer")
     assert "swiglu" in registered_parts("ffn") and registered_parts("block") == ["hyper_prenorm", "mix_in_embedding", "parallel", "postnorm", "prenorm", "sandwich", "toy_two_mixers"]
+    assert "dynamic_tanh" in registered_parts("norm") and "gated_delta_rule" in registered_parts("mixer") and "exp_gated_memory" in registered_parts("mixer")
     assert "routed_experts" in registered_parts("ffn") and "mlp" in registered_parts("ffn") and "latent_attention" in registered_parts("mixer")
     assert "mamba2" in registered_parts("mixer") and "selective_scan" in registered_parts("mixer") and "pooled_attention" in registered_parts("mixer") and "layernorm" in registered_parts("norm")
     assert "table_sum" in registered_parts("embedding") and "log_distance_bias" in registered_parts("position")

@@ -28,7 +28,7 @@ __device__ __forceinline__ void memory_barrier_shared() {
 #endif
 }
 
-// The sum over the 16 lanes of a row, in every one of them, by rotations inside the vector unit.
+// The sum over a row of 16 lanes in every one of them, by four rotations inside the vector unit.
 template <int CTRL>
 __device__ __forceinline__ float row_rotated(float v) {
 #ifdef __HIP_DEVICE_COMPILE__
@@ -37,11 +37,18 @@ __device__ __forceinline__ float row_rotated(float v) {
   return v;
 #endif
 }
-__device__ __forceinline__ float row16_sum(float v) {
-  v += row_rotated<0x128>(v);
-  v += row_rotated<0x124>(v);
-  v += row_rotated<0x122>(v);
-  v += row_rotated<0x121>(v);
+template <int STEP>
+__device__ __forceinline__ void row_sum_step(float& v) {
+  if constexpr (STEP == 0) v += row_rotated<0x128>(v);
+  if constexpr (STEP == 1) v += row_rotated<0x124>(v);
+  if constexpr (STEP == 2) v += row_rotated<0x122>(v);
+  if constexpr (STEP == 3) v += row_rotated<0x121>(v);
+}
+__device__ __forceinline__ float row_sum(float v) {
+  row_sum_step<0>(v);
+  row_sum_step<1>(v);
+  row_sum_step<2>(v);
+  row_sum_step<3>(v);
   return v;
 }
 
@@ -57,35 +64,41 @@ struct MemoryArgs {
   const int* entry_slot;
   float* out;               // [T, heads * P]
   float* norm_out;          // [T, heads]: n . q (RULE_SUM)
-  int q_ld, k_ld, v_ld, gate_ld;
+  int q_ld, k_ld, v_ld, gate_ld;      // q_ld == k_ld in steps with portions
   int heads, kv_heads, N, P, write_state;
   float q_scale;
 };
 
 // ------------------------------------------------------------------ portions of prompts
-// One block of W waves per (entry, head, slice of 4 W value columns); with RULE_SUM the column behind the last is the
-// normaliser.  Lane (r, c) = (lane % 16, lane / 16) of a wave keeps NPT rows of column c in registers; the sixteen
-// lanes of a column hold its 16 NPT >= N rows and add up by rotations inside the wave, so no sum crosses waves and no
-// token waits for a barrier.  An entry's tokens are walked in chunks of CH: the chunk's q, k, v, g and b lie in shared memory, the
-// next chunk's are fetched into registers before the current one is worked on and put into the other buffer
-// afterwards; a token's values are read a token ahead.  Lane r keeps token r's result until the chunk's end.
-template <int W, int NPT, bool DELTA, bool VEC>
-__global__ void __launch_bounds__(64 * W)
+// One block of four waves per (entry, head, slice of 16 value columns); with RULE_SUM the column behind the last is the
+// normaliser.  Lane (r, c) = (lane % 16, lane / 16) of a wave keeps NPT rows of column c in registers; the sixteen lanes
+// of a column hold its 16 NPT >= N rows and add up inside the wave, so no sum crosses waves and no token waits for a
+// barrier.  An entry's tokens are walked in chunks of CH: the chunk's q, k, v, g and b lie in shared memory, the next
+// chunk's are fetched into registers before the current one is worked on and put into the other buffer afterwards; a
+// token's values are read two tokens ahead.  A token's read-out is formed while the next token's S^T k is on its way
+// through the lanes (both read the same S), in an order the source fixes.  Lane r keeps token r's result until the chunk's end.  Tokens past the entry's end
+// repeat its last token's values with b = 0 and g = 1, which changes nothing.
+template <int NPT, bool DELTA, bool VEC>
+__global__ void __launch_bounds__(256)
 memory_scan_kernel(const MemoryArgs a) {
-  constexpr int NP = 16 * NPT;                       // padded key channels
-  constexpr int CH = NPT > 16 ? 4 : NPT > 8 ? 8 : 16;
-  constexpr int COLS = 4 * W, THREADS = 64 * W;
+  constexpr int W = 4, LANES = 16;
+  constexpr int NP = LANES * NPT;                    // padded key channels
+  constexpr int CH = NP > 256 ? 4 : NP > 128 ? 8 : 16;
+  constexpr int WC = 64 / LANES;                     // columns of a wave
+  constexpr int COLS = WC * W, THREADS = 64 * W;
   constexpr int ROW = 2 * NP + COLS + 4;             // a token's q | k | v | g b
-  constexpr int QK_PIECES = CH * 2 * NP / 4;         // pieces of four channels
-  constexpr int PER = (QK_PIECES + THREADS - 1) / THREADS;
+  constexpr int TOK_PIECES = NP / 2;                 // pieces of four channels of a token's q | k
+  constexpr int PER = CH * TOK_PIECES > THREADS ? CH * TOK_PIECES / THREADS : 1;
+  constexpr int STEP = THREADS / TOK_PIECES;         // tokens between a thread's pieces
   constexpr int V_PER = (CH * COLS + THREADS - 1) / THREADS;
-  static_assert(QK_PIECES % THREADS == 0 || QK_PIECES < THREADS, "whole rounds of pieces");
+  static_assert(THREADS % TOK_PIECES == 0, "a thread's pieces lie in one place of different tokens");
+  static_assert(ROW % 4 == 0 && COLS % 4 == 0, "16-byte pieces");
   __shared__ __attribute__((aligned(16))) float buf[2][CH * ROW];
   const int b = blockIdx.x, h = blockIdx.y, c0 = blockIdx.z * COLS;
-  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, r = lane & 15, cw = lane >> 4;
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, r = lane % LANES, cw = lane / LANES;
   const int N = a.N, P = a.P;
   const int kvh = h / (a.heads / a.kv_heads);
-  const int col = c0 + 4 * wave + cw;
+  const int col = c0 + WC * wave + cw;
   const bool live_col = col < P || (!DELTA && col == P);
   const int first = a.q_start[b], end = a.q_start[b + 1];
   if (first >= end) return;
@@ -94,7 +107,7 @@ memory_scan_kernel(const MemoryArgs a) {
   float* column = col < P ? row + a.state_off + (size_t)h * N * P + col : row + a.norm_off + (size_t)h * N;
   const int row_step = col < P ? P : 1;
   auto row_of = [&](int i) __attribute__((always_inline)) {
-    return NPT % 4 == 0 ? (i / 4) * 64 + 4 * r + i % 4 : r * NPT + i;
+    return NPT % 4 == 0 ? (i / 4) * (4 * LANES) + 4 * r + i % 4 : r * NPT + i;
   };
   float s[NPT];
 #pragma unroll
@@ -102,54 +115,64 @@ memory_scan_kernel(const MemoryArgs a) {
     const int n = row_of(i);
     s[i] = (live_col && n < N) ? column[(size_t)n * row_step] : 0.f;
   }
+  // staging: this thread brings channels n .. n + 3 of q or of k for the tokens tl, tl + STEP, ..
+  const int tl = tid / TOK_PIECES, which = (tid / (NP / 4)) & 1, n = 4 * (tid % (NP / 4));
+  const float* src = (which ? a.k : a.q) + (size_t)kvh * N;
+  mem_f32x4 factor;                                  // q's scale, zero for channels past N
+#pragma unroll
+  for (int j = 0; j < 4; ++j) factor[j] = n + j < N ? (which ? 1.f : a.q_scale) : 0.f;
+  if constexpr (VEC) src += n < N ? n : 0;
+  const int v_col = c0 + tid % COLS;
+  const float* src_v = a.v + (size_t)h * P + (v_col < P ? v_col : P - 1);
+  const float* src_g = (tid & 1 ? a.take : a.keep) + h;
   mem_f32x4 raw[PER];
   float raw_v[V_PER], raw_g = 1.f;
-  const float* q = a.q + (size_t)kvh * N;
-  const float* k = a.k + (size_t)kvh * N;
-  // every load is issued whatever it is for (an index past the end reads a valid element again; the value is
-  // replaced on its way into shared memory), so that all of them are on their way at once
-  auto fetch = [&](int t0) __attribute__((always_inline)) {
+  auto piece = [&](const float* p) __attribute__((always_inline)) {
+    mem_f32x4 x;
+    if constexpr (VEC) {
+      x = *reinterpret_cast<const mem_f32x4*>(p);
+    } else {
 #pragma unroll
-    for (int i = 0; i < PER; ++i) {
-      const int e = i * THREADS + tid;
-      const int tl = e / (NP / 2), which = (e / (NP / 4)) & 1, n = 4 * (e % (NP / 4));
-      const int tok = t0 + tl < end ? t0 + tl : end - 1;
-      const float* src = which ? k + (size_t)tok * a.k_ld : q + (size_t)tok * a.q_ld;
-      if constexpr (VEC) {
-        raw[i] = *reinterpret_cast<const mem_f32x4*>(src + (n < N ? n : 0));
-      } else {
-#pragma unroll
-        for (int j = 0; j < 4; ++j) raw[i][j] = src[n + j < N ? n + j : N - 1];
-      }
+      for (int j = 0; j < 4; ++j) x[j] = p[n + j < N ? n + j : N - 1];
     }
+    return x;
+  };
+  // every load is issued whatever it is for, so that all of them are on their way at once; whole chunks step through
+  // memory evenly, the last one may not read past the entry's end
+  auto fetch = [&](int t0) __attribute__((always_inline)) {
+    if (t0 + CH <= end) {
+      const float* p = src + (size_t)(t0 + tl % CH) * a.q_ld;
 #pragma unroll
-    for (int i = 0; i < V_PER; ++i) {
-      const int e = i * THREADS + tid, tl = e / COLS, c = c0 + e % COLS;
-      const int tok = t0 + tl < end ? t0 + tl : end - 1;
-      raw_v[i] = a.v[(size_t)tok * a.v_ld + (size_t)h * P + (c < P ? c : P - 1)];
+      for (int i = 0; i < PER; ++i) raw[i] = piece(p + (size_t)(i * STEP) * a.q_ld);
+      const float* pv = src_v + (size_t)(t0 + (tid / COLS) % CH) * a.v_ld;
+#pragma unroll
+      for (int i = 0; i < V_PER; ++i) raw_v[i] = pv[(size_t)(i * (THREADS / COLS)) * a.v_ld];
+    } else {
+#pragma unroll
+      for (int i = 0; i < PER; ++i) {
+        const int tok = t0 + tl + i * STEP < end ? t0 + tl + i * STEP : end - 1;
+        raw[i] = piece(src + (size_t)tok * a.q_ld);
+      }
+#pragma unroll
+      for (int i = 0; i < V_PER; ++i) {
+        const int tok = t0 + tid / COLS + i * (THREADS / COLS) < end ? t0 + tid / COLS + i * (THREADS / COLS) : end - 1;
+        raw_v[i] = src_v[(size_t)tok * a.v_ld];
+      }
     }
     if (tid < 2 * CH) {
       const int tok = t0 + (tid >> 1) < end ? t0 + (tid >> 1) : end - 1;
-      raw_g = (tid & 1 ? a.take : a.keep)[(size_t)tok * a.gate_ld + h];
+      raw_g = src_g[(size_t)tok * a.gate_ld];
     }
   };
-  // tokens past the entry's end: k = 0, b = 0 and g = 1, which changes nothing
   auto put = [&](int t0, float* dst) __attribute__((always_inline)) {
+    float* to = dst + tl * ROW + which * NP + n;
 #pragma unroll
-    for (int i = 0; i < PER; ++i) {
-      const int e = i * THREADS + tid;
-      if (QK_PIECES % THREADS && e >= QK_PIECES) break;
-      const int tl = e / (NP / 2), which = (e / (NP / 4)) & 1, n = 4 * (e % (NP / 4));
-      const bool live = t0 + tl < end;
-      mem_f32x4 x = raw[i];
-#pragma unroll
-      for (int j = 0; j < 4; ++j) x[j] = (live && n + j < N) ? (which ? x[j] : x[j] * a.q_scale) : 0.f;
-      *reinterpret_cast<mem_f32x4*>(dst + tl * ROW + which * NP + n) = x;
-    }
+    for (int i = 0; i < PER; ++i)
+      if (CH * TOK_PIECES >= THREADS || tl < CH) *reinterpret_cast<mem_f32x4*>(to + i * STEP * ROW) = raw[i] * factor;
 #pragma unroll
     for (int i = 0; i < V_PER; ++i) {
-      const int e = i * THREADS + tid, tl = e / COLS, c = c0 + e % COLS;
-      if (tl < CH) dst[tl * ROW + 2 * NP + e % COLS] = (t0 + tl < end && c <= P) ? ((!DELTA && c == P) ? 1.f : (c < P ? raw_v[i] : 0.f)) : 0.f;
+      const int at = tid / COLS + i * (THREADS / COLS);
+      if (CH * COLS >= THREADS || at < CH) dst[at * ROW + 2 * NP + tid % COLS] = (!DELTA && v_col == P) ? 1.f : raw_v[i];
     }
     if (tid < 2 * CH) dst[(tid >> 1) * ROW + 2 * NP + COLS + (tid & 1)] = t0 + (tid >> 1) < end ? raw_g : (tid & 1 ? 0.f : 1.f);
   };
@@ -157,39 +180,69 @@ memory_scan_kernel(const MemoryArgs a) {
     float q[NPT], k[NPT];
     float v, g, b;
   };
-  auto read_token = [&](const float* src, TokenIn& in) __attribute__((always_inline)) {
+  auto read_token = [&](const float* from, TokenIn& in) __attribute__((always_inline)) {
     if constexpr (NPT % 4 == 0) {
 #pragma unroll
       for (int i = 0; i < NPT; i += 4) {
-        const mem_f32x4 kk = *reinterpret_cast<const mem_f32x4*>(src + NP + 16 * i + 4 * r);
-        const mem_f32x4 qq = *reinterpret_cast<const mem_f32x4*>(src + 16 * i + 4 * r);
+        const mem_f32x4 kk = *reinterpret_cast<const mem_f32x4*>(from + NP + LANES * i + 4 * r);
+        const mem_f32x4 qq = *reinterpret_cast<const mem_f32x4*>(from + LANES * i + 4 * r);
 #pragma unroll
         for (int j = 0; j < 4; ++j) in.k[i + j] = kk[j], in.q[i + j] = qq[j];
       }
     } else {
 #pragma unroll
-      for (int i = 0; i < NPT; ++i) in.k[i] = src[NP + r * NPT + i], in.q[i] = src[r * NPT + i];
+      for (int i = 0; i < NPT; ++i) in.k[i] = from[NP + r * NPT + i], in.q[i] = from[r * NPT + i];
     }
-    in.v = src[2 * NP + 4 * wave + cw];
-    const mem_f32x2 gb = *reinterpret_cast<const mem_f32x2*>(src + 2 * NP + COLS);
+    in.v = from[2 * NP + WC * wave + cw];
+    const mem_f32x2 gb = *reinterpret_cast<const mem_f32x2*>(from + 2 * NP + COLS);
     in.g = gb.x, in.b = gb.y;
   };
   auto dot = [&](const float* x) __attribute__((always_inline)) {
-    float lo = 0.f, hi = 0.f;
+    float lo = s[0] * x[0], hi = NPT > 1 ? s[NPT > 1 ? 1 : 0] * x[NPT > 1 ? 1 : 0] : 0.f;
 #pragma unroll
-    for (int i = 0; i < NPT; i += 2) {
-      lo += s[i] * x[i];
-      if (i + 1 < NPT) hi += s[i + 1] * x[i + 1];
-    }
+    for (int i = 2; i < NPT; i += 2) lo += s[i] * x[i], hi += s[i + 1] * x[i + 1];
     return lo + hi;
   };
-  auto move = [&](const TokenIn& in) __attribute__((always_inline)) {
-    float u;
-    if constexpr (DELTA) u = in.b * (in.v - in.g * row16_sum(dot(in.k)));
-    else u = in.b * in.v;
+#define KEEP_ORDER __builtin_amdgcn_sched_barrier(0)
+  // one token, and the read-out of the token before (the S it left is the one this token finds)
+  auto move = [&](const TokenIn& in, const TokenIn& before) __attribute__((always_inline)) {
+    float o;
+    if constexpr (DELTA) {
+      float p = dot(in.k);
+      KEEP_ORDER;
+      row_sum_step<0>(p);
+      o = dot(before.q);
+      KEEP_ORDER;
+      row_sum_step<1>(p);
 #pragma unroll
-    for (int i = 0; i < NPT; ++i) s[i] = in.g * s[i] + in.k[i] * u;
-    return row16_sum(dot(in.q));
+      for (int i = 0; i < NPT / 2; ++i) s[i] *= in.g;
+      KEEP_ORDER;
+      row_sum_step<2>(p);
+#pragma unroll
+      for (int i = NPT / 2; i < NPT; ++i) s[i] *= in.g;
+      KEEP_ORDER;
+      row_sum_step<3>(p);
+      row_sum_step<0>(o);
+      KEEP_ORDER;
+      row_sum_step<1>(o);
+      KEEP_ORDER;
+      const float u = in.b * (in.v - in.g * p);
+#pragma unroll
+      for (int i = 0; i < NPT / 2; ++i) s[i] = fmaf(in.k[i], u, s[i]);
+      row_sum_step<2>(o);
+      KEEP_ORDER;
+#pragma unroll
+      for (int i = NPT / 2; i < NPT; ++i) s[i] = fmaf(in.k[i], u, s[i]);
+      row_sum_step<3>(o);
+      KEEP_ORDER;
+    } else {
+      o = dot(before.q);
+      const float u = in.b * in.v;
+#pragma unroll
+      for (int i = 0; i < NPT; ++i) s[i] = fmaf(in.k[i], u, in.g * s[i]);
+      o = row_sum(o);
+    }
+    return o;
   };
   fetch(first);
   put(first, buf[0]);
@@ -199,18 +252,19 @@ memory_scan_kernel(const MemoryArgs a) {
     const float* cur = buf[turn];
     const bool more = t0 + CH < end;
     if (more) fetch(t0 + CH);
-    TokenIn in_a, in_b;
+    TokenIn in[4];
     float kept = 0.f;
-    read_token(cur, in_a);
+    read_token(cur, in[0]);
+    read_token(cur + ROW, in[1]);
 #pragma unroll
-    for (int t = 0; t < CH; t += 2) {
-      read_token(cur + (t + 1) * ROW, in_b);
-      const float oa = move(in_a);
-      kept = r == t ? oa : kept;
-      if (t + 2 < CH) read_token(cur + (t + 2) * ROW, in_a);
-      const float ob = move(in_b);
-      kept = r == t + 1 ? ob : kept;
+    for (int t = 0; t < CH; ++t) {
+      if (t == 0) in[3] = in[0];                       // no token before the chunk's first: what it reads is not kept
+      if (t + 2 < CH) read_token(cur + (t + 2) * ROW, in[(t + 2) & 3]);
+      const float o = move(in[t & 3], in[(t + 3) & 3]);
+      if (t > 0) kept = r == t - 1 ? o : kept;
     }
+    const float o = row_sum(dot(in[(CH - 1) & 3].q));
+    kept = r == CH - 1 ? o : kept;
     if (more) put(t0 + CH, buf[1 - turn]);
     if (r < CH && t0 + r < end) {
       if (col < P) a.out[(size_t)(t0 + r) * a.heads * P + (size_t)h * P + col] = kept;
@@ -222,10 +276,11 @@ memory_scan_kernel(const MemoryArgs a) {
   if (a.write_state && live_col) {
 #pragma unroll
     for (int i = 0; i < NPT; ++i) {
-      const int n = row_of(i);
-      if (n < N) column[(size_t)n * row_step] = s[i];
+      const int at = row_of(i);
+      if (at < N) column[(size_t)at * row_step] = s[i];
     }
   }
+#undef KEEP_ORDER
 }
 
 // ------------------------------------------------------------------ steps of single tokens
@@ -314,17 +369,13 @@ memory_step_kernel(const MemoryArgs a) {
   }
 }
 
-template <int NPT, bool DELTA>
+template <int NP, bool DELTA>
 static int launch_scan(const MemoryArgs& a, int B_, hipStream_t stream) {
-  const int cols = a.P + (DELTA ? 0 : 1);
-  const bool vec = a.N % 4 == 0 && a.q_ld % 4 == 0 && a.k_ld % 4 == 0 && ((uintptr_t)a.q | (uintptr_t)a.k) % 16 == 0;
-  // four waves a block where there are blocks enough, else two: half as many columns, so that twice as many compute
-  // units have a block
-  const bool wide = (long long)B_ * a.heads * ((cols + 15) / 16) >= 256;
-#define GO(W, V) hipLaunchKernelGGL((memory_scan_kernel<W, NPT, DELTA, V>), dim3(B_, a.heads, (cols + 4 * W - 1) / (4 * W)), dim3(64 * W), 0, stream, a)
-  if (wide) { if (vec) GO(4, true); else GO(4, false); }
-  else { if (vec) GO(2, true); else GO(2, false); }
-#undef GO
+  const dim3 grid(B_, a.heads, (a.P + (DELTA ? 0 : 1) + 15) / 16);
+  if (a.N % 4 == 0 && a.q_ld % 4 == 0 && ((uintptr_t)a.q | (uintptr_t)a.k) % 16 == 0)
+    hipLaunchKernelGGL((memory_scan_kernel<NP / 16, DELTA, true>), grid, dim3(256), 0, stream, a);
+  else
+    hipLaunchKernelGGL((memory_scan_kernel<NP / 16, DELTA, false>), grid, dim3(256), 0, stream, a);
   ULLM_LAUNCH_CHECK();
 }
 
@@ -338,12 +389,12 @@ template <bool DELTA>
 static int memory_any(const MemoryArgs& a, int B_, bool single, hipStream_t stream) {
   const int N = a.N;
   if (!single) {
-    if (N <= 16) return launch_scan<1, DELTA>(a, B_, stream);
-    if (N <= 32) return launch_scan<2, DELTA>(a, B_, stream);
-    if (N <= 64) return launch_scan<4, DELTA>(a, B_, stream);
-    if (N <= 128) return launch_scan<8, DELTA>(a, B_, stream);
-    if (N <= 256) return launch_scan<16, DELTA>(a, B_, stream);
-    return launch_scan<32, DELTA>(a, B_, stream);
+    if (N <= 16) return launch_scan<16, DELTA>(a, B_, stream);
+    if (N <= 32) return launch_scan<32, DELTA>(a, B_, stream);
+    if (N <= 64) return launch_scan<64, DELTA>(a, B_, stream);
+    if (N <= 128) return launch_scan<128, DELTA>(a, B_, stream);
+    if (N <= 256) return launch_scan<256, DELTA>(a, B_, stream);
+    return launch_scan<512, DELTA>(a, B_, stream);
   }
   // rows of 64 value channels a block (whole lines of state) where there are blocks enough without narrow slices
   if (a.P % 64 == 0 && N <= 128 && (long long)B_ * a.heads >= 1024) {
@@ -368,6 +419,7 @@ extern "C" int ullm_matrix_memory(const float* q, int q_ld, const float* k, int 
   if (B_ <= 0) return 0;
   if (heads < 1 || kv_heads < 1 || heads % kv_heads || N < 1 || P < 1 || N > MEMORY_MAX_KEYS || heads > 65535) return ULLM_ERR_SHAPE;
   if ((P + 8) / 8 > 65535) return ULLM_ERR_SHAPE;
+  if (!single && q_ld != k_ld) return ULLM_ERR_UNSUPPORTED;
   if (rule != 0 && (rule != 1 || norm_out == nullptr)) return ULLM_ERR_UNSUPPORTED;
   MemoryArgs a;
   a.q = q, a.k = k, a.v = v, a.keep = keep, a.take = take, a.state = state, a.state_stride = state_stride, a.state_off = state_off;

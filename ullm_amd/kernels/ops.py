@@ -822,7 +822,7 @@ def matrix_memory(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, keep: torch
     _f32_rows(v, "v", T, heads * value_dim)
     _f32_rows(keep, "keep", T, heads)
     _f32_rows(take, "take", T, heads)
-    _need(keep.stride(0) == take.stride(0), "keep and take must be columns of rows equally far apart")
+    _need(keep.stride(0) == take.stride(0) and q.stride(0) == k.stride(0), "keep and take, and q and k, must be columns of rows equally far apart")
     _need(1 <= key_dim <= MEMORY_MAX_KEYS, f"{key_dim} key channels a head: at most {MEMORY_MAX_KEYS}")
     _check_step_state(state, state_off, heads * key_dim * value_dim, "the memories")
     if rule == MEMORY_SUM:
