@@ -149,6 +149,14 @@ def close(got, want, dtype, gaps=None, name=""):
 
 def agree(models, name, toks, got, dtype, rows=None):
     want, gaps = oracle_and_gaps(models, name, toks)
+    if dtype == "float32" and rows is None and np.abs(got - want).max() > REL[dtype] * np.abs(want).max():
+        # a row that is ill-conditioned in itself (one value over its own magnitude, next to zero): four times what the plain
+        # implementation loses there in 32-bit
+        _, cfg, w = models[name]
+        narrow = plain.forward({k: v.float() for k, v in w.items()}, cfg, list(toks)).numpy()
+        over = np.abs(got - want).max(-1) > np.maximum(REL[dtype] * np.abs(want).max(), 4 * np.abs(narrow - want).max(-1))
+        assert not over.any(), np.nonzero(over)
+        return
     if rows is not None:
         want, gaps = want[rows], gaps[rows]
     close(got, want, dtype, gaps, name)
@@ -446,10 +454,14 @@ def test_random_weights_for_the_named_size():
 
 def step_context(lens, starts=None, slots=None):
     """What the kernels read of a step with entries of these lengths (slots in another order than the entries)."""
+    from ullm_amd.parts.base import StepShape
+    from ullm_amd.parts.memory import plan_memory_chunks
     q = np.concatenate(([0], np.cumsum(lens))).astype(np.int32)
     starts = starts or [0] * len(lens)
     to = lambda a: torch.from_numpy(np.ascontiguousarray(np.asarray(a, dtype=np.int32))).to(DEV)      # noqa: E731
-    return SimpleNamespace(q_start=to(q), token_entry=to(np.repeat(np.arange(len(lens)), lens)), num_entries=len(lens),
+    chunks = plan_memory_chunks(StepShape(tuple(lens), tuple(starts)))
+    chunks.arrays = {k: to(v) for k, v in chunks.arrays.items()}
+    return SimpleNamespace(chunks=chunks, q_start=to(q), token_entry=to(np.repeat(np.arange(len(lens)), lens)), num_entries=len(lens),
                            entry_slot=to(slots if slots is not None else np.arange(len(lens))[::-1] + 1),
                            positions=to(np.concatenate([s + np.arange(n) for s, n in zip(starts, lens)])),
                            decode_only=all(n == 1 for n in lens), max_q_len=max(lens))
@@ -502,7 +514,7 @@ def test_the_matrix_memory_alone(heads, kv, N, P, rule):
         wide = torch.cat((v, q, k), dim=1)
         gates = torch.stack((keep, take), dim=1)
         o, n = ops.matrix_memory(wide[:, v.shape[1]:v.shape[1] + kv * N], wide[:, v.shape[1] + kv * N:], wide[:, :v.shape[1]], gates[:, 0], gates[:, 1],
-                                 ops.MEMORY_DELTA if rule == "delta" else ops.MEMORY_SUM, state, off, ctx, heads, kv, N, P, q_scale=0.7,
+                                 ops.MEMORY_DELTA if rule == "delta" else ops.MEMORY_SUM, state, off, ctx, heads, kv, N, P, ctx.chunks, q_scale=0.7,
                                  norm_off=off + heads * N * P)
         return (o,) if n is None else (o, n)
     got = over_steps(seqs, STEPS, call)
@@ -539,7 +551,7 @@ def test_the_matrix_memory_of_many_entries(heads=8, N=40, P=128):
             T = sum(lens)
             q, k, v = torch.randn(T, heads * N, generator=g), torch.nn.functional.normalize(torch.randn(T, heads, N, generator=g), dim=-1).view(T, -1), torch.randn(T, heads * P, generator=g)
             keep, take = torch.rand(T, heads, generator=g), torch.rand(T, heads, generator=g)
-            o, norm = ops.matrix_memory(q.to(DEV), k.to(DEV), v.to(DEV), keep.to(DEV), take.to(DEV), rule, state, 0, ctx, heads, heads, N, P, norm_off=heads * N * P)
+            o, norm = ops.matrix_memory(q.to(DEV), k.to(DEV), v.to(DEV), keep.to(DEV), take.to(DEV), rule, state, 0, ctx, heads, heads, N, P, ctx.chunks, norm_off=heads * N * P)
             want, want_n = torch.zeros(T, heads, P).double(), torch.zeros(T, heads).double()
             t = 0
             for b, L in enumerate(lens):

@@ -220,3 +220,19 @@ def test_every_mechanism_of_the_plain_model_moves_its_logits():
         x = dict(w)
         x[name] = x[name] * 0.5 + 0.1
         assert moved(weights=x) > 2e-4, name
+
+
+def test_the_chunks_of_a_step_cover_every_token_once():
+    from ullm_amd.parts.base import StepShape
+    from ullm_amd.parts.memory import plan_memory_chunks
+    lens = (1, 16, 17, 40, 2)
+    p = plan_memory_chunks(StepShape(lens, (0,) * 5))
+    items = p.arrays["items"].reshape(-1, 2).tolist()
+    assert p.facts == {"num_items": 8} and p.arrays["entry_item"].tolist() == [0, 1, 2, 4, 7]
+    at = 0
+    for first, n in items:
+        assert first == at and 1 <= n <= 16
+        at += n
+    assert at == sum(lens) and [n for _, n in items] == [1, 16, 16, 1, 16, 16, 8, 2]
+    single = plan_memory_chunks(StepShape((1, 1), (5, 9)))
+    assert single.facts == {"num_items": 0} and all(a.size == 0 for a in single.arrays.values())

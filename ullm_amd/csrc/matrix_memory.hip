@@ -9,13 +9,12 @@
 //
 // A batch is any mix of prompt portions and single tokens: entry b owns tokens q_start[b] .. q_start[b+1]-1 and the
 // state row entry_slot[b]; rows of requests that start at their first token are zero when a step begins.  Everything
-// is 32-bit.  A portion goes through the same operations in the same order wherever a prompt is cut; steps of single
-// tokens add up in another order.
+// is 32-bit, the matrix cores' products included.  A portion's chunks are counted from its first token, and steps of single
+// tokens add up in another order: whole and cut prompts agree to rounding.
 #include "common.h"
 #include "short_conv.h"
 
 typedef __attribute__((ext_vector_type(4))) float mem_f32x4;
-typedef __attribute__((ext_vector_type(2))) float mem_f32x2;
 
 #define MEMORY_MAX_KEYS 512
 
@@ -28,28 +27,15 @@ __device__ __forceinline__ void memory_barrier_shared() {
 #endif
 }
 
-// The sum over a row of 16 lanes in every one of them, by four rotations inside the vector unit.
-template <int CTRL>
-__device__ __forceinline__ float row_rotated(float v) {
+// D[i][j] = C[i][j] + sum_k A[i][k] B[k][j] for 16 x 4 by 4 x 16 in 32-bit: lane (c, g) = (lane % 16, lane / 16) holds A[c][k]
+// and B[k][c] for its own k and D[4 g + r][c] in register r.  Which k a lane group stands for is free as long as A and B
+// agree: a 16 x 16 result's register r is, as it lies, the B operand of the step whose groups stand for k = 4 g + r.
+__device__ __forceinline__ mem_f32x4 mma(float a, float b, mem_f32x4 c) {
 #ifdef __HIP_DEVICE_COMPILE__
-  return __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), CTRL, 0xf, 0xf, true));
+  return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0);
 #else
-  return v;
+  return c;
 #endif
-}
-template <int STEP>
-__device__ __forceinline__ void row_sum_step(float& v) {
-  if constexpr (STEP == 0) v += row_rotated<0x128>(v);
-  if constexpr (STEP == 1) v += row_rotated<0x124>(v);
-  if constexpr (STEP == 2) v += row_rotated<0x122>(v);
-  if constexpr (STEP == 3) v += row_rotated<0x121>(v);
-}
-__device__ __forceinline__ float row_sum(float v) {
-  row_sum_step<0>(v);
-  row_sum_step<1>(v);
-  row_sum_step<2>(v);
-  row_sum_step<3>(v);
-  return v;
 }
 
 struct MemoryArgs {
@@ -62,43 +48,135 @@ struct MemoryArgs {
   long long state_stride, state_off, norm_off;      // norm_off: the heads' normalisers [heads, N] (RULE_SUM)
   const int* q_start;
   const int* entry_slot;
+  const int* items;         // the chunks of a step with portions: (first token, tokens) each, an entry's side by side
+  const int* entry_item;    // [B]: an entry's first item
+  float* chunks;            // [items, heads, CHUNK_FLOATS]
   float* out;               // [T, heads * P]
   float* norm_out;          // [T, heads]: n . q (RULE_SUM)
-  int q_ld, k_ld, v_ld, gate_ld;      // q_ld == k_ld in steps with portions
+  int q_ld, k_ld, v_ld, gate_ld;
   int heads, kv_heads, N, P, write_state;
   float q_scale;
 };
 
-// ------------------------------------------------------------------ portions of prompts
+// ------------------------------------------------------------------ portions of prompts, in chunks of 16 tokens
+// Inside a chunk, with S0 the memory it finds, G_ij = g_(j+1) .. g_i, c_i = g_1 .. g_i and d_j = g_(j+1) .. g_16:
+//   u_i + b_i sum_(j<i) G_ij (k_i . k_j) u_j = b_i (v_i - c_i S0^T k_i)      (RULE_DELTA; u_i = b_i v_i with RULE_SUM)
+//   o_i = c_i S0^T q_i + sum_(j<=i) G_ij (q_i . k_j) u_j,     S1 = c_16 S0 + sum_j d_j k_j u_j^T
+// What does not depend on S0 is made for all chunks at once: the products of keys and queries, and the inverse of the
+// unit lower triangle by substitution (memory_chunk_kernel).  What is left per chunk are products of 16-row tiles.
+// Products of decays are formed as products: no logarithm, no quotient.  Tokens past an entry's end repeat its last
+// token's vectors with g = 1 and b = 0, which changes nothing.
+#define CHUNK_TOKENS 16
+#define CHUNK_T 0          // [16][16]: inverse times b_j (RULE_DELTA)
+#define CHUNK_M 256        // [16][16]: G_ij (q_i . k_j) for j <= i
+#define CHUNK_C 512        // c_i
+#define CHUNK_D 528        // d_j
+#define CHUNK_B 544        // b_j
+#define CHUNK_FLOATS 576
+
+// Four neighbouring values of a row of N; past the end valid elements again (what meets them is zero).
+template <bool VEC>
+__device__ __forceinline__ mem_f32x4 row_piece(const float* row, int n, int N) {
+  mem_f32x4 x;
+  if constexpr (VEC) {
+    x = *reinterpret_cast<const mem_f32x4*>(row + (n < N ? n : 0));
+  } else {
+#pragma unroll
+    for (int j = 0; j < 4; ++j) x[j] = row[n + j < N ? n + j : N - 1];
+  }
+  return x;
+}
+
+// One wave per (chunk, head).
+template <bool DELTA, bool VEC>
+__global__ void __launch_bounds__(64)
+memory_chunk_kernel(const MemoryArgs a) {
+  __shared__ float s_g[16], s_b[16], s_l[16 * 20];
+  const int item = blockIdx.x, h = blockIdx.y, lane = threadIdx.x, c = lane & 15, g = lane >> 4;
+  const int t0 = a.items[2 * item], n_tok = a.items[2 * item + 1], N = a.N;
+  const int kvh = h / (a.heads / a.kv_heads);
+  const int tok = t0 + (c < n_tok ? c : n_tok - 1);
+  const float gm = c < n_tok ? a.keep[(size_t)tok * a.gate_ld + h] : 1.f;
+  const float bm = c < n_tok ? a.take[(size_t)tok * a.gate_ld + h] : 0.f;
+  const float* qr = a.q + (size_t)tok * a.q_ld + (size_t)kvh * N;
+  const float* kr = a.k + (size_t)tok * a.k_ld + (size_t)kvh * N;
+  mem_f32x4 kk = {0.f, 0.f, 0.f, 0.f}, qk = kk;
+#pragma unroll 4
+  for (int n0 = 0; n0 < N; n0 += 16) {
+    const int n = n0 + 4 * g;
+    mem_f32x4 kv = row_piece<VEC>(kr, n, N);
+    const mem_f32x4 qv = row_piece<VEC>(qr, n, N);
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      kv[r] = n + r < N ? kv[r] : 0.f;
+      qk = mma(qv[r], kv[r], qk);
+      if constexpr (DELTA) kk = mma(kv[r], kv[r], kk);
+    }
+  }
+  float before = gm, after = __shfl_down(gm, 1, 16);
+  if (c == 15) after = 1.f;
+#pragma unroll
+  for (int d = 1; d < 16; d *= 2) {
+    const float lo = __shfl_up(before, d, 16), hi = __shfl_down(after, d, 16);
+    if (c >= d) before *= lo;
+    if (c + d < 16) after *= hi;
+  }
+  if (g == 0) s_g[c] = gm, s_b[c] = bm;
+  __syncthreads();
+  // register r: row i = 4 g + r, column j = c
+  float decay[4];
+  float p = 1.f;
+#pragma unroll
+  for (int m = 1; m <= 12; ++m)
+    if (m <= 4 * g && m > c) p *= s_g[m];
+  decay[0] = p;
+#pragma unroll
+  for (int r = 1; r < 4; ++r) {
+    if (4 * g + r > c) p *= s_g[4 * g + r];
+    decay[r] = p;
+  }
+  float* to = a.chunks + ((size_t)item * a.heads + h) * CHUNK_FLOATS;
+#pragma unroll
+  for (int r = 0; r < 4; ++r) {
+    const int i = 4 * g + r;
+    to[CHUNK_M + i * 16 + c] = c <= i ? decay[r] * (qk[r] * a.q_scale) : 0.f;
+    if constexpr (DELTA) s_l[i * 20 + c] = c < i ? s_b[i] * decay[r] * kk[r] : 0.f;
+  }
+  if (g == 0) to[CHUNK_C + c] = before, to[CHUNK_D + c] = after, to[CHUNK_B + c] = bm;
+  if constexpr (DELTA) {
+    __syncthreads();
+    // the inverse column by column (the four lane groups do the same): x_i = (i == c) - sum_(m < i) L_im x_m
+    float x[16];
+#pragma unroll
+    for (int i = 0; i < 16; ++i) {
+      float v = i == c ? 1.f : 0.f;
+#pragma unroll
+      for (int m = 0; m < i; ++m) v -= s_l[i * 20 + m] * x[m];
+      x[i] = v;
+    }
+#pragma unroll
+    for (int i = 0; i < 16; ++i)
+      if (i / 4 == g) to[CHUNK_T + i * 16 + c] = x[i] * bm;
+  }
+}
+
 // One block of four waves per (entry, head, slice of 16 value columns); with RULE_SUM the column behind the last is the
-// normaliser.  Lane (r, c) = (lane % 16, lane / 16) of a wave keeps NPT rows of column c in registers; the sixteen lanes
-// of a column hold its 16 NPT >= N rows and add up inside the wave, so no sum crosses waves and no token waits for a
-// barrier.  An entry's tokens are walked in chunks of CH: the chunk's q, k, v, g and b lie in shared memory, the next
-// chunk's are fetched into registers before the current one is worked on and put into the other buffer afterwards; a
-// token's values are read two tokens ahead.  A token's read-out is formed while the next token's S^T k is on its way
-// through the lanes (both read the same S), in an order the source fixes.  Lane r keeps token r's result until the chunk's end.  Tokens past the entry's end
-// repeat its last token's values with b = 0 and g = 1, which changes nothing.
-template <int NPT, bool DELTA, bool VEC>
+// normaliser.  Wave w keeps the RT row tiles w RT .. of S's slice in registers (64 RT >= N rows in all).  Per chunk it forms its
+// rows' part of S0^T k and S0^T q; the parts of S0^T k meet in shared memory, then every wave forms u (the same in all four), adds
+// a quarter of the tokens' part to its outputs, and moves its rows on.  The outputs' parts meet in the next chunk's
+// exchange: one barrier a chunk.  A chunk's operands are asked for AHEAD chunks ahead, straight into registers; the keys pass
+// through the wave's own shared memory once, to be read the other way round.
+template <int RT, int AHEAD, bool DELTA, bool VEC>
 __global__ void __launch_bounds__(256)
 memory_scan_kernel(const MemoryArgs a) {
-  constexpr int W = 4, LANES = 16;
-  constexpr int NP = LANES * NPT;                    // padded key channels
-  constexpr int CH = NP > 256 ? 4 : NP > 128 ? 8 : 16;
-  constexpr int WC = 64 / LANES;                     // columns of a wave
-  constexpr int COLS = WC * W, THREADS = 64 * W;
-  constexpr int ROW = 2 * NP + COLS + 4;             // a token's q | k | v | g b
-  constexpr int TOK_PIECES = NP / 2;                 // pieces of four channels of a token's q | k
-  constexpr int PER = CH * TOK_PIECES > THREADS ? CH * TOK_PIECES / THREADS : 1;
-  constexpr int STEP = THREADS / TOK_PIECES;         // tokens between a thread's pieces
-  constexpr int V_PER = (CH * COLS + THREADS - 1) / THREADS;
-  static_assert(THREADS % TOK_PIECES == 0, "a thread's pieces lie in one place of different tokens");
-  static_assert(ROW % 4 == 0 && COLS % 4 == 0, "16-byte pieces");
-  __shared__ __attribute__((aligned(16))) float buf[2][CH * ROW];
-  const int b = blockIdx.x, h = blockIdx.y, c0 = blockIdx.z * COLS;
-  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, r = lane % LANES, cw = lane / LANES;
-  const int N = a.N, P = a.P;
+  constexpr int KT_ROW = 16 * RT + 4;
+  __shared__ mem_f32x4 s_w[2][4][64], s_o[2][4][64];
+  __shared__ __attribute__((aligned(16))) float s_kt[4][16 * KT_ROW];
+  const int b = blockIdx.x, h = blockIdx.y;
+  const int lane = threadIdx.x & 63, c = lane & 15, g = lane >> 4;
+  const int w = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+  const int N = a.N, P = a.P, col = blockIdx.z * 16 + c;
   const int kvh = h / (a.heads / a.kv_heads);
-  const int col = c0 + WC * wave + cw;
   const bool live_col = col < P || (!DELTA && col == P);
   const int first = a.q_start[b], end = a.q_start[b + 1];
   if (first >= end) return;
@@ -106,181 +184,176 @@ memory_scan_kernel(const MemoryArgs a) {
   // where this lane's column lies: rows of S are P apart, the normaliser's values side by side
   float* column = col < P ? row + a.state_off + (size_t)h * N * P + col : row + a.norm_off + (size_t)h * N;
   const int row_step = col < P ? P : 1;
-  auto row_of = [&](int i) __attribute__((always_inline)) {
-    return NPT % 4 == 0 ? (i / 4) * (4 * LANES) + 4 * r + i % 4 : r * NPT + i;
-  };
-  float s[NPT];
+  const int n_first = 16 * w * RT;                   // this wave's first row
+  mem_f32x4 S[RT];
 #pragma unroll
-  for (int i = 0; i < NPT; ++i) {
-    const int n = row_of(i);
-    s[i] = (live_col && n < N) ? column[(size_t)n * row_step] : 0.f;
-  }
-  // staging: this thread brings channels n .. n + 3 of q or of k for the tokens tl, tl + STEP, ..
-  const int tl = tid / TOK_PIECES, which = (tid / (NP / 4)) & 1, n = 4 * (tid % (NP / 4));
-  const float* src = (which ? a.k : a.q) + (size_t)kvh * N;
-  mem_f32x4 factor;                                  // q's scale, zero for channels past N
+  for (int t = 0; t < RT; ++t)
 #pragma unroll
-  for (int j = 0; j < 4; ++j) factor[j] = n + j < N ? (which ? 1.f : a.q_scale) : 0.f;
-  if constexpr (VEC) src += n < N ? n : 0;
-  const int v_col = c0 + tid % COLS;
-  const float* src_v = a.v + (size_t)h * P + (v_col < P ? v_col : P - 1);
-  const float* src_g = (tid & 1 ? a.take : a.keep) + h;
-  mem_f32x4 raw[PER];
-  float raw_v[V_PER], raw_g = 1.f;
-  auto piece = [&](const float* p) __attribute__((always_inline)) {
-    mem_f32x4 x;
-    if constexpr (VEC) {
-      x = *reinterpret_cast<const mem_f32x4*>(p);
-    } else {
-#pragma unroll
-      for (int j = 0; j < 4; ++j) x[j] = p[n + j < N ? n + j : N - 1];
+    for (int r = 0; r < 4; ++r) {
+      const int n = n_first + 16 * t + 4 * g + r;
+      S[t][r] = (live_col && n < N) ? column[(size_t)n * row_step] : 0.f;
     }
-    return x;
+  struct In {
+    mem_f32x4 k[RT], q[RT];                          // token c's channels
+    mem_f32x4 v, tri, cum, tail, take;               // tokens 4 g + r (tri: row c)
+    float m, all;
   };
-  // every load is issued whatever it is for, so that all of them are on their way at once; whole chunks step through
-  // memory evenly, the last one may not read past the entry's end
-  auto fetch = [&](int t0) __attribute__((always_inline)) {
-    if (t0 + CH <= end) {
-      const float* p = src + (size_t)(t0 + tl % CH) * a.q_ld;
+  // offsets inside a chunk, in values; the last chunk of an entry may not reach past its end and repeats the last token
+  int last = CHUNK_TOKENS - 1;
+  unsigned off_k, off_q, off_v[4];
+  auto offsets = [&]() __attribute__((always_inline)) {
+    const int tc = c < last ? c : last;
+    off_k = (unsigned)(tc * a.k_ld), off_q = (unsigned)(tc * a.q_ld);
 #pragma unroll
-      for (int i = 0; i < PER; ++i) raw[i] = piece(p + (size_t)(i * STEP) * a.q_ld);
-      const float* pv = src_v + (size_t)(t0 + (tid / COLS) % CH) * a.v_ld;
+    for (int r = 0; r < 4; ++r) {
+      const int tr = 4 * g + r < last ? 4 * g + r : last;
+      off_v[r] = (unsigned)(tr * a.v_ld) + (unsigned)(col < P ? col : P - 1);
+    }
+  };
+  offsets();
+  const float* kh = a.k + (size_t)kvh * N;
+  const float* qh = a.q + (size_t)kvh * N;
+  const float* vh = a.v + (size_t)h * P;
+  const float* pre = a.chunks + ((size_t)a.entry_item[b] * a.heads + h) * CHUNK_FLOATS;
+  const int last_chunk = first + (end - first - 1) / CHUNK_TOKENS * CHUNK_TOKENS;
+  // always as many loads, whatever is left of the entry (behind its last chunk that one again): the waits for those asked
+  // for earlier can then be counted
+  auto fetch = [&](int t0, In& in) __attribute__((always_inline)) {
+    t0 = t0 < last_chunk ? t0 : last_chunk;
+    if (t0 + CHUNK_TOKENS > end) {
+      last = end - 1 - t0;
+      offsets();
+    }
+    const float* kr = kh + (size_t)t0 * a.k_ld;
+    const float* qr = qh + (size_t)t0 * a.q_ld;
+    const float* vr = vh + (size_t)t0 * a.v_ld;
 #pragma unroll
-      for (int i = 0; i < V_PER; ++i) raw_v[i] = pv[(size_t)(i * (THREADS / COLS)) * a.v_ld];
-    } else {
-#pragma unroll
-      for (int i = 0; i < PER; ++i) {
-        const int tok = t0 + tl + i * STEP < end ? t0 + tl + i * STEP : end - 1;
-        raw[i] = piece(src + (size_t)tok * a.q_ld);
+    for (int t = 0; t < RT; ++t) {
+      const int n = n_first + 16 * t + 4 * g;
+      if constexpr (VEC) {
+        const unsigned at = (unsigned)(n < N ? n : 0);
+        in.k[t] = *reinterpret_cast<const mem_f32x4*>(kr + (off_k + at));
+        in.q[t] = *reinterpret_cast<const mem_f32x4*>(qr + (off_q + at));
+      } else {
+        in.k[t] = row_piece<false>(kr + off_k, n, N);
+        in.q[t] = row_piece<false>(qr + off_q, n, N);
       }
-#pragma unroll
-      for (int i = 0; i < V_PER; ++i) {
-        const int tok = t0 + tid / COLS + i * (THREADS / COLS) < end ? t0 + tid / COLS + i * (THREADS / COLS) : end - 1;
-        raw_v[i] = src_v[(size_t)tok * a.v_ld];
-      }
     }
-    if (tid < 2 * CH) {
-      const int tok = t0 + (tid >> 1) < end ? t0 + (tid >> 1) : end - 1;
-      raw_g = src_g[(size_t)tok * a.gate_ld];
-    }
+#pragma unroll
+    for (int r = 0; r < 4; ++r) in.v[r] = vr[off_v[r]];
+    const float* at = pre + (size_t)((t0 - first) / CHUNK_TOKENS) * a.heads * CHUNK_FLOATS;
+    if constexpr (DELTA) in.tri = *reinterpret_cast<const mem_f32x4*>(at + (CHUNK_T + 16 * c + 4 * g));
+    else in.take = *reinterpret_cast<const mem_f32x4*>(at + (CHUNK_B + 4 * g));
+    in.m = at[CHUNK_M + 16 * c + 4 * g + w];
+    in.cum = *reinterpret_cast<const mem_f32x4*>(at + (CHUNK_C + 4 * g));
+    in.tail = *reinterpret_cast<const mem_f32x4*>(at + (CHUNK_D + 4 * g));
+    in.all = at[CHUNK_C + 15];
   };
-  auto put = [&](int t0, float* dst) __attribute__((always_inline)) {
-    float* to = dst + tl * ROW + which * NP + n;
+  // the outputs of the chunk that began at t0: this wave adds up the parts of tokens 4 g + w
+  const int o_step = col < P ? a.heads * P : a.heads;
+  float* o_at = (col < P ? a.out + (size_t)h * P + col : a.norm_out + h) + (size_t)(first + 4 * g + w) * o_step;
+  auto finish = [&](int t0, int turn) __attribute__((always_inline)) {
+    float o = 0.f;
 #pragma unroll
-    for (int i = 0; i < PER; ++i)
-      if (CH * TOK_PIECES >= THREADS || tl < CH) *reinterpret_cast<mem_f32x4*>(to + i * STEP * ROW) = raw[i] * factor;
-#pragma unroll
-    for (int i = 0; i < V_PER; ++i) {
-      const int at = tid / COLS + i * (THREADS / COLS);
-      if (CH * COLS >= THREADS || at < CH) dst[at * ROW + 2 * NP + tid % COLS] = (!DELTA && v_col == P) ? 1.f : raw_v[i];
-    }
-    if (tid < 2 * CH) dst[(tid >> 1) * ROW + 2 * NP + COLS + (tid & 1)] = t0 + (tid >> 1) < end ? raw_g : (tid & 1 ? 0.f : 1.f);
+    for (int i = 0; i < 4; ++i) o += reinterpret_cast<const float*>(&s_o[turn][i][lane])[w];
+    if (live_col && t0 + 4 * g + w < end) *o_at = o;
+    o_at += (size_t)CHUNK_TOKENS * o_step;
   };
-  struct TokenIn {
-    float q[NPT], k[NPT];
-    float v, g, b;
-  };
-  auto read_token = [&](const float* from, TokenIn& in) __attribute__((always_inline)) {
-    if constexpr (NPT % 4 == 0) {
-#pragma unroll
-      for (int i = 0; i < NPT; i += 4) {
-        const mem_f32x4 kk = *reinterpret_cast<const mem_f32x4*>(from + NP + LANES * i + 4 * r);
-        const mem_f32x4 qq = *reinterpret_cast<const mem_f32x4*>(from + LANES * i + 4 * r);
-#pragma unroll
-        for (int j = 0; j < 4; ++j) in.k[i + j] = kk[j], in.q[i + j] = qq[j];
-      }
-    } else {
-#pragma unroll
-      for (int i = 0; i < NPT; ++i) in.k[i] = from[NP + r * NPT + i], in.q[i] = from[r * NPT + i];
-    }
-    in.v = from[2 * NP + WC * wave + cw];
-    const mem_f32x2 gb = *reinterpret_cast<const mem_f32x2*>(from + 2 * NP + COLS);
-    in.g = gb.x, in.b = gb.y;
-  };
-  auto dot = [&](const float* x) __attribute__((always_inline)) {
-    float lo = s[0] * x[0], hi = NPT > 1 ? s[NPT > 1 ? 1 : 0] * x[NPT > 1 ? 1 : 0] : 0.f;
-#pragma unroll
-    for (int i = 2; i < NPT; i += 2) lo += s[i] * x[i], hi += s[i + 1] * x[i + 1];
-    return lo + hi;
-  };
+  float* kt_in = s_kt[w] + c * KT_ROW + 4 * g;
+  const float* kt_out = s_kt[w] + 4 * g * KT_ROW + c;
 #define KEEP_ORDER __builtin_amdgcn_sched_barrier(0)
-  // one token, and the read-out of the token before (the S it left is the one this token finds)
-  auto move = [&](const TokenIn& in, const TokenIn& before) __attribute__((always_inline)) {
-    float o;
+  const bool whole = N == 64 * RT;
+  const bool odd = threadIdx.x & 64, upper = threadIdx.x & 128;
+  auto chunk = [&](int t0, int turn, In& in, In& later) __attribute__((always_inline)) {
+    fetch(t0 + AHEAD * CHUNK_TOKENS, later);
+    const mem_f32x4 zero = {0.f, 0.f, 0.f, 0.f};
+    mem_f32x4 sk = zero, sq = zero, kt[RT];
+    if (!whole) {                                    // rows past N stay zero
+#pragma unroll
+      for (int t = 0; t < RT; ++t)
+#pragma unroll
+        for (int j = 0; j < 4; ++j) in.k[t][j] = n_first + 16 * t + 4 * g + j < N ? in.k[t][j] : 0.f;
+    }
+#pragma unroll
+    for (int t = 0; t < RT; ++t) *reinterpret_cast<mem_f32x4*>(kt_in + 16 * t) = in.k[t];
+    // S0^T k first: the other waves wait for it, and S0^T q is worked on while it is on its way
     if constexpr (DELTA) {
-      float p = dot(in.k);
-      KEEP_ORDER;
-      row_sum_step<0>(p);
-      o = dot(before.q);
-      KEEP_ORDER;
-      row_sum_step<1>(p);
 #pragma unroll
-      for (int i = 0; i < NPT / 2; ++i) s[i] *= in.g;
-      KEEP_ORDER;
-      row_sum_step<2>(p);
+      for (int t = 0; t < RT; ++t)
 #pragma unroll
-      for (int i = NPT / 2; i < NPT; ++i) s[i] *= in.g;
+        for (int r = 0; r < 4; ++r) sk = mma(in.k[t][r], S[t][r], sk);
       KEEP_ORDER;
-      row_sum_step<3>(p);
-      row_sum_step<0>(o);
-      KEEP_ORDER;
-      row_sum_step<1>(o);
-      KEEP_ORDER;
-      const float u = in.b * (in.v - in.g * p);
-#pragma unroll
-      for (int i = 0; i < NPT / 2; ++i) s[i] = fmaf(in.k[i], u, s[i]);
-      row_sum_step<2>(o);
-      KEEP_ORDER;
-#pragma unroll
-      for (int i = NPT / 2; i < NPT; ++i) s[i] = fmaf(in.k[i], u, s[i]);
-      row_sum_step<3>(o);
-      KEEP_ORDER;
-    } else {
-      o = dot(before.q);
-      const float u = in.b * in.v;
-#pragma unroll
-      for (int i = 0; i < NPT; ++i) s[i] = fmaf(in.k[i], u, in.g * s[i]);
-      o = row_sum(o);
     }
-    return o;
-  };
-  fetch(first);
-  put(first, buf[0]);
-  memory_barrier_shared();
-  int turn = 0;
-  for (int t0 = first; t0 < end; t0 += CH) {
-    const float* cur = buf[turn];
-    const bool more = t0 + CH < end;
-    if (more) fetch(t0 + CH);
-    TokenIn in[4];
-    float kept = 0.f;
-    read_token(cur, in[0]);
-    read_token(cur + ROW, in[1]);
 #pragma unroll
-    for (int t = 0; t < CH; ++t) {
-      if (t == 0) in[3] = in[0];                       // no token before the chunk's first: what it reads is not kept
-      if (t + 2 < CH) read_token(cur + (t + 2) * ROW, in[(t + 2) & 3]);
-      const float o = move(in[t & 3], in[(t + 3) & 3]);
-      if (t > 0) kept = r == t - 1 ? o : kept;
-    }
-    const float o = row_sum(dot(in[(CH - 1) & 3].q));
-    kept = r == CH - 1 ? o : kept;
-    if (more) put(t0 + CH, buf[1 - turn]);
-    if (r < CH && t0 + r < end) {
-      if (col < P) a.out[(size_t)(t0 + r) * a.heads * P + (size_t)h * P + col] = kept;
-      else if (!DELTA && col == P) a.norm_out[(size_t)(t0 + r) * a.heads + h] = kept;
-    }
+    for (int t = 0; t < RT; ++t)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        sq = mma(in.q[t][r], S[t][r], sq);
+        if (t == 0 && r == 1) {
+          KEEP_ORDER;
+          if constexpr (DELTA) s_w[turn][w][lane] = sk;
+#pragma unroll
+          for (int i = 0; i < RT; ++i)
+#pragma unroll
+            for (int j = 0; j < 4; ++j) kt[i][j] = kt_out[j * KT_ROW + 16 * i];
+          KEEP_ORDER;
+        }
+      }
     memory_barrier_shared();
-    turn = 1 - turn;
-  }
-  if (a.write_state && live_col) {
+    if constexpr (DELTA) {
+      sk = s_w[turn][0][lane];
 #pragma unroll
-    for (int i = 0; i < NPT; ++i) {
-      const int at = row_of(i);
-      if (at < N) column[(size_t)at * row_step] = s[i];
+      for (int i = 1; i < 4; ++i) sk += s_w[turn][i][lane];
+    }
+    mem_f32x4 u;
+    if constexpr (DELTA) {
+      u = zero;
+#pragma unroll
+      for (int r = 0; r < 4; ++r) u = mma(in.tri[r], in.v[r] - in.cum[r] * sk[r], u);
+    } else {
+      u = in.take * ((!DELTA && col == P) ? zero + 1.f : in.v);
+    }
+    const mem_f32x4 part = in.cum * (sq * a.q_scale);
+#pragma unroll
+    for (int t = 0; t < RT; ++t) S[t] *= in.all;
+    const mem_f32x4 ut = u * in.tail;
+    const float lo = odd ? u[1] : u[0], hi = odd ? u[3] : u[2];
+    s_o[turn][w][lane] = mma(in.m, upper ? hi : lo, part);
+#pragma unroll
+    for (int r = 0; r < 4; ++r)
+#pragma unroll
+      for (int t = 0; t < RT; ++t) S[t] = mma(kt[t][r], ut[r], S[t]);
+    if (t0 > first) finish(t0 - CHUNK_TOKENS, 1 - turn);
+  };
+  In in[AHEAD + 1];
+#pragma unroll
+  for (int i = 0; i < AHEAD; ++i) fetch(first + i * CHUNK_TOKENS, in[i]);
+  // the sets of registers take turns, and so do the halves of the exchange: both come round after ROUND chunks
+  constexpr int ROUND = AHEAD == 1 ? 2 : 2 * (AHEAD + 1);
+  int t0 = first;
+  for (bool more = true; more;) {
+#pragma unroll
+    for (int i = 0; i < ROUND; ++i) {
+      chunk(t0, i & 1, in[i % (AHEAD + 1)], in[(i + AHEAD) % (AHEAD + 1)]);
+      t0 += CHUNK_TOKENS;
+      if (t0 >= end) {
+        more = false;
+        break;
+      }
     }
   }
 #undef KEEP_ORDER
+  memory_barrier_shared();
+  finish(last_chunk, (last_chunk - first) / CHUNK_TOKENS & 1);
+  if (a.write_state && live_col) {
+#pragma unroll
+    for (int t = 0; t < RT; ++t)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int n = n_first + 16 * t + 4 * g + r;
+        if (n < N) column[(size_t)n * row_step] = S[t][r];
+      }
+  }
 }
 
 // ------------------------------------------------------------------ steps of single tokens
@@ -369,13 +442,20 @@ memory_step_kernel(const MemoryArgs a) {
   }
 }
 
-template <int NP, bool DELTA>
-static int launch_scan(const MemoryArgs& a, int B_, hipStream_t stream) {
+template <int RT, bool DELTA>
+static int launch_scan(const MemoryArgs& a, int B_, int n_items, hipStream_t stream) {
   const dim3 grid(B_, a.heads, (a.P + (DELTA ? 0 : 1) + 15) / 16);
-  if (a.N % 4 == 0 && a.q_ld % 4 == 0 && ((uintptr_t)a.q | (uintptr_t)a.k) % 16 == 0)
-    hipLaunchKernelGGL((memory_scan_kernel<NP / 16, DELTA, true>), grid, dim3(256), 0, stream, a);
-  else
-    hipLaunchKernelGGL((memory_scan_kernel<NP / 16, DELTA, false>), grid, dim3(256), 0, stream, a);
+  if (a.N % 4 == 0 && a.q_ld % 4 == 0 && a.k_ld % 4 == 0 && ((uintptr_t)a.q | (uintptr_t)a.k) % 16 == 0) {
+    hipLaunchKernelGGL((memory_chunk_kernel<DELTA, true>), dim3(n_items, a.heads), dim3(64), 0, stream, a);
+    // few blocks: nothing else runs while a chunk's operands are on their way, so they are asked for two chunks ahead
+    if (RT <= 4 && (long long)grid.x * grid.y * grid.z < 512)
+      hipLaunchKernelGGL((memory_scan_kernel<RT, RT <= 4 ? 2 : 1, DELTA, true>), grid, dim3(256), 0, stream, a);
+    else
+      hipLaunchKernelGGL((memory_scan_kernel<RT, 1, DELTA, true>), grid, dim3(256), 0, stream, a);
+  } else {
+    hipLaunchKernelGGL((memory_chunk_kernel<DELTA, false>), dim3(n_items, a.heads), dim3(64), 0, stream, a);
+    hipLaunchKernelGGL((memory_scan_kernel<RT, 1, DELTA, false>), grid, dim3(256), 0, stream, a);
+  }
   ULLM_LAUNCH_CHECK();
 }
 
@@ -386,15 +466,13 @@ static int launch_step(const MemoryArgs& a, int B_, hipStream_t stream) {
 }
 
 template <bool DELTA>
-static int memory_any(const MemoryArgs& a, int B_, bool single, hipStream_t stream) {
+static int memory_any(const MemoryArgs& a, int B_, int n_items, bool single, hipStream_t stream) {
   const int N = a.N;
   if (!single) {
-    if (N <= 16) return launch_scan<16, DELTA>(a, B_, stream);
-    if (N <= 32) return launch_scan<32, DELTA>(a, B_, stream);
-    if (N <= 64) return launch_scan<64, DELTA>(a, B_, stream);
-    if (N <= 128) return launch_scan<128, DELTA>(a, B_, stream);
-    if (N <= 256) return launch_scan<256, DELTA>(a, B_, stream);
-    return launch_scan<512, DELTA>(a, B_, stream);
+    if (N <= 64) return launch_scan<1, DELTA>(a, B_, n_items, stream);
+    if (N <= 128) return launch_scan<2, DELTA>(a, B_, n_items, stream);
+    if (N <= 256) return launch_scan<4, DELTA>(a, B_, n_items, stream);
+    return launch_scan<8, DELTA>(a, B_, n_items, stream);
   }
   // rows of 64 value channels a block (whole lines of state) where there are blocks enough without narrow slices
   if (a.P % 64 == 0 && N <= 128 && (long long)B_ * a.heads >= 1024) {
@@ -410,23 +488,25 @@ static int memory_any(const MemoryArgs& a, int B_, bool single, hipStream_t stre
   return launch_step<16, 32, DELTA>(a, B_, stream);
 }
 
-// rule 0: RULE_DELTA, 1: RULE_SUM.  `single`: every entry brings exactly one token.
+// rule 0: RULE_DELTA, 1: RULE_SUM.  `single`: every entry brings exactly one token; else `items` (first token, tokens) lists
+// the step's chunks of up to 16 tokens, `entry_item` every entry's first, and `chunks` has room for what is made of them.
 extern "C" int ullm_matrix_memory(const float* q, int q_ld, const float* k, int k_ld, const float* v, int v_ld, const float* keep,
                                   const float* take, int gate_ld, int rule, float q_scale, float* state, long long state_stride,
-                                  long long state_off, long long norm_off, const int* q_start, const int* entry_slot, float* out,
-                                  float* norm_out, int B_, int heads, int kv_heads, int N, int P, int write_state, int single,
-                                  hipStream_t stream) {
+                                  long long state_off, long long norm_off, const int* q_start, const int* entry_slot, const int* items,
+                                  const int* entry_item, int n_items, float* chunks, float* out, float* norm_out, int B_, int heads,
+                                  int kv_heads, int N, int P, int write_state, int single, hipStream_t stream) {
   if (B_ <= 0) return 0;
   if (heads < 1 || kv_heads < 1 || heads % kv_heads || N < 1 || P < 1 || N > MEMORY_MAX_KEYS || heads > 65535) return ULLM_ERR_SHAPE;
-  if ((P + 8) / 8 > 65535) return ULLM_ERR_SHAPE;
-  if (!single && q_ld != k_ld) return ULLM_ERR_UNSUPPORTED;
+  if ((P + 16) / 16 > 65535) return ULLM_ERR_SHAPE;
+  if (!single && (q_ld > (1 << 26) || k_ld > (1 << 26) || v_ld > (1 << 26))) return ULLM_ERR_SHAPE;   // 32-bit offsets inside a chunk
+  if (!single && (n_items < B_ || !items || !entry_item || !chunks || (uintptr_t)chunks % 16)) return ULLM_ERR_SHAPE;
   if (rule != 0 && (rule != 1 || norm_out == nullptr)) return ULLM_ERR_UNSUPPORTED;
   MemoryArgs a;
   a.q = q, a.k = k, a.v = v, a.keep = keep, a.take = take, a.state = state, a.state_stride = state_stride, a.state_off = state_off;
-  a.norm_off = norm_off, a.q_start = q_start, a.entry_slot = entry_slot, a.out = out, a.norm_out = norm_out;
-  a.q_ld = q_ld, a.k_ld = k_ld, a.v_ld = v_ld, a.gate_ld = gate_ld, a.heads = heads, a.kv_heads = kv_heads, a.N = N, a.P = P;
-  a.write_state = write_state, a.q_scale = q_scale;
-  return rule == 0 ? memory_any<true>(a, B_, single != 0, stream) : memory_any<false>(a, B_, single != 0, stream);
+  a.norm_off = norm_off, a.q_start = q_start, a.entry_slot = entry_slot, a.items = items, a.entry_item = entry_item, a.chunks = chunks;
+  a.out = out, a.norm_out = norm_out, a.q_ld = q_ld, a.k_ld = k_ld, a.v_ld = v_ld, a.gate_ld = gate_ld, a.heads = heads;
+  a.kv_heads = kv_heads, a.N = N, a.P = P, a.write_state = write_state, a.q_scale = q_scale;
+  return rule == 0 ? memory_any<true>(a, B_, n_items, single != 0, stream) : memory_any<false>(a, B_, n_items, single != 0, stream);
 }
 
 // ------------------------------------------------------------------ ahead of the delta rule

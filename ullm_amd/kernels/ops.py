@@ -797,6 +797,7 @@ def gated_unit_norm(o: torch.Tensor, gate: torch.Tensor, gain: torch.Tensor, eps
 # ---------------------------------------------------------------------------------- matrix memories with a decay per token
 
 MEMORY_DELTA, MEMORY_SUM = 0, 1          # how a matrix memory takes a token in
+MEMORY_CHUNK, MEMORY_CHUNK_FLOATS = 16, 576     # tokens of a chunk, and what is made of one per head ahead of the recurrence
 MEMORY_MAX_KEYS = 512                    # key channels a head; a convolved head's value channels too
 
 
@@ -807,13 +808,15 @@ def _check_step(q_start, entry_slot, n_entries: int) -> None:
 
 def matrix_memory(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, keep: torch.Tensor, take: torch.Tensor, rule: int,
                   state: torch.Tensor, state_off: int, ctx, heads: int, kv_heads: int, key_dim: int, value_dim: int,
-                  q_scale: float = 1.0, norm_off: int = 0, write_state: bool = True):
+                  plan=None, q_scale: float = 1.0, norm_off: int = 0, write_state: bool = True):
     """A recurrence per head over each entry's tokens, with the head's memory S [key_dim, value_dim] (float32, at
     ``state[slot, state_off + head * key_dim * value_dim ..]``) and one decay ``keep`` and one strength ``take`` per token and
     head (float32 [T, heads], columns of wider rows).  MEMORY_DELTA: S <- keep S, u = take (v - S^T k), S <- S + k u^T.
     MEMORY_SUM: S <- keep S + k (take v)^T, and the same with v = 1 for the normaliser n [key_dim] at ``norm_off + head * key_dim``.
     ``q``, ``k`` (float32 [T, kv_heads * key_dim], head h takes kv head h // (heads // kv_heads)) and ``v`` (float32 [T, heads *
-    value_dim]) may be column ranges of wider rows; q is multiplied by ``q_scale``.  Returns (S^T q float32 [T, heads * value_dim],
+    value_dim]) may be column ranges of wider rows; q is multiplied by ``q_scale``.  ``plan``: a step with portions needs the list of
+    its chunks of up to MEMORY_CHUNK tokens (arrays ``items`` [n, 2] = (first token, tokens), an entry's side by side, and
+    ``entry_item`` [B]; number ``num_items``).  Returns (S^T q float32 [T, heads * value_dim],
     n . q float32 [T, heads] or None), both after the token's update."""
     T = q.shape[0]
     _need(heads % kv_heads == 0, f"{heads} heads are not a multiple of {kv_heads} key heads")
@@ -822,7 +825,7 @@ def matrix_memory(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, keep: torch
     _f32_rows(v, "v", T, heads * value_dim)
     _f32_rows(keep, "keep", T, heads)
     _f32_rows(take, "take", T, heads)
-    _need(keep.stride(0) == take.stride(0) and q.stride(0) == k.stride(0), "keep and take, and q and k, must be columns of rows equally far apart")
+    _need(keep.stride(0) == take.stride(0), "keep and take must be columns of rows equally far apart")
     _need(1 <= key_dim <= MEMORY_MAX_KEYS, f"{key_dim} key channels a head: at most {MEMORY_MAX_KEYS}")
     _check_step_state(state, state_off, heads * key_dim * value_dim, "the memories")
     if rule == MEMORY_SUM:
@@ -832,10 +835,19 @@ def matrix_memory(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, keep: torch
     ll = ctypes.c_longlong
     out = torch.empty((T, heads * value_dim), dtype=torch.float32, device=q.device)
     norm = torch.empty((T, heads), dtype=torch.float32, device=q.device) if rule == MEMORY_SUM else None
+    items = entry_item = chunks = None
+    n_items = 0
+    if not ctx.decode_only:
+        _need(plan is not None, "a step with portions needs the list of its chunks (a step plan)")
+        items, entry_item, n_items = plan.arrays["items"], plan.arrays["entry_item"], plan.facts["num_items"]
+        _i32(items, "items", 2 * n_items)
+        _i32(entry_item, "entry_item", ctx.num_entries)
+        chunks = torch.empty((n_items, heads, MEMORY_CHUNK_FLOATS), dtype=torch.float32, device=q.device)
     _check(build.load("matrix_memory").ullm_matrix_memory(
         _p(q), _c_int(q.stride(0)), _p(k), _c_int(k.stride(0)), _p(v), _c_int(v.stride(0)), _p(keep), _p(take), _c_int(keep.stride(0)),
         _c_int(rule), _c_float(q_scale), _p(state), ll(state.stride(0)), ll(state_off), ll(norm_off), _p(ctx.q_start),
-        _p(ctx.entry_slot), _p(out), _p(norm), _c_int(ctx.num_entries), _c_int(heads), _c_int(kv_heads), _c_int(key_dim),
+        _p(ctx.entry_slot), _p(items), _p(entry_item), _c_int(n_items), _p(chunks), _p(out), _p(norm), _c_int(ctx.num_entries),
+        _c_int(heads), _c_int(kv_heads), _c_int(key_dim),
         _c_int(value_dim), _c_int(1 if write_state else 0), _c_int(1 if ctx.decode_only else 0), _stream()), "matrix_memory")
     return out, norm
 

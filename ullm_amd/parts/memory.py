@@ -18,16 +18,32 @@ from __future__ import annotations
 
 from typing import Dict, List, Optional
 
+import numpy as np
 import torch
 
 from ..kernels import ops
-from .base import LayerCache, Mixer, PartEnv, StateNeed, StepContext, WeightDecl, register_part
+from .base import LayerCache, Mixer, PartEnv, StateNeed, StepContext, StepPlan, StepShape, WeightDecl, register_part
 from .linear import linear, linear_into_stream
+
+
+def plan_memory_chunks(shape: StepShape) -> StepPlan:
+    """The chunks of up to ``ops.MEMORY_CHUNK`` tokens every entry's tokens are cut into, (first token, tokens) each, an
+    entry's side by side, and every entry's first.  A step of single tokens lists none."""
+    items, entry_item, t0 = [], [], 0
+    if any(n != 1 for n in shape.lens):
+        for n in shape.lens:
+            entry_item.append(len(items) // 2)
+            for at in range(0, n, ops.MEMORY_CHUNK):
+                items.extend((t0 + at, min(ops.MEMORY_CHUNK, n - at)))
+            t0 += n
+    return StepPlan(arrays={"items": np.asarray(items, dtype=np.int32), "entry_item": np.asarray(entry_item, dtype=np.int32)},
+                    facts={"num_items": len(items) // 2})
 
 
 class _MemoryMixer(Mixer):
     """What the two have in common: sizes, names, one input matrix whose columns are padded to whole 64-byte pieces."""
     DEFAULT_NAMES: Dict[str, str] = {}
+    step_planners = {"memory chunks": plan_memory_chunks}
 
     def __init__(self, hidden_size: int, heads: int, kv_heads: int, key_dim: int, value_dim: int, norm_eps: float, prefix: str,
                  names: Optional[Dict[str, str]] = None):
@@ -119,7 +135,7 @@ class GatedDeltaRule(_MemoryMixer):
                                        self.dt_bias, rows, self.memory, ctx, self.heads, self.kv_heads, self.key_dim, self.value_dim,
                                        self.key_dim ** -0.5, write_state=cache.owner)
         o, _ = ops.matrix_memory(qkv[:, at["q"]], qkv[:, at["k"]], qkv[:, at["v"]], gates[:, 0], gates[:, 1], ops.MEMORY_DELTA, rows, 0,
-                                 ctx, self.heads, self.kv_heads, self.key_dim, self.value_dim, write_state=cache.owner)
+                                 ctx, self.heads, self.kv_heads, self.key_dim, self.value_dim, ctx.plans["memory chunks"], write_state=cache.owner)
         y = ops.gated_unit_norm(o, proj[:, at["g"]], self.gain, self.norm_eps, self.heads, ops.GATE_SILU, ctx.dtype)
         return linear_into_stream(y, self.w_o, ctx)
 
@@ -162,7 +178,7 @@ class ExpGatedMemory(_MemoryMixer):
         gates = ops.exp_gates(proj[:, at["i"]], proj[:, at["f"]], self.b_i, self.b_f, self.cap, rows, self.m_at, ctx,
                               write_state=cache.owner)
         o, norm = ops.matrix_memory(proj[:, at["q"]], proj[:, at["k"]], proj[:, at["v"]], gates[:, 0], gates[:, 1], ops.MEMORY_SUM, rows,
-                                    0, ctx, self.heads, self.heads, self.key_dim, self.value_dim, q_scale=self.key_dim ** -0.5,
+                                    0, ctx, self.heads, self.heads, self.key_dim, self.value_dim, ctx.plans["memory chunks"], q_scale=self.key_dim ** -0.5,
                                     norm_off=self.norm_at, write_state=cache.owner)
         y = ops.gated_unit_norm(o, proj[:, at["g"]], self.gain, self.norm_eps, self.heads, ops.GATE_SIGMOID, ctx.dtype, den=norm,
                                 least=gates[:, 2])
