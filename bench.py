@@ -238,7 +238,7 @@ def nadevik_config(shape):
 
 # Risolorn at a design shape: the same width, heads and depth.  Of every four layers one is a matrix memory with exponential
 # gates and two are the gated delta rule (heads of the head size, as many states as Kumudra's lightning layers have; the
-# other stacks' key heads, four taps), one attention (the other stacks' heads, chunks of 1024 positions, sinks, half of each
+# other stacks' key heads, four taps), one attention (the other stacks' heads, chunks of 2048 positions, sinks, half of each
 # head rotated, stretched).  Every feed-forward is routed, with as many columns a token as the dense stack's (top 4 of 32
 # experts of a sixth of it, in four groups of which three are kept).
 def risolorn_config(shape):
@@ -247,7 +247,7 @@ def risolorn_config(shape):
     delta = dict(type="delta", mlp=mlp, mixer=dict(heads=H, kv_heads=G, dim=D, vdim=D, conv=4))
     memory = dict(type="mlstm", mlp=mlp, mixer=dict(heads=H, dim=D, vdim=D, gate_cap=10.0))
     rot = dict(base=500000.0, dims=D // 2, scaling=dict(factor=8.0, original=4096, fast=32.0, slow=1.0))
-    att = dict(type="attention", mlp=mlp, mixer=dict(heads=H, kv_heads=G, dim=D, vdim=D, scale=D ** -0.5, mask=dict(size=1024), rot=rot))
+    att = dict(type="attention", mlp=mlp, mixer=dict(heads=H, kv_heads=G, dim=D, vdim=D, scale=D ** -0.5, mask=dict(size=2048), rot=rot))
     return dict(architecture="Risolorn", vocab=DESIGN_VOCAB, width=W, norm=dict(eps=1e-6), embedding=dict(scale=1.0), logit_scale=0.7,
                 layers=[(memory, delta, att, delta)[i % 4] for i in range(L)])
 
