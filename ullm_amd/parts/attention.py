@@ -141,6 +141,9 @@ class GQAttention(Mixer):
     def children(self):
         return [self.position] if self.position is not None else []
 
+    def kernel_families(self, dtype):
+        return ("attention_mfma",) if dtype == torch.bfloat16 else ("attention_generic",)
+
     def cache_need(self):
         return KVNeed(self.nkv, self.hd, self.window, chunk=self.chunk)
 
